@@ -18,6 +18,7 @@ class GroupGeometry:
     num_pages: int
     window: int = 0
     keep_first: int = 0     # with a window: the first positions that every query still sees; their pages are kept
+    chunked: bool = False   # with a window: it is the size of chunks counted from position 0, and a query sees its own
 
 
 class CacheError(RuntimeError):
@@ -74,7 +75,8 @@ class CacheManager:
         self._h = self._lib.mgpt_cache_create(n, arr([g.page_size for g in self.groups]),
                                               arr([g.num_pages for g in self.groups]),
                                               arr([g.window for g in self.groups]),
-                                              arr([g.keep_first for g in self.groups]), self.max_requests)
+                                              arr([g.keep_first for g in self.groups]),
+                                              arr([1 if g.chunked else 0 for g in self.groups]), self.max_requests)
         if not self._h:
             raise CacheError(library.host_error())
 

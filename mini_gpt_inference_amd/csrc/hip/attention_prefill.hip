@@ -7,7 +7,12 @@
 //
 // With `keep_first` > 0 a query behind a window also sees the keys at positions below keep_first (a tile walks
 // the stretches of those keys first, then the window's); with `score_bias` a visible key's weight is
-// sigmoid(score + score_bias[head]) and nothing is normalised.
+// sigmoid(score + score_bias[head]) and nothing is normalised.  With `chunked` a query sees its own chunk of
+// `window` positions instead of the last `window`.
+//
+// With a table of numbers by distance (BIAS; in the scores' units before log2 e) the numbers that a step's
+// stretch of keys needs for the tile's 64 queries, one per distance, lie in LDS in the order of the key, so that a
+// lane's four neighbouring keys read four neighbouring numbers.
 //
 // A workgroup takes 64 consecutive queries of one request and one head, 16 per wave (four waves,
 // or eight in two groups that share the keys between them, see the kernel).  It walks the keys in blocks of 128 (aligned to multiples of 128 of the key position):
@@ -26,6 +31,7 @@
 // costs: exp2(score * scale' - max) is one fused multiply-add and one v_exp_f32 (scale' holds
 // log2 e), the maximum over the four lanes that share a query goes through two lane swaps
 // instead of LDS, and the row sum stays split over those lanes until the end.
+#include "attention_mask.h"
 #include "common.h"
 #include "launchers.h"
 
@@ -63,14 +69,15 @@ __device__ __forceinline__ float pf_sum_over_rows(float v) {
 // thread stages as much per step as with one group, and on each SIMD a wave of one group has its
 // softmax arithmetic while the other group's wave has its MFMAs.  Head sizes whose two stretches
 // do not fit LDS run with one group.
-template <int D, int G>
+template <int D, int G, bool BIAS>
 __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     const bf16_t* __restrict__ q, long ldq, bf16_t* __restrict__ out, long ldo,
     const bf16_t* __restrict__ kpool, const bf16_t* __restrict__ vpool,
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ seq_lens, int n_head, int n_kv_head, int page_size, float scale, int window,
     int single_below, const float* __restrict__ sinks, float softcap, const bf16_t* __restrict__ gate, long ldg,
-    int keep_first, const float* __restrict__ score_bias) {
+    int keep_first, const float* __restrict__ score_bias, int chunked, const float* __restrict__ dist_bias,
+    int bias_len) {
   constexpr int THREADS = 256 * G;
   constexpr int SB = PF_KT * G;    // keys staged per step
   // Key and value rows in LDS: as long as the head size where that is a power of two, the 16-byte
@@ -86,6 +93,9 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
   // offset; -1: not a key this tile sees), worked out three steps ahead by one thread per key: the
   // loads that fetch a stretch then wait for no block-table entry and divide nothing.
   int* const row_tab = reinterpret_cast<int*>(pf_lds + 4 * KS_SIZE);   // [4][SB]
+  // entry e of a buffer: the number (times log2 e) for distance tile_pos_hi - first key of the stretch - e
+  constexpr int NB = SB + PF_QT;
+  float* const bias_tab = reinterpret_cast<float*>(row_tab + 4 * SB);  // [2][NB]
 
   const int r = blockIdx.y, h = blockIdx.z;
   const int q_start = cu_q[r], q_len = cu_q[r + 1] - q_start;
@@ -106,7 +116,8 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
   const int my_pos = ctx + my_q;
   const int tile_q_hi = (q0 + PF_QT < q_len ? q0 + PF_QT : q_len) - 1;
   const int pos_lo = ctx + q0, pos_hi = ctx + tile_q_hi;
-  const int kv_begin = (window > 0 && pos_lo - window + 1 > 0) ? pos_lo - window + 1 : 0;
+  const int kv_begin = first_seen(pos_lo, window, chunked);
+  const int my_begin = first_seen(my_pos, window, chunked);
   const int kv_end = pos_hi + 1;
 
   bf16x8_t qf[KK];
@@ -167,20 +178,30 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     }
   };
 
-  // scores are kept in units of log2(e), so that the exponential is one v_exp_f32 (scale > 0 here)
-  const float sc2 = scale * 1.4426950408889634f;
+  // scores are kept in units of log2(e), so that the exponential is one v_exp_f32 (scale > 0 here; with numbers
+  // by distance the scores are scaled when those are added)
+  const float raw2 = scale * 1.4426950408889634f;
+  const float sc2 = BIAS ? 1.0f : raw2;
   const bool weigh = score_bias != nullptr;   // sigmoid weights, no softmax
   const float bias2 = weigh ? score_bias[h] * 1.4426950408889634f : 0.f;
   const int c_first = (kv_begin / SB) * SB;
   // the stretches of the kept first keys (those before the window's first stretch), then the window's
   const int kept_steps = keep_first > 0 ? ((keep_first + SB - 1) / SB < c_first / SB ? (keep_first + SB - 1) / SB : c_first / SB) : 0;
   const int n_steps = kept_steps + (kv_end - c_first + SB - 1) / SB;
+  const int wave_begin_hi = first_seen(ctx + q0 + qwave * 16 + 15, window, chunked);   // what the wave's last query sees from
   auto stretch_start = [&](int step) -> int { return step < kept_steps ? step * SB : c_first + (step - kept_steps) * SB; };
+  auto fill_bias = [&](int step) {
+    const int c_start = stretch_start(step);
+    for (int e = tid; e < NB; e += THREADS)
+      bias_tab[(step & 1) * NB + e] =
+          dist_bias[(long)h * bias_len + distance_entry(pos_lo + PF_QT - 1 - c_start - e, bias_len)] * 1.4426950408889634f;
+  };
   // the rows of the first three stretches
   for (int t = tid; t < 3 * SB; t += THREADS) row_tab[t] = lookup(stretch_start(t / SB) + t % SB);
   __syncthreads();
   fetch(0);
   deposit(0);
+  if (BIAS) fill_bias(0);
   if (n_steps > 1) fetch(1);
   __syncthreads();
   for (int b = 0; b < n_steps; ++b) {
@@ -189,6 +210,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     int row_ahead = -1;
     if (b + 1 < n_steps) {
       deposit(buf ^ 1);   // its readers finished before the last barrier
+      if (BIAS) fill_bias(b + 1);
       if (b + 2 < n_steps) fetch(b + 2);
       // asked for now, written to the table at the end of this step's work
       if (b + 3 < n_steps && tid < SB) row_ahead = lookup(stretch_start(b + 3) + tid);
@@ -216,6 +238,13 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
 #pragma unroll
           for (int kt = 0; kt < NKT; ++kt)
             s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[kk][kt], qf[kk], s[kt], 0, 0, 0);
+      }
+      if (BIAS) {
+        const float* mine = bias_tab + buf * NB + grp * PF_KT + (PF_QT - 1 - (qwave * 16 + qi)) + g * 4;
+#pragma unroll
+        for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) s[kt][i] = __builtin_fmaf(s[kt][i], raw2, mine[kt * 16 + i]);
       }
       if (softcap > 0.f) {
         // capped scores: cap * tanh(s * scale / cap), kept in the raw scores' units (times cap / scale)
@@ -246,8 +275,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
       // lane: query qi, keys c0 + kt*16 + g*4 + i.  A half that every query of this wave sees whole
       // (the common case away from the diagonal) needs no mask.
       const int wave_pos_lo = ctx + q0 + qwave * 16;   // first query position of this wave
-      const bool whole = c0 + PF_KT - 1 <= wave_pos_lo && c0 >= kv_begin && wave_pos_lo + 15 < ctx + q_len &&
-                         (window <= 0 || c0 > wave_pos_lo + 15 - window);
+      const bool whole = c0 + PF_KT - 1 <= wave_pos_lo && wave_pos_lo + 15 < ctx + q_len && c0 >= wave_begin_hi;
       float mx = -INFINITY;
       if (whole) {
 #pragma unroll
@@ -260,7 +288,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int key = c0 + kt * 16 + g * 4 + i;
-            const bool see = q_ok && key <= my_pos && (window <= 0 || key > my_pos - window || key < keep_first);
+            const bool see = q_ok && key <= my_pos && (key >= my_begin || key < keep_first);
             const float v = see ? s[kt][i] : -INFINITY;
             s[kt][i] = v;
             mx = fmaxf(mx, v);
@@ -373,32 +401,38 @@ extern "C" int mgpt_prefill_attention_bf16(
     const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, int n_req,
     int max_q_len, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     int single_below, const float* sinks, float softcap, const void* gate, long ldg, int keep_first,
-    const float* score_bias, hipStream_t stream) {
+    const float* score_bias, int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
   if (n_req == 0 || max_q_len == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !cu_q || !seq_lens) return MGPT_ERR_NULL;
   if (n_req < 0 || max_q_len < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 ||
       page_size <= 0 || max_blocks <= 0 || window < 0 || (ldq % 8) != 0 || (ldo % 4) != 0 ||
-      (((size_t)out) & 7) != 0 || !(scale > 0.f) || keep_first < 0 || (score_bias && (sinks || softcap > 0.f)))
+      (((size_t)out) & 7) != 0 || !(scale > 0.f) || keep_first < 0 || (score_bias && (sinks || softcap > 0.f)) ||
+      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
     return MGPT_ERR_BAD_SHAPE;
   if (window == 0) keep_first = 0;
   if (n_req > 65535 || n_head > 65535) return MGPT_ERR_TOO_LARGE;
   dim3 grid((max_q_len + PF_QT - 1) / PF_QT, n_req, n_head);
-#define PF_LAUNCH(DD, GG)                                                                                       \
-  {                                                                                                             \
-    constexpr int sb = PF_KT * GG;                                                                              \
-    constexpr int kld = (DD & (DD - 1)) == 0 ? DD : DD + 8;                                                     \
-    constexpr int lds_bytes = 4 * sb * kld * (int)sizeof(bf16_t) + 4 * sb * 4;                                  \
-    static bool allowed = false; /* more LDS than a kernel gets without asking */                               \
-    if (!allowed) {                                                                                             \
-      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prefill_attention_kernel<DD, GG>), \
-                                               hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);         \
-      if (e != hipSuccess) return (int)e;                                                                       \
-      allowed = true;                                                                                           \
-    }                                                                                                           \
-    hipLaunchKernelGGL((prefill_attention_kernel<DD, GG>), grid, dim3(256 * GG), lds_bytes, stream,             \
-                       (const bf16_t*)q, ldq, (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool,    \
-                       block_tables, max_blocks, cu_q, seq_lens, n_head, n_kv_head, page_size, scale, window,   \
-                       single_below, sinks, softcap, (const bf16_t*)gate, ldg, keep_first, score_bias);                                                                          \
+#define PF_LAUNCH2(DD, GG, BI)                                                                                      \
+  {                                                                                                                 \
+    constexpr int sb = PF_KT * GG;                                                                                  \
+    constexpr int kld = (DD & (DD - 1)) == 0 ? DD : DD + 8;                                                         \
+    constexpr int lds_bytes = 4 * sb * kld * (int)sizeof(bf16_t) + 4 * sb * 4 + (BI ? 2 * (sb + PF_QT) * 4 : 0);    \
+    static bool allowed = false; /* more LDS than a kernel gets without asking */                                   \
+    if (!allowed) {                                                                                                 \
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prefill_attention_kernel<DD, GG, BI>), \
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);             \
+      if (e != hipSuccess) return (int)e;                                                                           \
+      allowed = true;                                                                                               \
+    }                                                                                                               \
+    hipLaunchKernelGGL((prefill_attention_kernel<DD, GG, BI>), grid, dim3(256 * GG), lds_bytes, stream,             \
+                       (const bf16_t*)q, ldq, (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool,        \
+                       block_tables, max_blocks, cu_q, seq_lens, n_head, n_kv_head, page_size, scale, window,       \
+                       single_below, sinks, softcap, (const bf16_t*)gate, ldg, keep_first, score_bias, chunked,     \
+                       dist_bias, bias_len);                                                                        \
+  }
+#define PF_LAUNCH(DD, GG)                                               \
+  {                                                                     \
+    if (dist_bias) PF_LAUNCH2(DD, GG, true) else PF_LAUNCH2(DD, GG, false) \
   }
   // Two wave groups halve the walk of a tile over its keys; one group leaves LDS for a second
   // workgroup on the compute unit.  The first serves a step with few tiles, the second one with many.
@@ -412,5 +446,6 @@ extern "C" int mgpt_prefill_attention_bf16(
     default: return MGPT_ERR_BAD_SHAPE;
   }
 #undef PF_LAUNCH
+#undef PF_LAUNCH2
   return mgpt_last_error();
 }

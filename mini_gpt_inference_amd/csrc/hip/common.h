@@ -89,6 +89,11 @@ __device__ __forceinline__ int wave_sum_int(int v) {
          (__builtin_amdgcn_readlane(v, 32) + __builtin_amdgcn_readlane(v, 48));
 }
 
+__device__ __forceinline__ float relu_squared(float v) {
+  const float r = fmaxf(v, 0.f);
+  return r * r;
+}
+
 // GELU with the tanh approximation, as F.gelu(approximate="tanh"):
 // 0.5*u*(1 + tanh(sqrt(2/pi)*(u + 0.044715*u^3)))
 __device__ __forceinline__ float gelu_tanh(float u) {

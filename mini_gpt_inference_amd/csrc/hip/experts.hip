@@ -17,6 +17,8 @@
 #define EX_TILE 16
 #define EX_BK 64
 #define EX_MAX_EXPERTS 1024
+#define EX_EPI_NONE 0
+#define EX_EPI_RELU2 5   // max(v, 0)^2
 
 template <typename T, bool FAST>
 __global__ void gated_unit_kernel(const T* __restrict__ z, long ldz, T* __restrict__ act, long lda, long total,
@@ -128,8 +130,14 @@ extern "C" int mgpt_gather_rows(const void* src, long ld, const int* slot_token,
 // A router: scores of every expert for a token, in float32 whatever the rows' dtype, and the `top`
 // largest.  logit[e] = w[e] . h; score = sigmoid(logit) (kind 0) or the logit itself (kind 1);
 // chosen[n][c] is the expert with the c-th largest score (of equal scores the lower number first) and
-// weight[n][c] its score.  One workgroup a token: its threads along the width in a fixed order, then the first
-// wave picks the largest `top` times.
+// weight[n][c] its score.  Optional steps:
+//  - `correction` (a number per expert) is added to the scores that the choice goes by, not to the weights;
+//  - with n_groups > keep > 0 the experts form n_groups equal groups of neighbours, a group's rank is the sum of
+//    its two largest choice scores, and only experts of the `keep` best groups can be chosen;
+//  - `normalise`: the chosen scores are divided by (their sum + 1e-20); every weight is multiplied by `scale`;
+//  - `extra` (one more row beside the matrix): extra_out[n] = sigmoid(extra . h).
+// One workgroup a token: its threads along the width in a fixed order, then the first wave picks the largest
+// `top` times.
 __device__ __forceinline__ float router_value(float v) { return v; }
 __device__ __forceinline__ float router_value(bf16_t v) { return bf16_to_float(v); }
 
@@ -154,23 +162,29 @@ __device__ __forceinline__ void router_load8(const bf16_t* p, float (&v)[8]) {
 template <typename HT, typename WT, bool VEC>
 __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__ h, long ldh, const WT* __restrict__ w,
                                                           const int* __restrict__ q_req, int width, int n_experts, int top,
-                                                          int kind, int* __restrict__ chosen, float* __restrict__ weight) {
-  __shared__ float logit[EX_MAX_EXPERTS];
+                                                          int kind, int* __restrict__ chosen, float* __restrict__ weight,
+                                                          const float* __restrict__ correction, int n_groups, int keep,
+                                                          int normalise, float scale, const WT* __restrict__ extra,
+                                                          float* __restrict__ extra_out) {
+  __shared__ float logit[EX_MAX_EXPERTS + 1];    // the extra row's comes last
+  __shared__ float key[EX_MAX_EXPERTS];          // what the choice goes by
+  __shared__ float rank[EX_MAX_EXPERTS];         // of a group
   __shared__ float part[4][8];
+  const int n_rows_w = n_experts + (extra ? 1 : 0);
   const int n = blockIdx.x;
   if (q_req && q_req[n] < 0) return;     // padded token
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (VEC) {
-    for (int e0 = 0; e0 < n_experts; e0 += 8) {
+    for (int e0 = 0; e0 < n_rows_w; e0 += 8) {
       float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
       for (int c = 8 * threadIdx.x; c < width; c += 8 * 256) {
         float hv[8];
         router_load8(h + (long)n * ldh + c, hv);
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
-          const int e = e0 + j < n_experts ? e0 + j : n_experts - 1;     // (behind the last expert: loaded again, not used)
+          const int e = e0 + j < n_experts ? e0 + j : n_experts - 1;     // (behind the last row: loaded again, not used)
           float wv[8];
-          router_load8(w + (long)e * width + c, wv);
+          router_load8((extra && e0 + j >= n_experts ? extra : w + (long)e * width) + c, wv);
 #pragma unroll
           for (int k = 0; k < 8; ++k) acc[j] = fmaf(wv[k], hv[k], acc[j]);
         }
@@ -181,26 +195,57 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
         if (lane == 0) part[wave][j] = sum;
       }
       __syncthreads();
-      if (threadIdx.x < 8 && e0 + threadIdx.x < n_experts)
+      if (threadIdx.x < 8 && e0 + threadIdx.x < n_rows_w)
         logit[e0 + threadIdx.x] = (part[0][threadIdx.x] + part[1][threadIdx.x]) + (part[2][threadIdx.x] + part[3][threadIdx.x]);
       __syncthreads();
     }
   } else {
-    for (int e = wave; e < n_experts; e += 4) {
+    for (int e = wave; e < n_rows_w; e += 4) {
+      const WT* we = e < n_experts ? w + (long)e * width : extra;
       float acc = 0.f;
       for (int c = lane; c < width; c += 64)
-        acc = fmaf(router_value(w[(long)e * width + c]), router_value(h[(long)n * ldh + c]), acc);
+        acc = fmaf(router_value(we[c]), router_value(h[(long)n * ldh + c]), acc);
       acc = wave_sum(acc);
       if (lane == 0) logit[e] = acc;
     }
     __syncthreads();
   }
+  if (extra && threadIdx.x == 0) extra_out[n] = 1.0f / (1.0f + expf(-logit[n_experts]));
+  // (without a correction and groups the choice goes by the logits, in whose order the scores come)
+  const bool grouped = n_groups > keep && keep > 0;
+  for (int e = threadIdx.x; e < n_experts; e += 256) {
+    const float z = logit[e];
+    key[e] = (correction || grouped) ? (kind == 0 ? 1.0f / (1.0f + expf(-z)) : z) + (correction ? correction[e] : 0.f) : z;
+  }
+  __syncthreads();
+  if (grouped) {
+    const int size = n_experts / n_groups;
+    for (int g = threadIdx.x; g < n_groups; g += 256) {
+      float a = -INFINITY, b = -INFINITY;     // the two largest
+      for (int i = 0; i < size; ++i) {
+        const float v = key[g * size + i];
+        if (v > a) { b = a; a = v; }
+        else if (v > b) b = v;
+      }
+      rank[g] = size > 1 ? a + b : a;
+    }
+    __syncthreads();
+    // a group stays if fewer than `keep` groups come before it (of equal ranks the lower number first)
+    for (int e = threadIdx.x; e < n_experts; e += 256) {
+      const int mine = e / size;
+      int before = 0;
+      for (int g = 0; g < n_groups; ++g) before += rank[g] > rank[mine] || (rank[g] == rank[mine] && g < mine);
+      if (before >= keep) key[e] = -INFINITY;
+    }
+    __syncthreads();
+  }
   if (wave != 0) return;
+  float sum = 0.f;
   for (int c = 0; c < top; ++c) {
     float best = -INFINITY;
     int at = 0x7fffffff;
     for (int e = lane; e < n_experts; e += 64) {
-      const float v = logit[e];
+      const float v = key[e];
       if (v > best) { best = v; at = e; }      // a lane's experts rise, so the lower number stays at a tie
     }
     const float all = wave_max(best);
@@ -211,35 +256,49 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
       cand = other < cand ? other : cand;
     }
     if (cand == 0x7fffffff) cand = 0;          // every score is -inf or NaN
+    const float score = kind == 0 ? 1.0f / (1.0f + expf(-logit[cand])) : logit[cand];
+    sum += score;                                         // (the same in every lane)
     if (lane == 0) {
       chosen[(long)n * top + c] = cand;
-      weight[(long)n * top + c] = kind == 0 ? 1.0f / (1.0f + expf(-all)) : all;
+      weight[(long)n * top + c] = score * scale;
+      rank[c] = score;                                    // (the groups' ranks are done with)
     }
-    if ((cand & 63) == lane) logit[cand] = -INFINITY;     // the lane that reads this expert takes it out
+    if ((cand & 63) == lane) key[cand] = -INFINITY;       // the lane that reads this expert takes it out
   }
+  if (!normalise) return;
+  __builtin_amdgcn_wave_barrier();
+  const float by = scale / (sum + 1e-20f);
+  if (lane == 0)
+    for (int c = 0; c < top; ++c) weight[(long)n * top + c] = rank[c] * by;
 }
 
 // h: [n_rows, ldh] rows in `dtype`; w: dense [n_experts, width] in w_dtype; chosen: int32 [n_rows, top]; weight:
-// float32 [n_rows, top].
+// float32 [n_rows, top].  correction: float32 [n_experts] or null; n_groups, keep: 0 or 1, 1 for no groups;
+// extra: [width] in w_dtype or null; extra_out: float32 [n_rows].
 extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
                                 int width, int n_experts, int top, int kind, int* chosen, float* weight,
-                                hipStream_t stream) {
+                                const float* correction, int n_groups, int keep, int normalise, float scale,
+                                const void* extra, float* extra_out, hipStream_t stream) {
   if (n_rows == 0) return MGPT_OK;
   if (!h || !w || !chosen || !weight) return MGPT_ERR_NULL;
   if (!dtype_ok(dtype) || !dtype_ok(w_dtype)) return MGPT_ERR_BAD_DTYPE;
   if (n_rows < 0 || width <= 0 || n_experts <= 0 || n_experts > EX_MAX_EXPERTS || top <= 0 || top > n_experts ||
-      (kind != 0 && kind != 1))
+      (kind != 0 && kind != 1) || n_groups < 0 || keep < 0)
     return MGPT_ERR_BAD_SHAPE;
+  if (n_groups > keep && keep > 0 && (n_experts % n_groups || top > keep * (n_experts / n_groups))) return MGPT_ERR_BAD_SHAPE;
+  if (extra && !extra_out) return MGPT_ERR_NULL;
   const size_t h_size = dtype == MGPT_F32 ? 4 : 2, w_size = w_dtype == MGPT_F32 ? 4 : 2;
-  const bool vec = !(width & 7) && !(((size_t)h | (size_t)(ldh * h_size)) & 15) && !((size_t)w & 15);
+  const bool vec = !(width & 7) && !(((size_t)h | (size_t)(ldh * h_size)) & 15) && !(((size_t)w | (size_t)extra) & 15);
 #define ROUTER_LAUNCH(HT, WT)                                                                                            \
   {                                                                                                                      \
     if (vec)                                                                                                             \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, true>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,      \
-                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight);                              \
+                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
+                         normalise, scale, (const WT*)extra, extra_out);                                                 \
     else                                                                                                                 \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, false>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,     \
-                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight);                              \
+                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
+                         normalise, scale, (const WT*)extra, extra_out);                                                 \
   }
   if (dtype == MGPT_F32 && w_dtype == MGPT_F32) ROUTER_LAUNCH(float, float)
   else if (dtype == MGPT_F32) ROUTER_LAUNCH(float, bf16_t)
@@ -373,7 +432,7 @@ template <typename T, typename OT>
 __global__ __launch_bounds__(256) void grouped_linear_kernel(
     const T* __restrict__ A, long lda, const int* __restrict__ a_rows, const T* __restrict__ W, long w_stride,
     const int* __restrict__ tile_expert, const int* __restrict__ slot_token, OT* __restrict__ out, long ldo,
-    const int* __restrict__ out_rows, int n_out, int k_dim, int blocks_per_tile) {
+    const int* __restrict__ out_rows, int n_out, int k_dim, int blocks_per_tile, int epilogue) {
   __shared__ float As[EX_TILE][EX_BK + 1];
   __shared__ float Ws[EX_TILE][EX_BK + 1];
   const int tile = blockIdx.y;                    // 16 slots; blocks_per_tile of them share an expert
@@ -404,16 +463,18 @@ __global__ __launch_bounds__(256) void grouped_linear_kernel(
   const int col = col0 + c;
   if (!a_ok || col >= n_out) return;
   const long orow = out_rows ? out_rows[slot] : slot;
-  out[orow * ldo + col] = from_float<OT>(acc);
+  out[orow * ldo + col] = from_float<OT>(epilogue == EX_EPI_RELU2 ? relu_squared(acc) : acc);
 }
 
 // out[out_rows[s] or s] = A[a_rows[s] or s] @ W[tile_expert[s / tile_rows]]^T for every slot s with
-// slot_token[s] >= 0.  W: [experts][n_out][k_dim], w_stride elements from one expert to the next.
+// slot_token[s] >= 0, with the squared relu behind it where the epilogue says so.  W: [experts][n_out][k_dim],
+// w_stride elements from one expert to the next.
 extern "C" int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, const void* w, long w_stride,
                                    const int* tile_expert, const int* slot_token, void* out, int out_dtype,
                                    long ldo, const int* out_rows, int n_tiles, int tile_rows, int n_out, int k_dim,
-                                   int dtype, hipStream_t stream) {
+                                   int dtype, int epilogue, hipStream_t stream) {
   if (n_tiles == 0 || n_out == 0) return MGPT_OK;
+  if (epilogue != EX_EPI_NONE && epilogue != EX_EPI_RELU2) return MGPT_ERR_BAD_SHAPE;
   if (!a || !w || !tile_expert || !slot_token || !out) return MGPT_ERR_NULL;
   if (n_tiles < 0 || n_out < 0 || k_dim <= 0 || lda < k_dim || ldo < n_out || (tile_rows != 16 && tile_rows != 64 && tile_rows != 256))
     return MGPT_ERR_BAD_SHAPE;
@@ -423,7 +484,7 @@ extern "C" int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, c
 #define GL_LAUNCH(T, OT)                                                                                     \
   hipLaunchKernelGGL((grouped_linear_kernel<T, OT>), grid, block, 0, stream, (const T*)a, lda, a_rows,       \
                      (const T*)w, w_stride, tile_expert, slot_token, (OT*)out, ldo, out_rows, n_out, k_dim,         \
-                     blocks_per_tile)
+                     blocks_per_tile, epilogue)
   if (dtype == MGPT_F32 && out_dtype == MGPT_F32) GL_LAUNCH(float, float);
   else if (dtype == MGPT_BF16 && out_dtype == MGPT_BF16) GL_LAUNCH(bf16_t, bf16_t);
   else if (dtype == MGPT_BF16 && out_dtype == MGPT_F32) GL_LAUNCH(bf16_t, float);
@@ -443,7 +504,7 @@ template <typename OT, int NJ, int NT>     // NT: slices of 16 slots a tile
 __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(
     const bf16_t* __restrict__ A, long lda, const int* __restrict__ a_rows, const bf16_t* __restrict__ W,
     long w_stride, const int* __restrict__ tile_expert, const int* __restrict__ slot_token, OT* __restrict__ out,
-    long ldo, const int* __restrict__ out_rows, int n_out, int k_dim) {
+    long ldo, const int* __restrict__ out_rows, int n_out, int k_dim, int epilogue) {
   // a wave owns NT * 16 slots x NJ * 16 columns: per 32 k it loads NJ slices of the matrix and NT of the
   // rows for NT * NJ MFMAs
   const int tile = blockIdx.y;
@@ -500,6 +561,10 @@ __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(
     for (int t = 0; t < NT; ++t) {
       if (!a_ok[t]) continue;
       OT* dst = out + orow[t] * ldo + c;
+      if (epilogue == EX_EPI_RELU2) {
+#pragma unroll
+        for (int v = 0; v < 4; ++v) acc[j][t][v] = relu_squared(acc[j][t][v]);
+      }
       if (sizeof(OT) == 4) {
         *reinterpret_cast<float4*>(dst) = make_float4(acc[j][t][0], acc[j][t][1], acc[j][t][2], acc[j][t][3]);
       } else {
@@ -518,8 +583,9 @@ __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(
 extern "C" int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_rows, const void* w, long w_stride,
                                         const int* tile_expert, const int* slot_token, void* out, int out_dtype,
                                         long ldo, const int* out_rows, int n_tiles, int tile_rows, int n_out, int k_dim,
-                                        hipStream_t stream) {
+                                        int epilogue, hipStream_t stream) {
   if (n_tiles == 0 || n_out == 0) return MGPT_OK;
+  if (epilogue != EX_EPI_NONE && epilogue != EX_EPI_RELU2) return MGPT_ERR_BAD_SHAPE;
   if (!a || !w || !tile_expert || !slot_token || !out) return MGPT_ERR_NULL;
   if (n_tiles < 0 || n_out < 0 || k_dim <= 0 || lda < k_dim || ldo < n_out || (tile_rows != 16 && tile_rows != 64))
     return MGPT_ERR_BAD_SHAPE;
@@ -535,7 +601,7 @@ extern "C" int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_ro
 #define GM_LAUNCH(OT, NJ, NT)                                                                                 \
   hipLaunchKernelGGL((grouped_linear_mfma_kernel<OT, NJ, NT>), grid, block, 0, stream, (const bf16_t*)a, lda, \
                      a_rows, (const bf16_t*)w, w_stride, tile_expert, slot_token, (OT*)out, ldo, out_rows,    \
-                     n_out, k_dim)
+                     n_out, k_dim, epilogue)
   if (out_dtype == MGPT_F32) {
     if (tile_rows == 16) GM_LAUNCH(float, 1, 1); else if (wide) GM_LAUNCH(float, 4, 4); else GM_LAUNCH(float, 1, 4);
   } else if (out_dtype == MGPT_BF16) {
@@ -549,7 +615,8 @@ extern "C" int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_ro
 
 __global__ void expert_combine_kernel(const float* __restrict__ pair_out, const int* __restrict__ pair_slot,
                                       const int* __restrict__ q_req, float* __restrict__ y, long total, int width,
-                                      int top, float weight) {
+                                      int top, float weight, const float* __restrict__ pair_weight,
+                                      const float* __restrict__ extra, const float* __restrict__ extra_gate) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long n = i / width;
@@ -558,15 +625,18 @@ __global__ void expert_combine_kernel(const float* __restrict__ pair_out, const 
   float acc = 0.f;
   for (int k = 0; k < top; ++k) {
     const long row = pair_slot ? pair_slot[n * top + k] : n * top + k;
-    acc += pair_out[row * (long)width + c];
+    acc = fmaf(pair_weight ? pair_weight[n * top + k] : 1.0f, pair_out[row * (long)width + c], acc);
   }
-  y[i] += acc * weight;
+  acc *= weight;
+  if (extra) acc = fmaf(extra_gate ? extra_gate[n] : 1.0f, extra[i], acc);
+  y[i] += acc;
 }
 
 // the same, four columns a thread (widths in steps of 4, 16-byte aligned buffers)
 __global__ void expert_combine4_kernel(const float4* __restrict__ pair_out, const int* __restrict__ pair_slot,
                                        const int* __restrict__ q_req, float4* __restrict__ y, long total, int width4,
-                                       int top, float weight) {
+                                       int top, float weight, const float* __restrict__ pair_weight,
+                                       const float4* __restrict__ extra, const float* __restrict__ extra_gate) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long n = i / width4;
@@ -576,28 +646,38 @@ __global__ void expert_combine4_kernel(const float4* __restrict__ pair_out, cons
   for (int k = 0; k < top; ++k) {
     const long row = pair_slot ? pair_slot[n * top + k] : n * top + k;
     const float4 v = pair_out[row * (long)width4 + c];
-    acc.x += v.x; acc.y += v.y; acc.z += v.z; acc.w += v.w;
+    const float w = pair_weight ? pair_weight[n * top + k] : 1.0f;
+    acc.x = fmaf(w, v.x, acc.x); acc.y = fmaf(w, v.y, acc.y); acc.z = fmaf(w, v.z, acc.z); acc.w = fmaf(w, v.w, acc.w);
+  }
+  acc.x *= weight; acc.y *= weight; acc.z *= weight; acc.w *= weight;
+  if (extra) {
+    const float4 v = extra[i];
+    const float g = extra_gate ? extra_gate[n] : 1.0f;
+    acc.x = fmaf(g, v.x, acc.x); acc.y = fmaf(g, v.y, acc.y); acc.z = fmaf(g, v.z, acc.z); acc.w = fmaf(g, v.w, acc.w);
   }
   float4 o = y[i];
-  o.x += acc.x * weight; o.y += acc.y * weight; o.z += acc.z * weight; o.w += acc.w * weight;
+  o.x += acc.x; o.y += acc.y; o.z += acc.z; o.w += acc.w;
   y[i] = o;
 }
 
-// y[n] += weight * sum_k pair_out[pair_slot[n * top + k]] (pair_slot null: row n * top + k itself)
+// y[n] += weight * sum_k pair_weight[n * top + k] pair_out[pair_slot[n * top + k]] (pair_slot null: row n * top + k
+// itself; pair_weight null: 1) + extra_gate[n] * extra[n] (extra null: nothing; extra_gate null: 1)
 extern "C" int mgpt_expert_combine(const float* pair_out, const int* pair_slot, const int* q_req, float* y, int n_rows,
-                                   int width, int top, float weight, hipStream_t stream) {
+                                   int width, int top, float weight, const float* pair_weight, const float* extra,
+                                   const float* extra_gate, hipStream_t stream) {
   if (n_rows == 0) return MGPT_OK;
   if (!pair_out || !y) return MGPT_ERR_NULL;
   if (n_rows < 0 || width <= 0 || top <= 0) return MGPT_ERR_BAD_SHAPE;
-  const bool vec = (width & 3) == 0 && ((((size_t)pair_out) | ((size_t)y)) & 15) == 0;
+  const bool vec = (width & 3) == 0 && ((((size_t)pair_out) | ((size_t)y) | ((size_t)extra)) & 15) == 0;
   const long total = (long)n_rows * (vec ? width / 4 : width);
   const long blocks = (total + 255) / 256;
   if (blocks > 0x7fffffffL) return MGPT_ERR_TOO_LARGE;
   if (vec)
     hipLaunchKernelGGL(expert_combine4_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, (const float4*)pair_out,
-                       pair_slot, q_req, (float4*)y, total, width / 4, top, weight);
+                       pair_slot, q_req, (float4*)y, total, width / 4, top, weight, pair_weight, (const float4*)extra,
+                       extra_gate);
   else
     hipLaunchKernelGGL(expert_combine_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, pair_out, pair_slot, q_req, y,
-                       total, width, top, weight);
+                       total, width, top, weight, pair_weight, extra, extra_gate);
   return mgpt_last_error();
 }

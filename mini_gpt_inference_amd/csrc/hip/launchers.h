@@ -10,20 +10,21 @@ extern "C" {
 int mgpt_paged_attention_split_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool, const
     void* vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int*
     q_req, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
-    const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias,
-    hipStream_t stream);
+    const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias, int chunked,
+    const float* dist_bias, int bias_len, hipStream_t stream);
 // attention_decode.hip
 int mgpt_paged_attention_split_fast_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool,
     const void* vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const
     int* q_req, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
-    const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias,
-    hipStream_t stream);
+    const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias, int chunked,
+    const float* dist_bias, int bias_len, hipStream_t stream);
 // attention_decode_wide.hip
 int mgpt_paged_attention_decode_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool, const
     void* vpool, const int* block_tables, int max_blocks, const int* positions, const int* q_req, const int*
     cu_q, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, int num_pages, float scale,
     int window, int identity, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const
-    float* score_bias, hipStream_t stream);
+    float* score_bias, int chunked,
+    const float* dist_bias, int bias_len, hipStream_t stream);
 // attention_generic.hip
 int mgpt_kv_write(const void* qkv, int dtype, long ld, int k_off, int v_off, void* kpool, void* vpool, const
     int* slot_mapping, int n_tokens, int n_kv_head, int head_dim, int page_size, hipStream_t stream);
@@ -32,13 +33,15 @@ int mgpt_paged_attention_generic(const void* q, long ldq, void* out, long ldo, c
     vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int* q_req,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window, int dtype,
     int fast_exp, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float*
-    score_bias, hipStream_t stream);
+    score_bias, int chunked,
+    const float* dist_bias, int bias_len, hipStream_t stream);
 // attention_prefill.hip
 int mgpt_prefill_attention_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool, const void*
     vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, int n_req, int
     max_q_len, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window, int
     single_below, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float*
-    score_bias, hipStream_t stream);
+    score_bias, int chunked,
+    const float* dist_bias, int bias_len, hipStream_t stream);
 // embed_norm.hip
 int mgpt_embed(const int* ids, const int* pos, const void* tok, const void* postab, float* x, int n_tokens,
     int width, int table_dtype, hipStream_t stream);
@@ -118,8 +121,8 @@ int mgpt_sample_advance(const float* logits, long ld, int n_rows, int vocab, int
     int max_blocks, int* history, int* history_pos, int history_rows, int history_stride, const float*
     tile_best, const int* tile_best_idx, int n_tiles, hipStream_t stream);
 // streams.hip
-int mgpt_embed_scaled(const int* ids, const void* tok, float* x, int n_tokens, int width, int table_dtype, float
-    scale, int copies, hipStream_t stream);
+int mgpt_embed_scaled(const int* ids, const void* tok, const int* pos, const void* postab, float* x, int n_tokens,
+    int width, int table_dtype, float scale, int copies, hipStream_t stream);
 int mgpt_streams_read(const float* x, const float* coef, float* u, float* zero, int n_rows, int width, int
     streams, hipStream_t stream);
 int mgpt_streams_write(float* x, const float* mix, const float* out, const float* y, int n_rows, int width, int
@@ -159,17 +162,19 @@ int mgpt_expert_route(const int* ids, const int* q_req, const int* table, int to
 int mgpt_gather_rows(const void* src, long ld, const int* slot_token, void* sorted, long lds, int n_slots, int width,
     hipStream_t stream);
 int mgpt_router_topk(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
-    int width, int n_experts, int top, int kind, int* chosen, float* weight, hipStream_t stream);
+    int width, int n_experts, int top, int kind, int* chosen, float* weight, const float* correction, int n_groups,
+    int keep, int normalise, float scale, const void* extra, float* extra_out, hipStream_t stream);
 int mgpt_gather_scale_rows(const void* src, int dtype, long ld, const int* slot_token, const int* slot_pair,
     const float* pair_weight, void* sorted, long lds, int n_slots, int width, hipStream_t stream);
 int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int*
     tile_expert, const int* slot_token, void* out, int out_dtype, long ldo, const int* out_rows, int n_tiles,
-    int tile_rows, int n_out, int k_dim, int dtype, hipStream_t stream);
+    int tile_rows, int n_out, int k_dim, int dtype, int epilogue, hipStream_t stream);
 int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int*
     tile_expert, const int* slot_token, void* out, int out_dtype, long ldo, const int* out_rows, int n_tiles,
-    int tile_rows, int n_out, int k_dim, hipStream_t stream);
+    int tile_rows, int n_out, int k_dim, int epilogue, hipStream_t stream);
 int mgpt_expert_combine(const float* pair_out, const int* pair_slot, const int* q_req, float* y, int n_rows, int
-    width, int top, float weight, hipStream_t stream);
+    width, int top, float weight, const float* pair_weight, const float* extra, const float* extra_gate,
+    hipStream_t stream);
 // rms_norm.hip
 int mgpt_rms_norm(const void* x, int x_dtype, long ldx, const int* rows, const float* gain, float offset, float eps,
     float mult, const void* gate, int gate_dtype, long ldg, int gate_act, void* out, int out_dtype, long ldo,
@@ -189,6 +194,17 @@ int mgpt_gated_state_chunked(const void* z, int dtype, long ldz, int q_off, int 
                              float q_scale, float inv_tau, const float* dt_bias, const float* a_log, const float* skip,
                              float* state, long ld_state, const int* state_slots, const int* cu_q, int n_req, int n_tokens,
                              const int* positions, float* qkg, float* out, long ldo, hipStream_t stream);
+// delta_state.hip
+int mgpt_delta_state(const void* x, int dtype, long ldx, int q_off, int k_off, int v_off, const void* z, long ldz,
+    int b_off, int a_off, int gate_off, int n_head, int n_group, int head_dim, int value_dim, float q_scale,
+    const float* dt_bias, const float* a_log, const float* norm_w, float eps, float* state, long ld_state,
+    const int* state_slots, const int* cu_q, int n_req, const int* positions, void* out, long ldo, hipStream_t stream);
+long mgpt_delta_image_floats(int n_tokens, int n_req, int n_head, int head_dim);
+int mgpt_delta_state_chunked(const void* x, int dtype, long ldx, int q_off, int k_off, int v_off, const void* z,
+    long ldz, int b_off, int a_off, int n_head, int n_group, int head_dim, int value_dim, float q_scale,
+    const float* dt_bias, const float* a_log, float* state, long ld_state, const int* state_slots, const int* cu_q,
+    int n_req, int n_tokens, const int* positions, float* images, long image_floats, float* out, long ldo,
+    hipStream_t stream);
 // short_conv.hip
 int mgpt_short_conv(const void* u, int dtype, long ldu, int u_off, const float* w, const float* bias, int act,
     float* state, long ld_state, const int* state_slots, const int* cu_q, const int* q_req, const int* positions,
@@ -211,7 +227,7 @@ int mgpt_decay_state_chunked(const void* z, int dtype, long ldz, int q_off, int 
 // linear_mfma.hip
 int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_stride, const int* row_expert, const
     int* row_valid, int group_rows, void* out, int out_dtype, long ldo, int n_rows, int n_out, int k_dim,
-    hipStream_t stream);
+    int epilogue, hipStream_t stream);
 }
 
 // MGPT_FOR_EACH_LAUNCHER(X) expands X(name) for every launcher above
@@ -270,4 +286,6 @@ int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_st
   X(mgpt_gather_scale_rows) \
   X(mgpt_gated_state) \
   X(mgpt_gated_state_chunked) \
+  X(mgpt_delta_state) \
+  X(mgpt_delta_state_chunked) \
   X(mgpt_short_conv)

@@ -351,6 +351,7 @@ __global__ __launch_bounds__(256) void linear_decode_kernel(SkinnyArgs a) {
       if (LN) v[i] = rstd * (v[i] - md * cs4[i]);
       v[i] += bias4[i];
       if (EPI == SK_EPI_GELU) v[i] = gelu_tanh_fast(v[i]);
+      if (EPI == SK_EPI_RELU2) v[i] = relu_squared(v[i]);
       if (EPI == SK_EPI_RESIDUAL) v[i] += old4[t][i];
     }
     if (VEC && sizeof(OT) == 4) {
@@ -411,6 +412,7 @@ static int launch_decode_epi(const SkinnyArgs& a, int epi, int out_dtype, dim3 g
   if (epi == SK_EPI_NONE && out_dtype == MGPT_BF16) LD_LAUNCH(SK_EPI_NONE, bf16_t);
   else if (epi == SK_EPI_NONE && out_dtype == MGPT_F32) LD_LAUNCH(SK_EPI_NONE, float);
   else if (epi == SK_EPI_GELU && out_dtype == MGPT_BF16) LD_LAUNCH(SK_EPI_GELU, bf16_t);
+  else if (epi == SK_EPI_RELU2 && out_dtype == MGPT_BF16) LD_LAUNCH(SK_EPI_RELU2, bf16_t);
   else if (epi == SK_EPI_RESIDUAL && out_dtype == MGPT_F32) LD_LAUNCH(SK_EPI_RESIDUAL, float);
   else if (epi == SK_EPI_QKV && out_dtype == MGPT_BF16) LD_LAUNCH(SK_EPI_QKV, bf16_t);
   else return MGPT_ERR_BAD_DTYPE;

@@ -79,6 +79,7 @@ __global__ __launch_bounds__(256) void linear_partials_epilogue_kernel(
   for (int i = 0; i < 4; ++i) {
     v[i] += b[i];
     if (EPI == SK_EPI_GELU) v[i] = gelu_tanh_fast(v[i]);
+    if (EPI == SK_EPI_RELU2) v[i] = relu_squared(v[i]);
   }
   if (sizeof(OT) == 4) {
     *reinterpret_cast<float4*>(orow) = make_float4(v[0] + old.x, v[1] + old.y, v[2] + old.z, v[3] + old.w);
@@ -113,6 +114,7 @@ static int launch_split(const SkinnyArgs& a0, int epilogue, int out_dtype, hipSt
   if (epilogue == SK_EPI_NONE && out_dtype == MGPT_BF16) LDR_EPI(SK_EPI_NONE, bf16_t);
   else if (epilogue == SK_EPI_NONE && out_dtype == MGPT_F32) LDR_EPI(SK_EPI_NONE, float);
   else if (epilogue == SK_EPI_GELU && out_dtype == MGPT_BF16) LDR_EPI(SK_EPI_GELU, bf16_t);
+  else if (epilogue == SK_EPI_RELU2 && out_dtype == MGPT_BF16) LDR_EPI(SK_EPI_RELU2, bf16_t);
   else if (epilogue == SK_EPI_RESIDUAL && out_dtype == MGPT_F32) LDR_EPI(SK_EPI_RESIDUAL, float);
   else return MGPT_ERR_BAD_DTYPE;
 #undef LDR_EPI

@@ -1,6 +1,6 @@
 // Plain tiled matrix product with 32-bit FMA accumulation, for every storage
 // type pair.  out[n, o] = sum_k A[n, k] * W[o, k] (+ bias[o]) with an optional
-// GELU-tanh or residual-add epilogue: y = x W^T + b as nn.Linear
+// GELU-tanh, squared-relu or residual-add epilogue: y = x W^T + b as nn.Linear
 // (reference: src/minigpt_infer/model.py:43-44,96-101).
 //
 // This is the kernel of the true 32-bit path: k runs 0..K-1 in order for every
@@ -13,6 +13,7 @@
 #define EPI_NONE 0
 #define EPI_GELU 1
 #define EPI_RESIDUAL 2  // out (float) += result
+#define EPI_RELU2 5     // max(result, 0)^2
 
 #define TILE 64
 #define BK 16
@@ -75,6 +76,7 @@ __global__ __launch_bounds__(256) void linear_generic_kernel(
       float v = acc[i][j];
       if (bias) v += bias[c];
       if (EPI == EPI_GELU) v = gelu_tanh(v);
+      if (EPI == EPI_RELU2) v = relu_squared(v);
       OT* dst = out + (long)r * ldo + c;
       if (EPI == EPI_RESIDUAL) {
         *dst = from_float<OT>(to_float<OT>(*dst) + v);
@@ -130,6 +132,7 @@ __global__ __launch_bounds__(256) void linear_generic_rows_kernel(
   float v = acc;
   if (bias) v += bias[col];
   if (EPI == EPI_GELU) v = gelu_tanh(v);
+  if (EPI == EPI_RELU2) v = relu_squared(v);
   OT* dst = out + (long)row * ldo + col;
   if (EPI == EPI_RESIDUAL) {
     *dst = from_float<OT>(to_float<OT>(*dst) + v);
@@ -155,6 +158,7 @@ static int launch_epi(const void* A, long lda, const void* W, const float* bias,
                        lda, (const WT*)W, bias, (OT*)out, ldo, n_rows, n_out, k_dim)
   if (epi == EPI_NONE) { LAUNCH(EPI_NONE); }
   else if (epi == EPI_GELU) { LAUNCH(EPI_GELU); }
+  else if (epi == EPI_RELU2) { LAUNCH(EPI_RELU2); }
   else if (epi == EPI_RESIDUAL) { LAUNCH(EPI_RESIDUAL); }
   else return MGPT_ERR_BAD_SHAPE;
 #undef LAUNCH

@@ -41,6 +41,7 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4_t;
 #define MM_EPI_GELU 1
 #define MM_EPI_RESIDUAL 2
 #define MM_EPI_QKV 3   // store, and scatter the key and value columns into their cache pages
+#define MM_EPI_RELU2 5 // max(v, 0)^2
 #define MM_EPI_XIELU 4 // a_p v^2 + v / 2 for v > 0, a_n (exp(v) - 1 - v) + v / 2 else, (a_p, a_n) from MfmaScatter::epi_coef
 
 __device__ __forceinline__ float mfma_xielu(float v, float a_p, float a_n) {
@@ -90,6 +91,7 @@ __device__ __forceinline__ void mfma_store4(const f32x4_t& a, const float b4[4],
   for (int e = 0; e < 4; ++e) {
     v[e] = a[e] + b4[e];
     if (EPI == MM_EPI_GELU) v[e] = gelu_tanh_fast(v[e]);
+    if (EPI == MM_EPI_RELU2) v[e] = relu_squared(v[e]);
     if (EPI == MM_EPI_XIELU) v[e] = mfma_xielu(v[e], a_p, a_n);
   }
   if (vec && sizeof(OT) == 4) {
@@ -465,6 +467,7 @@ __global__ __launch_bounds__(64 * WVM * WVN * KG) void linear_mfma_kernel(
             for (int e = 0; e < 4; ++e) {
               v[e] = acc[i][j][e] + b4[e];
               if (EPI == MM_EPI_GELU) v[e] = gelu_tanh_fast(v[e]);
+              if (EPI == MM_EPI_RELU2) v[e] = relu_squared(v[e]);
               if (EPI == MM_EPI_XIELU) v[e] = mfma_xielu(v[e], xa_p, xa_n);
             }
             uint2 pk;
@@ -573,6 +576,7 @@ int launch_shape(const void* act, long lda, const void* w, const float* bias, vo
   if (epilogue == MM_EPI_NONE && out_dtype == MGPT_BF16) MM_LAUNCH(MM_EPI_NONE, bf16_t);
   if (epilogue == MM_EPI_NONE && out_dtype == MGPT_F32) MM_LAUNCH(MM_EPI_NONE, float);
   if (epilogue == MM_EPI_GELU && out_dtype == MGPT_BF16) MM_LAUNCH(MM_EPI_GELU, bf16_t);
+  if (epilogue == MM_EPI_RELU2 && out_dtype == MGPT_BF16) MM_LAUNCH(MM_EPI_RELU2, bf16_t);
   if (epilogue == MM_EPI_XIELU && out_dtype == MGPT_BF16) MM_LAUNCH(MM_EPI_XIELU, bf16_t);
   if (epilogue == MM_EPI_RESIDUAL && out_dtype == MGPT_F32) MM_LAUNCH(MM_EPI_RESIDUAL, float);
   if (epilogue == MM_EPI_QKV && out_dtype == MGPT_BF16) MM_LAUNCH(MM_EPI_QKV, bf16_t);
@@ -706,6 +710,9 @@ __global__ __launch_bounds__(256) void linear_mfma_join_kernel(const float* __re
   if (EPI == MM_EPI_GELU) {
     v.x = gelu_tanh_fast(v.x); v.y = gelu_tanh_fast(v.y); v.z = gelu_tanh_fast(v.z); v.w = gelu_tanh_fast(v.w);
   }
+  if (EPI == MM_EPI_RELU2) {
+    v.x = relu_squared(v.x); v.y = relu_squared(v.y); v.z = relu_squared(v.z); v.w = relu_squared(v.w);
+  }
   if (EPI == MM_EPI_XIELU) {
     const float a_p = epi_coef[0], a_n = epi_coef[1];
     v.x = mfma_xielu(v.x, a_p, a_n); v.y = mfma_xielu(v.y, a_p, a_n); v.z = mfma_xielu(v.z, a_p, a_n); v.w = mfma_xielu(v.w, a_p, a_n);
@@ -729,6 +736,7 @@ int launch_join(const float* partials, int k_parts, const float* bias, void* out
   if (epilogue == MM_EPI_NONE && out_dtype == MGPT_BF16) MM_JOIN(MM_EPI_NONE, bf16_t);
   else if (epilogue == MM_EPI_NONE && out_dtype == MGPT_F32) MM_JOIN(MM_EPI_NONE, float);
   else if (epilogue == MM_EPI_GELU && out_dtype == MGPT_BF16) MM_JOIN(MM_EPI_GELU, bf16_t);
+  else if (epilogue == MM_EPI_RELU2 && out_dtype == MGPT_BF16) MM_JOIN(MM_EPI_RELU2, bf16_t);
   else if (epilogue == MM_EPI_XIELU && out_dtype == MGPT_BF16) MM_JOIN(MM_EPI_XIELU, bf16_t);
   else if (epilogue == MM_EPI_RESIDUAL && out_dtype == MGPT_F32) MM_JOIN(MM_EPI_RESIDUAL, float);
   else return MGPT_ERR_BAD_DTYPE;
@@ -974,11 +982,12 @@ extern "C" int mgpt_linear_mfma_shape(int shape, int k_parts, const void* act, l
 // Rows in groups of group_rows (256) that each multiply a matrix of their own: out[r] = act[r] W_e^T with
 // e = row_expert[r / group_rows] (negative: nothing is computed for the group) and W_e = w + e * w_stride;
 // row_valid[r] < 0 marks the padding that ends a group, and a tile that starts in it is skipped.  bfloat16 or
-// float32 out, no bias, the inner size never split.
+// float32 out, no bias, no epilogue or (bfloat16 out) the squared relu, the inner size never split.
 extern "C" int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_stride, const int* row_expert,
                                         const int* row_valid, int group_rows, void* out, int out_dtype, long ldo,
-                                        int n_rows, int n_out, int k_dim, hipStream_t stream) {
+                                        int n_rows, int n_out, int k_dim, int epilogue, hipStream_t stream) {
   if (!row_expert || !row_valid) return MGPT_ERR_NULL;
+  if (epilogue != MM_EPI_NONE && epilogue != MM_EPI_RELU2) return MGPT_ERR_BAD_SHAPE;
   // every tile shape's rows (32 to 256) divide a group
   if (group_rows != 256 || (n_rows % group_rows) != 0 || w_stride < (long)n_out * k_dim || (w_stride & 7) != 0)
     return MGPT_ERR_BAD_SHAPE;
@@ -987,7 +996,7 @@ extern "C" int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w
   sc.row_valid = row_valid;
   sc.group_rows = group_rows;
   sc.w_stride = w_stride;
-  return launch_any(-1, 1, act, lda, w, nullptr, out, out_dtype, ldo, n_rows, n_out, k_dim, MM_EPI_NONE, nullptr, 0, sc,
+  return launch_any(-1, 1, act, lda, w, nullptr, out, out_dtype, ldo, n_rows, n_out, k_dim, epilogue, nullptr, 0, sc,
                     stream);
 }
 

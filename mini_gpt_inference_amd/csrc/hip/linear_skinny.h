@@ -9,6 +9,7 @@ typedef __attribute__((__vector_size__(4 * sizeof(float)))) float f32x4_t;
 #define SK_EPI_GELU 1
 #define SK_EPI_RESIDUAL 2
 #define SK_EPI_QKV 3
+#define SK_EPI_RELU2 5
 
 #define SK_ROWS_SHARE_W 2
 #define SK_ROWS_GROUPS 3

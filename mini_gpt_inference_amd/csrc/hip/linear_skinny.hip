@@ -18,7 +18,7 @@
 // bfloat16 on the way into the MFMA, with an optional gather of rows for the output head),
 // gathers each row's sum and sum of squares from the very values it loads, and applies
 // rstd * (acc - mean * S[o]) + b'[o] in the epilogue.  Nothing waits for the statistics.
-// Epilogues: plain store (bfloat16 or float32), GELU-tanh, add into the float32
+// Epilogues: plain store (bfloat16 or float32), GELU-tanh, squared relu, add into the float32
 // residual stream, or store plus scatter of the key and value columns into
 // their cache pages by slot_mapping (src/minigpt_infer/cache/paged.py:125-137).
 #include "linear_skinny.h"
@@ -241,6 +241,7 @@ __global__ __launch_bounds__(WAVES * 64) void linear_skinny_kernel(SkinnyArgs a)
         if (LN && oc + i < a.n_out) v[i] = rstd * (v[i] - md * a.colsum[oc + i]);
         if (a.bias && oc + i < a.n_out) v[i] += a.bias[oc + i];
         if (EPI == SK_EPI_GELU) v[i] = gelu_tanh_fast(v[i]);
+        if (EPI == SK_EPI_RELU2) v[i] = relu_squared(v[i]);
       }
       OT* orow = reinterpret_cast<OT*>(a.out) + (long)n * a.ldo;
       const bool whole = oc + 4 <= a.n_out && (a.ldo & 3) == 0;  // four columns, one aligned vector
@@ -296,6 +297,7 @@ static int launch_nt(const SkinnyArgs& a, int epi, int out_dtype, dim3 grid, siz
   if (epi == SK_EPI_NONE && out_dtype == MGPT_BF16) SK_LAUNCH(SK_EPI_NONE, bf16_t);
   else if (epi == SK_EPI_NONE && out_dtype == MGPT_F32) SK_LAUNCH(SK_EPI_NONE, float);
   else if (epi == SK_EPI_GELU && out_dtype == MGPT_BF16) SK_LAUNCH(SK_EPI_GELU, bf16_t);
+  else if (epi == SK_EPI_RELU2 && out_dtype == MGPT_BF16) SK_LAUNCH(SK_EPI_RELU2, bf16_t);
   else if (epi == SK_EPI_RESIDUAL && out_dtype == MGPT_F32) SK_LAUNCH(SK_EPI_RESIDUAL, float);
   else if (epi == SK_EPI_QKV && out_dtype == MGPT_BF16) SK_LAUNCH(SK_EPI_QKV, bf16_t);
   else return MGPT_ERR_BAD_DTYPE;

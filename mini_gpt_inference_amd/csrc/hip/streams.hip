@@ -12,30 +12,34 @@
 
 template <typename WT>
 __global__ void embed_scaled_kernel(const int* __restrict__ ids, const WT* __restrict__ tok,
+                                    const int* __restrict__ pos, const WT* __restrict__ postab,
                                     float* __restrict__ x, int n_tokens, int width, float scale, int copies) {
   const int n = blockIdx.x;
   if (n >= n_tokens) return;
   const WT* trow = tok + (long)ids[n] * width;
+  const WT* prow = postab ? postab + (long)pos[n] * width : nullptr;
   float* xr = x + (long)n * copies * width;
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    const float v = to_float<WT>(trow[c]) * scale;
+    float v = to_float<WT>(trow[c]) * scale;
+    if (prow) v += to_float<WT>(prow[c]);
     for (int s = 0; s < copies; ++s) xr[(long)s * width + c] = v;
   }
 }
 
-// x[n][s] = tok[ids[n]] * scale for every s < copies
-extern "C" int mgpt_embed_scaled(const int* ids, const void* tok, float* x, int n_tokens, int width,
+// x[n][s] = tok[ids[n]] * scale (+ postab[pos[n]], of the same type) for every s < copies
+extern "C" int mgpt_embed_scaled(const int* ids, const void* tok, const int* pos, const void* postab, float* x,
+                                 int n_tokens, int width,
                                  int table_dtype, float scale, int copies, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
-  if (!ids || !tok || !x) return MGPT_ERR_NULL;
+  if (!ids || !tok || !x || (postab && !pos)) return MGPT_ERR_NULL;
   if (n_tokens < 0 || width <= 0 || copies <= 0) return MGPT_ERR_BAD_SHAPE;
   const int threads = width >= 256 ? 256 : 64;
   if (table_dtype == MGPT_F32) {
     hipLaunchKernelGGL(embed_scaled_kernel<float>, dim3(n_tokens), dim3(threads), 0, stream, ids,
-                       (const float*)tok, x, n_tokens, width, scale, copies);
+                       (const float*)tok, pos, (const float*)postab, x, n_tokens, width, scale, copies);
   } else if (table_dtype == MGPT_BF16) {
     hipLaunchKernelGGL(embed_scaled_kernel<bf16_t>, dim3(n_tokens), dim3(threads), 0, stream, ids,
-                       (const bf16_t*)tok, x, n_tokens, width, scale, copies);
+                       (const bf16_t*)tok, pos, (const bf16_t*)postab, x, n_tokens, width, scale, copies);
   } else {
     return MGPT_ERR_BAD_DTYPE;
   }

@@ -80,7 +80,7 @@ int CacheManager::release_passed(int slot, int n_computed) {
     const int w = groups_[g].window;
     if (w <= 0) continue;
     // the query at position n_computed is the earliest still to come; it sees keys from here on
-    const int earliest = n_computed - w + 1;
+    const int earliest = groups_[g].chunked ? n_computed - n_computed % w : n_computed - w + 1;
     if (earliest <= 0) continue;
     const int keep_from = std::min(earliest / groups_[g].page_size, (int)s.tables[g].size());
     // pages that hold one of the kept first positions stay

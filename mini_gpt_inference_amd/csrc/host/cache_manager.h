@@ -3,8 +3,8 @@
 // Follows the reference's BlockManager (src/minigpt_infer/cache/paged.py:32-94):
 // a LIFO free list of page ids, tables that grow by whole pages, nothing is
 // cleared when it is given back.  Beyond the reference: several groups of
-// layers, each with a page pool of its own (all keys, or a window of them whose
-// passed pages return early), and a fixed number of request slots that index
+// layers, each with a page pool of its own (all keys, or a window of them, sliding
+// or chunk by chunk, whose passed pages return early), and a fixed number of request slots that index
 // both the tables and any fixed-size per-request state.
 #pragma once
 
@@ -18,6 +18,7 @@ struct GroupSpec {
   int num_pages;  // pages in this group's pool
   int window;     // 0: a query sees all earlier keys; w > 0: only the last w positions
   int keep_first = 0;  // with a window: every query also sees the first keep_first positions, whose pages stay
+  int chunked = 0;     // with a window: it is the size of chunks counted from position 0, and a query sees its own chunk
 };
 
 class CacheManager {

@@ -173,7 +173,8 @@ class LLMEngine:
         pages = plan_group_pages(layout.groups, engine_config.block_size, engine_config.num_blocks,
                                  engine_config.kv_cache_bytes, 2 if self.dtype == torch.bfloat16 else 4,
                                  model.spec.max_positions)
-        geometry = [GroupGeometry(engine_config.block_size, n, g.window, g.keep_first) for g, n in zip(layout.groups, pages)]
+        geometry = [GroupGeometry(engine_config.block_size, n, g.window, g.keep_first, g.chunked)
+                    for g, n in zip(layout.groups, pages)]
         self.cache = CacheManager(geometry, engine_config.max_batch_size)
         self.store = KVStore(layout, geometry, engine_config.max_batch_size, self.dtype, self.device)
         max_positions = model.spec.max_positions

@@ -18,6 +18,7 @@ from . import library
 
 F32, BF16 = 0, 1
 EPI_NONE, EPI_GELU, EPI_RESIDUAL = 0, 1, 2
+EPI_RELU2 = 5      # max(result, 0)^2
 EPI_XIELU = 4      # only through linear_mfma_xielu, which brings the activation's coefficients
 
 _ERRORS = {
@@ -179,16 +180,25 @@ def kv_write(qkv: torch.Tensor, k_off: int, v_off: int, k_pool: torch.Tensor, v_
     _check(rc, "kv_write")
 
 
-def _mask_args(keep_first: int, score_bias: Optional[torch.Tensor], n_head: int, sinks, softcap: float):
-    """(first positions that a window keeps, pointer of the per-head number added to a score before its sigmoid):
-    the two optional arguments behind the gate's.  With score_bias the weights are sigmoids and not a softmax, so
-    sinks and a score cap do not go with it."""
+def _mask_args(keep_first: int, score_bias: Optional[torch.Tensor], n_head: int, sinks, softcap: float,
+               chunked: bool = False, dist_bias: Optional[torch.Tensor] = None):
+    """(first positions that a window keeps, pointer of the per-head number added to a score before its sigmoid,
+    whether the window is a chunk, pointer and row length of the numbers by distance): the optional arguments
+    behind the gate's.  With score_bias the weights are sigmoids and not a softmax, so sinks and a score cap do not
+    go with it; numbers by distance go with neither score_bias nor a score cap."""
     _need(int(keep_first) >= 0, "keep_first must not be negative")
     if score_bias is not None:
         _need(score_bias.is_cuda and score_bias.dtype == torch.float32 and score_bias.is_contiguous()
               and score_bias.numel() == n_head, "score_bias must be float32 [n_head] on the GPU")
         _need(sinks is None and not softcap > 0.0, "sigmoid weights take neither sinks nor a score cap")
-    return int(keep_first), _ptr(score_bias)
+    bias_len = 0
+    if dist_bias is not None:
+        _need(dist_bias.is_cuda and dist_bias.dtype == torch.float32 and dist_bias.is_contiguous()
+              and dist_bias.dim() == 2 and dist_bias.shape[0] == n_head and dist_bias.shape[1] > 0,
+              "dist_bias must be dense float32 [n_head, distances] on the GPU")
+        _need(score_bias is None and not softcap > 0.0, "numbers by distance go with neither score_bias nor a score cap")
+        bias_len = dist_bias.shape[1]
+    return int(keep_first), _ptr(score_bias), 1 if chunked else 0, _ptr(dist_bias), bias_len
 
 
 def _gate_args(gate: Optional[torch.Tensor], q: torch.Tensor, n_tokens: int, n_head: int):
@@ -226,12 +236,15 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Te
                             q_req: torch.Tensor, n_tokens: int, n_req: int, n_head: int, scale: float,
                             window: int = 0, fast_exp: bool = False, sinks: Optional[torch.Tensor] = None,
                             softcap: float = 0.0, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
-                            score_bias: Optional[torch.Tensor] = None) -> None:
+                            score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
+                            dist_bias: Optional[torch.Tensor] = None) -> None:
     """Causal attention of the step's tokens over their requests' pages (any q_len, any dtype).
     sinks: float32 [n_head], one more term exp(sinks[h]) in every softmax denominator of head h.
     softcap > 0: every score becomes softcap * tanh(score / softcap) before the softmax.
     keep_first: behind a window a query also sees the keys at positions below it.  score_bias: float32 [n_head];
-    a visible key's weight is sigmoid(score + score_bias[h]), not normalised over the keys."""
+    a visible key's weight is sigmoid(score + score_bias[h]), not normalised over the keys.  chunked: `window` is the
+    size of chunks counted from position 0, and a query sees its own chunk.  dist_bias: float32 [n_head, L], the
+    number at [h, min(i - j, L - 1)] is added to the scaled score of query i and key j."""
     n_kv_head, page_size, head_dim = _check_attention_args(
         q, out, k_pool, v_pool, block_tables, cu_q, seq_lens, q_req, n_tokens, n_req, n_head)
     _need(head_dim <= 1024, f"head size {head_dim} exceeds the kernel's limit of 1024")
@@ -240,7 +253,7 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Te
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), _ptr(q_req), n_tokens, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), _dtype_code(q), int(fast_exp), _ptr(sinks), float(softcap), *_gate_args(gate, q, n_tokens, n_head),
-        *_mask_args(keep_first, score_bias, n_head, sinks, softcap), _stream())
+        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
     _check(rc, "paged_attention_generic")
 
 
@@ -363,7 +376,7 @@ def linear_skinny(a: Optional[torch.Tensor], w: torch.Tensor, bias: Optional[tor
     _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == n_out), "bias must be float32 [out]")
     if epilogue == EPI_RESIDUAL:
         _need(out.dtype == torch.float32, "the residual stream is float32")
-    elif epilogue in (EPI_GELU, SK_EPI_QKV):
+    elif epilogue in (EPI_GELU, EPI_RELU2, SK_EPI_QKV):
         _need(out.dtype == torch.bfloat16, "this epilogue writes bfloat16")
     lda = 0
     if ln_x is not None:
@@ -516,7 +529,8 @@ def paged_attention_split_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch
                                q_req: torch.Tensor, n_tokens: int, n_req: int, n_head: int, scale: float,
                                window: int = 0, fast: bool = True, sinks: Optional[torch.Tensor] = None,
                                softcap: float = 0.0, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
-                               score_bias: Optional[torch.Tensor] = None) -> bool:
+                               score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
+                               dist_bias: Optional[torch.Tensor] = None) -> bool:
     """bfloat16 attention with each (token, head)'s keys split over four waves.  False if refused.
     fast=False keeps to the variant that takes every head size."""
     if q.dtype != torch.bfloat16:
@@ -533,7 +547,7 @@ def paged_attention_split_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), _ptr(q_req), n_tokens, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), _ptr(sinks), float(softcap), *_gate_args(gate, q, n_tokens, n_head),
-        *_mask_args(keep_first, score_bias, n_head, sinks, softcap), _stream())
+        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
     if rc == -2:
         return False
     _check(rc, "paged_attention_split_bf16")
@@ -546,7 +560,8 @@ def paged_attention_decode_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torc
                                 identity: bool = False, cu_q: Optional[torch.Tensor] = None,
                                 sinks: Optional[torch.Tensor] = None, softcap: float = 0.0,
                                 gate: Optional[torch.Tensor] = None, keep_first: int = 0,
-                                score_bias: Optional[torch.Tensor] = None) -> bool:
+                                score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
+                                dist_bias: Optional[torch.Tensor] = None) -> bool:
     """bfloat16 attention for single tokens (one query per request and step), keys split over eight
     waves.  positions[n] is token n's absolute position, q_req[n] its block table row or -1 for a
     padded token; identity=True promises q_req[n] in (n, -1).  With cu_q (the requests' token offsets;
@@ -582,7 +597,7 @@ def paged_attention_decode_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torc
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(positions), _ptr(q_req), _ptr(cu_q), n_tokens, n_head, n_kv_head, head_dim, page_size,
         num_pages, float(scale), int(window), 1 if identity else 0, _ptr(sinks), float(softcap),
-        *_gate_args(gate, q, n_tokens, n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap), _stream())
+        *_gate_args(gate, q, n_tokens, n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
     if rc == -2:
         return False
     _check(rc, "paged_attention_decode_bf16")
@@ -651,7 +666,8 @@ def linear_mfma(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], 
     if scatter is not None and (epilogue != EPI_NONE or out.dtype != torch.bfloat16):
         return False
     if (epilogue, out.dtype) not in ((EPI_NONE, torch.bfloat16), (EPI_NONE, torch.float32),
-                                     (EPI_GELU, torch.bfloat16), (EPI_RESIDUAL, torch.float32)):
+                                     (EPI_GELU, torch.bfloat16), (EPI_RELU2, torch.bfloat16),
+                                     (EPI_RESIDUAL, torch.float32)):
         return False
     _need_cuda(a, w, bias, out)
     _need(w.is_contiguous(), "weight must be dense [out, in]")
@@ -723,7 +739,8 @@ def prefill_attention_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Ten
                            max_q_len: int, n_head: int, scale: float, window: int = 0,
                            single_below: int = 0, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0,
                            gate: Optional[torch.Tensor] = None, keep_first: int = 0,
-                           score_bias: Optional[torch.Tensor] = None) -> bool:
+                           score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
+                           dist_bias: Optional[torch.Tensor] = None) -> bool:
     """MFMA tile attention for steps with prompt portions (every request's tokens are consecutive
     rows of q from cu_q; a request may bring none).  Requests that bring exactly one token, and that
     among the step's first `single_below` tokens, are left to another kernel.  False when it does
@@ -751,7 +768,7 @@ def prefill_attention_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Ten
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), n_req, max_q_len, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), int(single_below), _ptr(sinks), float(softcap),
-        *_gate_args(gate, q, q.shape[0], n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap), _stream())
+        *_gate_args(gate, q, q.shape[0], n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
     if rc == -2:
         return False
     _check(rc, "prefill_attention_bf16")
@@ -1002,16 +1019,23 @@ MAX_STREAMS = 8
 
 
 def embed_scaled(ids: torch.Tensor, table: torch.Tensor, x: torch.Tensor, n_tokens: int, scale: float,
-                 copies: int = 1) -> None:
-    """x[t][s] = table[ids[t]] * scale for every s < copies; x is float32 [>=n_tokens, copies * width]."""
-    _need_cuda(ids, table, x)
+                 copies: int = 1, positions: Optional[torch.Tensor] = None,
+                 pos_table: Optional[torch.Tensor] = None) -> None:
+    """x[t][s] = table[ids[t]] * scale (+ pos_table[positions[t]]) for every s < copies; x is float32 [>=n_tokens,
+    copies * width]."""
+    _need_cuda(ids, table, x, positions, pos_table)
     width = table.shape[1]
     _need(table.dim() == 2 and table.is_contiguous(), "embedding table must be dense [vocab, width]")
     _need(x.dtype == torch.float32 and x.is_contiguous() and x.shape[1] == copies * width and x.shape[0] >= n_tokens,
           "residual streams must be dense float32 [>=n_tokens, copies * width]")
     _need_i32("ids", ids, n_tokens)
-    rc = library.kernels().mgpt_embed_scaled(_ptr(ids), _ptr(table), _ptr(x), n_tokens, width, _dtype_code(table),
-                                             float(scale), int(copies), _stream())
+    if pos_table is not None:
+        _need(pos_table.dtype == table.dtype and pos_table.is_contiguous() and pos_table.shape[1] == width,
+              "position table must match the token table's dtype and width")
+        _need(positions is not None, "positions are needed with a position table")
+        _need_i32("positions", positions, n_tokens)
+    rc = library.kernels().mgpt_embed_scaled(_ptr(ids), _ptr(table), _ptr(positions), _ptr(pos_table), _ptr(x), n_tokens,
+                                             width, _dtype_code(table), float(scale), int(copies), _stream())
     _check(rc, "embed_scaled")
 
 
@@ -1309,9 +1333,9 @@ def expert_route(ids: Optional[torch.Tensor], q_req: Optional[torch.Tensor], tab
 
 def grouped_linear(a: torch.Tensor, a_rows: Optional[torch.Tensor], w: torch.Tensor, tile_expert: torch.Tensor,
                    slot_token: torch.Tensor, out: torch.Tensor, out_rows: Optional[torch.Tensor], n_slots: int,
-                   tile: int, fast: bool = False) -> None:
-    """out[out_rows[s] or s] = a[a_rows[s] or s] @ w[expert of s's tile].T for every used slot s < n_slots.
-    w: [experts, n_out, k_dim]."""
+                   tile: int, fast: bool = False, epilogue: int = EPI_NONE) -> None:
+    """out[out_rows[s] or s] = a[a_rows[s] or s] @ w[expert of s's tile].T for every used slot s < n_slots, with
+    the squared relu behind it where the epilogue is EPI_RELU2.  w: [experts, n_out, k_dim]."""
     _need_cuda(a, a_rows, w, tile_expert, slot_token, out, out_rows)
     _need(w.dim() == 3 and w.is_contiguous(), "the experts' matrices must be dense [experts, out, in]")
     _, n_out, k_dim = w.shape
@@ -1331,22 +1355,25 @@ def grouped_linear(a: torch.Tensor, a_rows: Optional[torch.Tensor], w: torch.Ten
         rc = library.kernels().mgpt_grouped_linear_mfma(_ptr(a), a.stride(0), _ptr(a_rows), _ptr(w), w.stride(0),
                                                         _ptr(tile_expert), _ptr(slot_token), _ptr(out),
                                                         _dtype_code(out), out.stride(0), _ptr(out_rows),
-                                                        n_slots // tile, tile, n_out, k_dim, _stream())
+                                                        n_slots // tile, tile, n_out, k_dim, epilogue, _stream())
         if rc != -2:
             _check(rc, "grouped_linear_mfma")
             return
     rc = library.kernels().mgpt_grouped_linear(_ptr(a), a.stride(0), _ptr(a_rows), _ptr(w), w.stride(0),
                                                _ptr(tile_expert), _ptr(slot_token), _ptr(out), _dtype_code(out),
                                                out.stride(0), _ptr(out_rows), n_slots // tile, tile, n_out, k_dim,
-                                               _dtype_code(a), _stream())
+                                               _dtype_code(a), epilogue, _stream())
     _check(rc, "grouped_linear")
 
 
 def expert_combine(pair_out: torch.Tensor, y: torch.Tensor, n_rows: int, top: int, weight: float,
-                   pair_slot: Optional[torch.Tensor] = None, q_req: Optional[torch.Tensor] = None) -> None:
-    """y[n] += weight * sum_k pair_out[pair_slot[n * top + k]] (without pair_slot: row n * top + k); both
-    float32.  Tokens whose q_req is negative (padding) are left alone."""
-    _need_cuda(pair_out, y, pair_slot, q_req)
+                   pair_slot: Optional[torch.Tensor] = None, q_req: Optional[torch.Tensor] = None,
+                   pair_weight: Optional[torch.Tensor] = None, extra: Optional[torch.Tensor] = None,
+                   extra_gate: Optional[torch.Tensor] = None) -> None:
+    """y[n] += weight * sum_k pair_weight[n * top + k] * pair_out[pair_slot[n * top + k]] (without pair_slot: row
+    n * top + k; without pair_weight: 1) + extra_gate[n] * extra[n] (without extra: nothing; without extra_gate:
+    1); all float32.  Tokens whose q_req is negative (padding) are left alone."""
+    _need_cuda(pair_out, y, pair_slot, q_req, pair_weight, extra, extra_gate)
     width = y.shape[1]
     _need_rows_f32("y", y, n_rows, width)
     if pair_slot is None:
@@ -1356,8 +1383,14 @@ def expert_combine(pair_out: torch.Tensor, y: torch.Tensor, n_rows: int, top: in
         _need_i32("pair_slot", pair_slot, n_rows * top)
     if q_req is not None:
         _need_i32("q_req", q_req, n_rows)
+    for name, t, count in (("pair_weight", pair_weight, n_rows * top), ("extra_gate", extra_gate, n_rows)):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() >= count),
+              f"{name} must be dense float32 of at least {count} entries")
+    if extra is not None:
+        _need_rows_f32("extra", extra, n_rows, width)
     rc = library.kernels().mgpt_expert_combine(_ptr(pair_out), _ptr(pair_slot), _ptr(q_req), _ptr(y), n_rows, width,
-                                               top, float(weight), _stream())
+                                               top, float(weight), _ptr(pair_weight), _ptr(extra), _ptr(extra_gate),
+                                               _stream())
     _check(rc, "expert_combine")
 
 
@@ -1382,11 +1415,18 @@ ROUTER_SCORES = {"sigmoid": 0, "logit": 1}
 
 
 def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen: torch.Tensor, weight: torch.Tensor,
-                q_req: Optional[torch.Tensor] = None, score: str = "sigmoid") -> None:
+                q_req: Optional[torch.Tensor] = None, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
+                groups=None, normalise: bool = False, scale: float = 1.0, extra: Optional[torch.Tensor] = None,
+                extra_out: Optional[torch.Tensor] = None) -> None:
     """chosen[n] = the `top` experts with the largest w[e] . h[n] (float32 sums), best first; weight[n] = their
     scores (sigmoid of the sum, or the sum itself).  w: dense [experts, width]; chosen int32 and weight float32,
-    dense [>= n_rows, top]."""
-    _need_cuda(h, w, chosen, weight, q_req)
+    dense [>= n_rows, top].
+
+    correction (float32 [experts]) is added to the scores that the choice goes by; groups = (count, keep): only the
+    experts of the `keep` groups (of `count` equal groups of neighbours) whose two largest choice scores have the
+    largest sums can be chosen; normalise: the weights are the chosen scores over (their sum + 1e-20); every weight
+    is multiplied by `scale`.  extra ([width], like w): extra_out[n] = sigmoid(extra . h[n]), float32."""
+    _need_cuda(h, w, chosen, weight, q_req, correction, extra, extra_out)
     _need(score in ROUTER_SCORES, f"router score {score!r} is none of {sorted(ROUTER_SCORES)}")
     _need(w.dim() == 2 and w.is_contiguous() and w.dtype in (torch.float32, torch.bfloat16), "the router's matrix must be dense")
     n_experts, width = w.shape
@@ -1399,8 +1439,19 @@ def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen:
           "weight must be float32, shaped like chosen")
     if q_req is not None:
         _need_i32("q_req", q_req, n_rows)
+    count, keep = (1, 1) if groups is None else (int(groups[0]), int(groups[1]))
+    _need(0 < keep <= count and n_experts % count == 0 and top <= keep * (n_experts // count),
+          f"groups {groups}: {n_experts} experts in equal groups of which enough stay for {top} choices")
+    _need(correction is None or (correction.dtype == torch.float32 and correction.is_contiguous()
+                                 and correction.numel() == n_experts), "correction must be float32 [experts]")
+    if extra is not None:
+        _need(extra.dtype == w.dtype and extra.is_contiguous() and extra.numel() == width, "extra must be a row like w's")
+        _need(extra_out is not None and extra_out.dtype == torch.float32 and extra_out.is_contiguous()
+              and extra_out.numel() >= n_rows, "extra_out must be dense float32 of n_rows entries")
     rc = library.kernels().mgpt_router_topk(_ptr(h), _dtype_code(h), h.stride(0), _ptr(w), _dtype_code(w), _ptr(q_req), n_rows,
-                                            width, n_experts, top, ROUTER_SCORES[score], _ptr(chosen), _ptr(weight), _stream())
+                                            width, n_experts, top, ROUTER_SCORES[score], _ptr(chosen), _ptr(weight),
+                                            _ptr(correction), count, keep, 1 if normalise else 0, float(scale), _ptr(extra),
+                                            _ptr(extra_out), _stream())
     _check(rc, "router_topk")
 
 
@@ -1422,9 +1473,9 @@ def gather_scale_rows(src: torch.Tensor, slot_token: torch.Tensor, slot_pair: to
 
 
 def grouped_linear_tiled(a: torch.Tensor, w: torch.Tensor, tile_expert: torch.Tensor, slot_token: torch.Tensor,
-                         out: torch.Tensor, n_slots: int) -> bool:
+                         out: torch.Tensor, n_slots: int, epilogue: int = EPI_NONE) -> bool:
     """out[s] = a[s] @ w[expert of s's tile of 256].T for the slots of every tile in use, through the
-    tiled MFMA kernel (bfloat16 operands, bfloat16 or float32 out).  False, with nothing launched,
+    tiled MFMA kernel (bfloat16 operands, bfloat16 or float32 out; EPI_RELU2: bfloat16 out).  False, with nothing launched,
     if that kernel does not take the sizes."""
     _need_cuda(a, w, tile_expert, slot_token, out)
     _need(w.dim() == 3 and w.is_contiguous(), "the experts' matrices must be dense [experts, out, in]")
@@ -1439,7 +1490,7 @@ def grouped_linear_tiled(a: torch.Tensor, w: torch.Tensor, tile_expert: torch.Te
     _need_i32("tile_expert", tile_expert, n_slots // 256)
     rc = library.kernels().mgpt_linear_mfma_grouped(_ptr(a), a.stride(0), _ptr(w), w.stride(0), _ptr(tile_expert),
                                                     _ptr(slot_token), 256, _ptr(out), _dtype_code(out), out.stride(0),
-                                                    n_slots, n_out, k_dim, _stream())
+                                                    n_slots, n_out, k_dim, epilogue, _stream())
     if rc == -2:
         return False
     _check(rc, "linear_mfma_grouped")
@@ -1750,6 +1801,86 @@ def gated_state_chunked(z: torch.Tensor, q_off: int, k_off: int, v_off: int, n_h
         _ptr(a_log), _ptr(skip), _ptr(state), state.stride(0), _ptr(state_slots), _ptr(cu_q), n_req, n_tokens,
         _ptr(positions), _ptr(qkg), _ptr(out), out.stride(0), _stream())
     _check(rc, "gated_state_chunked", 2)
+    return True
+
+
+def _check_delta_args(x, q_off, k_off, v_off, z, b_off, a_off, n_head, n_group, head_dim, value_dim, dt_bias, a_log,
+                      state, state_slots, cu_q, n_req, positions, out, n_tokens):
+    _need_cuda(x, z, dt_bias, a_log, state, state_slots, cu_q, positions, out)
+    _rows_2d("delta_state x", x, n_tokens)
+    _rows_2d("delta_state z", z, n_tokens)
+    _need(x.dtype == z.dtype, "delta_state: x and z must share a dtype")
+    _need(n_head % n_group == 0, "delta_state: heads must be a multiple of groups")
+    _need(min(q_off, k_off, v_off) >= 0 and x.shape[1] >= max(q_off, k_off) + n_group * head_dim
+          and x.shape[1] >= v_off + n_head * value_dim, "delta_state: x is too narrow")
+    _need(min(b_off, a_off) >= 0 and z.shape[1] >= max(b_off, a_off) + n_head, "delta_state: z is too narrow")
+    _need(0 < head_dim <= 256 and 0 < value_dim <= 256, "delta_state takes head sizes up to 256")
+    _need(out.dim() == 2 and out.stride(1) == 1 and out.shape[0] >= n_tokens and out.shape[1] >= n_head * value_dim,
+          "delta_state: out must be rows of all heads' values")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+          and state.shape[1] == n_head * head_dim * value_dim, "delta_state: state must be float32 rows of heads * dim * vdim")
+    for name, t in (("dt_bias", dt_bias), ("a_log", a_log)):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n_head, f"delta_state: {name} must be float32 [heads]")
+    _need_i32("state_slots", state_slots, n_req)
+    _need_i32("cu_q", cu_q, n_req + 1)
+    _need_i32("positions", positions, n_tokens)
+
+
+def delta_state(x: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Tensor, b_off: int, a_off: int, n_head: int,
+                n_group: int, head_dim: int, value_dim: int, dt_bias: torch.Tensor, a_log: torch.Tensor,
+                state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor, n_req: int, positions: torch.Tensor,
+                out: torch.Tensor, n_tokens: int, q_scale: float = 1.0, gate_off: int = -1,
+                norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0) -> None:
+    """The gated delta rule, token by token: per request and head the state S [head_dim, value_dim] (float32, in the
+    request's slot of `state`, zero before position 0) goes over the request's tokens of this step: S = g S,
+    u = beta (v - S^T k), S = S + k u^T, o = S^T q.  q and k (n_group groups that heads share in turn; made unit
+    vectors here, q also times q_scale) and v (per head) are columns of x's rows; beta = sigmoid(z[b_off + h]),
+    g = exp(-exp(a_log[h]) softplus(z[a_off + h] + dt_bias[h])).  gate_off < 0: out receives o as float32;
+    otherwise each head's o divided by its root mean square (eps), times norm_weight [value_dim], times silu of
+    z's columns from gate_off on, in x's dtype.  state: float32 rows (a view of a pool's columns will do)."""
+    _check_delta_args(x, q_off, k_off, v_off, z, b_off, a_off, n_head, n_group, head_dim, value_dim, dt_bias, a_log, state,
+                      state_slots, cu_q, n_req, positions, out, n_tokens)
+    if gate_off >= 0:
+        _need_cuda(norm_weight)
+        _need(out.dtype == x.dtype, "delta_state: gated outputs have x's dtype")
+        _need(z.shape[1] >= gate_off + n_head * value_dim, "delta_state: z has no room for the gates")
+        _need(norm_weight is not None and norm_weight.dtype == torch.float32 and norm_weight.is_contiguous()
+              and norm_weight.numel() == value_dim, "delta_state: norm_weight must be float32 [value_dim]")
+    else:
+        _need(out.dtype == torch.float32, "delta_state: outputs without the gate are float32")
+    rc = library.kernels().mgpt_delta_state(
+        _ptr(x), _dtype_code(x), x.stride(0), q_off, k_off, v_off, _ptr(z), z.stride(0), b_off, a_off, gate_off, n_head,
+        n_group, head_dim, value_dim, float(q_scale), _ptr(dt_bias), _ptr(a_log), _ptr(norm_weight), float(eps), _ptr(state),
+        state.stride(0), _ptr(state_slots), _ptr(cu_q), n_req, _ptr(positions), _ptr(out), out.stride(0), _stream())
+    _check(rc, "delta_state")
+
+
+def delta_image_floats(n_tokens: int, n_req: int, n_head: int, head_dim: int) -> int:
+    """Floats of scratch that delta_state_chunked needs for a step of these sizes; 0 if it does not take them."""
+    return int(library.kernels().mgpt_delta_image_floats(n_tokens, n_req, n_head, head_dim))
+
+
+def delta_state_chunked(x: torch.Tensor, q_off: int, k_off: int, v_off: int, z: torch.Tensor, b_off: int, a_off: int,
+                        n_head: int, n_group: int, head_dim: int, value_dim: int, dt_bias: torch.Tensor,
+                        a_log: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor, n_req: int,
+                        positions: torch.Tensor, images: torch.Tensor, out: torch.Tensor, n_tokens: int,
+                        q_scale: float = 1.0) -> bool:
+    """delta_state without the gate for steps with prompt portions: the recurrence 32 tokens at a time as float32
+    matrix products.  images: dense float32 scratch of delta_image_floats(...) elements; out: float32 rows.  False,
+    with nothing launched, for head sizes beyond CHUNKED_STATE_MAX_DIM."""
+    if head_dim > CHUNKED_STATE_MAX_DIM:
+        return False
+    _check_delta_args(x, q_off, k_off, v_off, z, b_off, a_off, n_head, n_group, head_dim, value_dim, dt_bias, a_log, state,
+                      state_slots, cu_q, n_req, positions, out, n_tokens)
+    _need(out.dtype == torch.float32, "delta_state: outputs without the gate are float32")
+    _need_cuda(images)
+    _need(images.dtype == torch.float32 and images.is_contiguous() and images.data_ptr() % 16 == 0
+          and images.numel() >= delta_image_floats(n_tokens, n_req, n_head, head_dim), "delta_state_chunked: images is too small")
+    rc = library.kernels().mgpt_delta_state_chunked(
+        _ptr(x), _dtype_code(x), x.stride(0), q_off, k_off, v_off, _ptr(z), z.stride(0), b_off, a_off, n_head, n_group,
+        head_dim, value_dim, float(q_scale), _ptr(dt_bias), _ptr(a_log), _ptr(state), state.stride(0), _ptr(state_slots),
+        _ptr(cu_q), n_req, n_tokens, _ptr(positions), _ptr(images), images.numel(), _ptr(out), out.stride(0), _stream())
+    _check(rc, "delta_state_chunked", 2)
     return True
 
 

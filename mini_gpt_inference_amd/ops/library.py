@@ -39,7 +39,7 @@ def kernels() -> ctypes.CDLL:
         lib.mgpt_layernorm.argtypes = [P, P, P, P, P, I, I, F, I, P]
         lib.mgpt_linear_generic.argtypes = [P, I, L, P, I, P, P, I, L, I, I, I, I, P]
         lib.mgpt_kv_write.argtypes = [P, I, L, I, I, P, P, P, I, I, I, I, P]
-        lib.mgpt_paged_attention_generic.argtypes = [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, P, F, P, L, I, P, P]
+        lib.mgpt_paged_attention_generic.argtypes = [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, P, F, P, L, I, P, I, P, I, P]
         lib.mgpt_sample.argtypes = [P, L, I, I, I, P, P, P, P, P, c_ulonglong, P, P, P, I, P]
         lib.mgpt_sample_advance.argtypes = [P, L, I, I, I, P, P, P, P, P, c_ulonglong, P,
                                             P, P, P, P, P, P, P, I, I, I, I, P, P, I, I, P, P, I, P]
@@ -127,16 +127,16 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_linear_skinny_partials": [I, I, I, I, I],
         "mgpt_linear_skinny_row_groups": [I, I, I],
         "mgpt_fold_layernorm": [P, P, P, P, P, P, P, I, I, P],
-        "mgpt_paged_attention_split_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, P],
-        "mgpt_paged_attention_split_fast_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, P],
-        "mgpt_paged_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, P],
+        "mgpt_paged_attention_split_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P],
+        "mgpt_paged_attention_split_fast_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P],
+        "mgpt_paged_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P],
         "mgpt_linear_mfma": [P, L, P, P, P, I, L, I, I, I, I, P, L, P],
         "mgpt_linear_mfma_xielu": [P, L, P, P, P, L, I, I, I, P, P, L, P],
         "mgpt_linear_mfma_shape": [I, I, P, L, P, P, P, I, L, I, I, I, I, P, L, P],
         "mgpt_linear_mfma_partials": [I, I, I, I],
         "mgpt_linear_mfma_parts": [P, L, P, P, P, L, I, I, I, P],
         "mgpt_linear_mfma_qkv": [P, L, P, P, P, L, I, I, I, P, P, P, I, I, I, I, I, I, P],
-        "mgpt_prefill_attention_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, P],
+        "mgpt_prefill_attention_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P],
         # a residual that is still a sum: base, partials, n_parts, part_stride, token table, position table, ids, positions
         "mgpt_fused_attention_decode": [P, P, I, L, P, P, P, P, P, P, P, P, F, P, P, P, P, P, L, P, P, P, P, I, P, P,
                                         I, I, I, I, I, I, F, P],
@@ -149,7 +149,7 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_residual_settle": [P, P, I, L, P, P, P, P, P, I, I, P],
         "mgpt_fused_parts_limit": [I],
         # several residual streams, scaled embedding, soft-capped logits
-        "mgpt_embed_scaled": [P, P, P, I, I, I, F, I, P],
+        "mgpt_embed_scaled": [P, P, P, P, P, I, I, I, F, I, P],
         "mgpt_streams_read": [P, P, P, P, I, I, I, P],
         "mgpt_streams_write": [P, P, P, P, I, I, I, P],
         "mgpt_streams_step": [P, P, P, P, I, I, P, P, P, P, F, P, I, I, I, I, P],
@@ -174,22 +174,27 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_decay_state_chunked": [P, I, L, I, I, I, I, I, I, I, P, P, I, F, P, P, P, P, I, I, P, P, L, P],
         "mgpt_expert_route": [P, P, P, I, I, I, P, P, P, P, I, I, I, P],
         "mgpt_gather_rows": [P, L, P, P, L, I, I, P],
-        "mgpt_linear_mfma_grouped": [P, L, P, L, P, P, I, P, I, L, I, I, I, P],
-        "mgpt_grouped_linear": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, P],
-        "mgpt_grouped_linear_mfma": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, P],
-        "mgpt_expert_combine": [P, P, P, P, I, I, I, F, P],
-        "mgpt_router_topk": [P, I, L, P, I, P, I, I, I, I, I, P, P, P],
+        "mgpt_linear_mfma_grouped": [P, L, P, L, P, P, I, P, I, L, I, I, I, I, P],
+        "mgpt_grouped_linear": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, I, P],
+        "mgpt_grouped_linear_mfma": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, P],
+        "mgpt_expert_combine": [P, P, P, P, I, I, I, F, P, P, P, P],
+        "mgpt_router_topk": [P, I, L, P, I, P, I, I, I, I, I, P, P, P, I, I, I, F, P, P, P],
         "mgpt_gather_scale_rows": [P, I, L, P, P, P, P, L, I, I, P],
         # a state with a decay made from the token, short convolutions
         "mgpt_gated_state": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, P, P, L, P],
         "mgpt_gated_state_chunked": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, I, P, P, P, L, P],
+        # the gated delta rule
+        "mgpt_delta_state": [P, I, L, I, I, I, P, L, I, I, I, I, I, I, I, F, P, P, P, F, P, L, P, P, I, P, P, L, P],
+        "mgpt_delta_image_floats": [I, I, I, I],
+        "mgpt_delta_state_chunked": [P, I, L, I, I, I, P, L, I, I, I, I, I, I, F, P, P, P, L, P, P, I, I, P, P, L, P, L, P],
         "mgpt_short_conv": [P, I, L, I, P, P, I, P, L, P, P, P, P, I, P, I, L, I, I, I, I, P],
     }
     for name, argtypes in table.items():
         fn = getattr(lib, name, None)
         if fn is not None:
             fn.argtypes = argtypes
-            fn.restype = L if name in ("mgpt_linear_skinny_partials", "mgpt_linear_mfma_partials") else I
+            fn.restype = L if name in ("mgpt_linear_skinny_partials", "mgpt_linear_mfma_partials",
+                                              "mgpt_delta_image_floats") else I
 
 
 def host() -> ctypes.CDLL:
@@ -201,7 +206,7 @@ def host() -> ctypes.CDLL:
         IP = POINTER(c_int)
         lib.mgpt_host_last_error.restype = c_char_p
         lib.mgpt_cache_create.restype = P
-        lib.mgpt_cache_create.argtypes = [I, IP, IP, IP, IP, I]
+        lib.mgpt_cache_create.argtypes = [I, IP, IP, IP, IP, IP, I]
         lib.mgpt_cache_destroy.argtypes = [P]
         lib.mgpt_cache_destroy.restype = None
         for name, args in {

@@ -47,6 +47,8 @@ class KVNeed:
     keep_first: int = 0   # with a window: every query also sees the first keep_first positions of its request
     state_numel: int = 0  # float32 values per request that the mixer keeps beside its pages (the last inputs of a
                           # short convolution in front of its keys, say); 0: none
+    chunked: bool = False   # with a window: it is the size of chunks counted from position 0, and a query sees the
+                            # keys of its own chunk up to its own
 
 
 @dataclass(frozen=True)

@@ -25,7 +25,7 @@ class TokenEmbedding(Part):
 
     def __init__(self, vocab_size: int, width: int, scale: float = 1.0, copies: int = 1) -> None:
         self.vocab_size, self.width = int(vocab_size), int(width)
-        # x0 = table row * scale, written `copies` times side by side (one per residual stream)
+        # x0 = table row * scale (+ the position's row, not scaled), written `copies` times side by side (one per residual stream)
         self.scale, self.copies = float(scale), int(copies)
         self.weight: Optional[torch.Tensor] = None
 
@@ -35,9 +35,8 @@ class TokenEmbedding(Part):
     def forward(self, ctx: StepContext, position: PositionEncoding, x: torch.Tensor) -> None:
         table = position.embedding_table()
         if self.scale != 1.0 or self.copies != 1:
-            if table is not None:
-                raise ValueError("a scaled or copied embedding takes no position table")
-            kernels.embed_scaled(ctx.token_ids, self.weight, x, ctx.n_rows, self.scale, self.copies)
+            kernels.embed_scaled(ctx.token_ids, self.weight, x, ctx.n_rows, self.scale, self.copies,
+                                 positions=ctx.positions if table is not None else None, pos_table=table)
             return
         if (residual.usable(ctx, self.width, 1) and self.weight.dtype == torch.bfloat16
                 and (table is None or table.dtype == torch.bfloat16)):

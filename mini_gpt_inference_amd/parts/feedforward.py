@@ -12,7 +12,9 @@ from .base import MATRIX, Part, StepContext, TABLE, VECTOR, WeightRequest, regis
 
 # activations of the dense feed-forward: an epilogue of the product kernels, or (None) one that brings coefficients
 # (ops.linear.linear_xielu: the tiled kernel's epilogue, elsewhere a kernel of its own behind the product)
-_ACTIVATIONS = {"gelu_tanh": kernels.EPI_GELU, "xielu": None}
+_ACTIVATIONS = {"gelu_tanh": kernels.EPI_GELU, "relu2": kernels.EPI_RELU2, "xielu": None}
+# activations of experts without a gate: epilogues of the grouped products as well
+_EXPERT_ACTIVATIONS = {"relu2": kernels.EPI_RELU2}
 
 
 class FeedForward(Part):
@@ -28,7 +30,8 @@ class DenseMLP(FeedForward):
     """u = h Wfc^T (+ b); g = 0.5 u (1 + tanh(sqrt(2/pi)(u + 0.044715 u^3))); m = g Wproj^T (+ b)
     (reference: src/minigpt_infer/model.py:96-101; there the hidden size is 4*n_embd, here it is
     a parameter).  With activation "xielu" g is instead, from two stored numbers (p, q) (the tensor `act`),
-    softplus(p) u^2 + u / 2 for u > 0 and (1/2 + softplus(q)) (exp(u) - 1 - u) + u / 2 for u <= 0."""
+    softplus(p) u^2 + u / 2 for u > 0 and (1/2 + softplus(q)) (exp(u) - 1 - u) + u / 2 for u <= 0; with "relu2"
+    it is max(u, 0)^2."""
 
     graph_safe = True
 
@@ -169,16 +172,21 @@ class TableExperts(FeedForward):
         self.vocab_size, self.shared_hidden = int(vocab_size), int(shared_hidden)
         if not 0 < self.top <= self.n_experts <= kernels.MAX_EXPERTS:
             raise ValueError(f"top {self.top} of {self.n_experts} experts: need 0 < top <= experts <= {kernels.MAX_EXPERTS}")
+        # an expert is a gated unit; without the gate (a subclass says so) it is down(act(up h)) with this activation
+        self.gated, self.epilogue = True, kernels.EPI_NONE
+        self.gates_shared = False       # the shared expert's output is multiplied by a number per token
         self.in_weights = self.down_weights = self.shared_in_weight = None
 
     def weight_requests(self) -> Dict[str, WeightRequest]:
         req = {"table": WeightRequest((self.vocab_size, self.top), TABLE)}
         for e in range(self.n_experts):
-            req[f"e{e}_gate"] = WeightRequest((self.hidden, self.width), MATRIX)
+            if self.gated:
+                req[f"e{e}_gate"] = WeightRequest((self.hidden, self.width), MATRIX)
             req[f"e{e}_up"] = WeightRequest((self.hidden, self.width), MATRIX)
             req[f"e{e}_down"] = WeightRequest((self.width, self.hidden), MATRIX)
         if self.shared_hidden:
-            req["shared_gate"] = WeightRequest((self.shared_hidden, self.width), MATRIX)
+            if self.gated:
+                req["shared_gate"] = WeightRequest((self.shared_hidden, self.width), MATRIX)
             req["shared_up"] = WeightRequest((self.shared_hidden, self.width), MATRIX)
             req["shared_down"] = WeightRequest((self.width, self.shared_hidden), MATRIX)
         return req
@@ -191,22 +199,32 @@ class TableExperts(FeedForward):
 
     def _bind_experts(self, tensors):
         f, views = self.hidden, {}
-        # [experts, 2 * hidden, width] and [experts, width, hidden]: an expert's matrices lie together
-        self.in_weights = torch.stack([torch.cat([tensors[f"e{e}_gate"], tensors[f"e{e}_up"]], dim=0)
-                                       for e in range(self.n_experts)]).contiguous()
+        # [experts, 2 * hidden, width] (without gates [experts, hidden, width]) and [experts, width, hidden]: an
+        # expert's matrices lie together
+        if self.gated:
+            self.in_weights = torch.stack([torch.cat([tensors[f"e{e}_gate"], tensors[f"e{e}_up"]], dim=0)
+                                           for e in range(self.n_experts)]).contiguous()
+        else:
+            self.in_weights = torch.stack([tensors[f"e{e}_up"] for e in range(self.n_experts)]).contiguous()
         self.down_weights = torch.stack([tensors[f"e{e}_down"] for e in range(self.n_experts)]).contiguous()
         for e in range(self.n_experts):
-            views[f"e{e}_gate"], views[f"e{e}_up"] = self.in_weights[e, :f], self.in_weights[e, f:]
+            if self.gated:
+                views[f"e{e}_gate"], views[f"e{e}_up"] = self.in_weights[e, :f], self.in_weights[e, f:]
+            else:
+                views[f"e{e}_up"] = self.in_weights[e]
             views[f"e{e}_down"] = self.down_weights[e]
         if self.shared_hidden:
             self.shared_down = tensors["shared_down"]
-            self.shared_in_weight, shared = _stack_gate_up(self, tensors, "shared_gate", "shared_up")
-            views.update(shared)
+            if self.gated:
+                self.shared_in_weight, shared = _stack_gate_up(self, tensors, "shared_gate", "shared_up")
+                views.update(shared)
+            else:
+                self.shared_in_weight = tensors["shared_up"]
         return views
 
     def token_matrix_elements(self) -> int:
         """Matrix elements one token goes through: its `top` experts and the shared one."""
-        return 3 * self.width * (self.top * self.hidden + self.shared_hidden)
+        return (3 if self.gated else 2) * self.width * (self.top * self.hidden + self.shared_hidden)
 
     def forward_add(self, ctx: StepContext, h, x: torch.Tensor) -> None:
         plain_residual(ctx, h, x)
@@ -214,13 +232,14 @@ class TableExperts(FeedForward):
         self._experts_add(ctx, hn, x, ctx.n_rows, ctx.token_ids, self.table, None, 1.0 / self.top)
 
     def _experts_add(self, ctx: StepContext, hn: torch.Tensor, x: torch.Tensor, n: int, ids, table: torch.Tensor,
-                     pair_weight, combine_weight: float) -> None:
+                     pair_weight, combine_weight: float, out_weight=None, shared_gate=None) -> None:
         """x += combine_weight * sum over token n's experts (row ids[n] of the table, or row n without ids) of
-        expert(w h), w = pair_weight[n][choice] (None: 1), plus the shared expert."""
+        v expert(w h), w = pair_weight[n][choice] and v = out_weight[n][choice] (None: 1), plus the shared expert
+        (times shared_gate[n])."""
         ws = ctx.workspace
         fast = not ctx.exact and ctx.dtype == torch.bfloat16
         if fast and n * self.top >= self.TILED_FROM_PAIRS and self.width % 16 == 0 and self.hidden % 16 == 0 \
-                and self._forward_tiled(ctx, hn, x, n, ids, table, pair_weight, combine_weight):
+                and self._forward_tiled(ctx, hn, x, n, ids, table, pair_weight, combine_weight, out_weight, shared_gate):
             return
         # tiles of 64 slots for the MFMA kernel of few rows, of 16 for the general one, and for the MFMA kernel too
         # where an expert gets 16 pairs at most on average (a decode step): a tile's empty slots are loaded and
@@ -231,22 +250,47 @@ class TableExperts(FeedForward):
         slot_pair = ws.get("expert_slot_pair", slots, 1, torch.int32).view(-1)
         tile_expert = ws.get("expert_tile", slots // tile, 1, torch.int32).view(-1)
         kernels.expert_route(ids, ctx.q_req, table, n, self.n_experts, slot_token, slot_pair, tile_expert, tile)
-        z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype)
+        act = ws.get("expert_act", slots, self.hidden, ctx.dtype)
+        z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype) if self.gated else act
         if pair_weight is None:
-            kernels.grouped_linear(hn, slot_token, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast)
+            kernels.grouped_linear(hn, slot_token, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast,
+                                   self.epilogue)
         else:
             # the weight multiplies the expert's input: every pair's row is made first, scaled, in the experts' order
             rows = ws.get("expert_rows", slots, self.width, ctx.dtype)
             kernels.gather_scale_rows(hn, slot_token, slot_pair, pair_weight, rows, slots)
-            kernels.grouped_linear(rows, None, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast)
-        act = ws.get("expert_act", slots, self.hidden, ctx.dtype)
-        kernels.gated_unit(z, act, slots, self.hidden, fast=not ctx.exact)
+            kernels.grouped_linear(rows, None, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast,
+                                   self.epilogue)
+        if self.gated:
+            kernels.gated_unit(z, act, slots, self.hidden, fast=not ctx.exact)
         pair_out = ws.get("expert_pair_out", n * self.top, self.width, torch.float32)
         kernels.grouped_linear(act, None, self.down_weights, tile_expert, slot_token, pair_out, slot_pair, slots,
                                tile, fast)
-        if self.shared_hidden:
+        extra = self._shared_add(ctx, hn, x, n)
+        kernels.expert_combine(pair_out, x, n, self.top, combine_weight, q_req=ctx.q_req, pair_weight=out_weight,
+                               extra=extra, extra_gate=shared_gate)
+
+    def _shared_add(self, ctx: StepContext, hn: torch.Tensor, x: torch.Tensor, n: int):
+        """The shared expert: added into x (returns None), or, if a number per token multiplies it, as rows of its own
+        that the kernel which adds up the experts' outputs takes along."""
+        if not self.shared_hidden:
+            return None
+        if self.gated and not self.gates_shared:
             _gated(ctx, hn, self.shared_in_weight, self.shared_down, x, n, self.shared_hidden)
-        kernels.expert_combine(pair_out, x, n, self.top, combine_weight, q_req=ctx.q_req)
+            return None
+        act = ctx.workspace.get("shared_act", n, self.shared_hidden, ctx.dtype)
+        if self.gated:
+            z = ctx.workspace.get("shared_z", n, 2 * self.shared_hidden, ctx.dtype)
+            linear(ctx, hn, self.shared_in_weight, None, z, n)
+            kernels.gated_unit(z, act, n, self.shared_hidden, fast=not ctx.exact)
+        else:
+            linear(ctx, hn, self.shared_in_weight, None, act, n, self.epilogue)
+        if not self.gates_shared:
+            linear_add(ctx, act, self.shared_down, None, x, n)
+            return None
+        rows = ctx.workspace.get("shared_out", n, self.width, torch.float32)
+        linear(ctx, act, self.shared_down, None, rows, n)
+        return rows
 
     # From this many (token, choice) pairs on, the experts' products go through the tiled MFMA kernel
     # of the dense layers: the pairs' rows are copied into the experts' order first, every expert's
@@ -256,7 +300,7 @@ class TableExperts(FeedForward):
     TILED_FROM_PAIRS = 512
 
     def _forward_tiled(self, ctx: StepContext, hn: torch.Tensor, x: torch.Tensor, n: int, ids, table: torch.Tensor,
-                       pair_weight, combine_weight: float) -> bool:
+                       pair_weight, combine_weight: float, out_weight=None, shared_gate=None) -> bool:
         ws, tile = ctx.workspace, 256
         slots = kernels.expert_slots(n, self.top, self.n_experts, tile)
         slot_token = ws.get("expert_slot_token", slots, 1, torch.int32).view(-1)
@@ -272,26 +316,35 @@ class TableExperts(FeedForward):
             kernels.gather_scale_rows(hn, slot_token, slot_pair, pair_weight, sorted_rows, slots)
         elif not kernels.gather_rows(hn, slot_token, sorted_rows, slots):
             return False
-        z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype)
-        if not kernels.grouped_linear_tiled(sorted_rows, self.in_weights, tile_expert, slot_token, z, slots):
-            return False
         act = ws.get("expert_act", slots, self.hidden, ctx.dtype)
-        kernels.gated_unit(z, act, slots, self.hidden, fast=True)
+        z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype) if self.gated else act
+        if not kernels.grouped_linear_tiled(sorted_rows, self.in_weights, tile_expert, slot_token, z, slots, self.epilogue):
+            return False
+        if self.gated:
+            kernels.gated_unit(z, act, slots, self.hidden, fast=True)
         slot_out = ws.get("expert_slot_out", slots, self.width, torch.float32)
         if not kernels.grouped_linear_tiled(act, self.down_weights, tile_expert, slot_token, slot_out, slots):
             return False
-        if self.shared_hidden:
-            _gated(ctx, hn, self.shared_in_weight, self.shared_down, x, n, self.shared_hidden)
-        kernels.expert_combine(slot_out, x, n, self.top, combine_weight, pair_slot=pair_slot, q_req=ctx.q_req)
+        extra = self._shared_add(ctx, hn, x, n)
+        kernels.expert_combine(slot_out, x, n, self.top, combine_weight, pair_slot=pair_slot, q_req=ctx.q_req,
+                               pair_weight=out_weight, extra=extra, extra_gate=shared_gate)
         return True
 
 
 @register_feed_forward("routed_experts")
 class RoutedExperts(TableExperts):
-    """A mixture of gated feed-forwards chosen by a router: scores s = sigmoid(h Wr^T), computed in
+    """A mixture of feed-forwards chosen by a router: scores s = sigmoid(h Wr^T), computed in
     float32; a token uses the `top` experts with the largest scores; the output is the sum over them of
     expert_e(s_e h), expert(u) = (silu(u Wgate^T) * (u Wup^T)) Wdown^T: the score multiplies the expert's
     input and is not renormalised.  A shared expert (shared_hidden > 0) takes every token unweighted.
+
+    Options: `activation` "relu2": experts without a gate, expert(u) = max(u Wup^T, 0)^2 Wdown^T; `weight_on`
+    "output": the weight multiplies the expert's output; `correction`: a number per expert is added to the scores
+    that the choice goes by (the weights are the scores without it); `groups` = (count, keep): the experts form
+    `count` equal groups of neighbours and only those of the `keep` groups whose two largest choice scores have the
+    largest sums can be chosen; `normalise`: the weights are the chosen scores over (their sum + 1e-20); `scale`
+    multiplies every weight; `shared_gate`: the shared expert's output is multiplied by sigmoid(h . w), one number per
+    token (the router kernel computes it, as one more row of its matrix).
 
     The router kernel writes the step's own table of experts and scores; from there on the experts run as
     those chosen by a stored table do."""
@@ -300,20 +353,43 @@ class RoutedExperts(TableExperts):
     plan_safe = True
 
     def __init__(self, width: int, hidden: int, n_experts: int, top: int, shared_hidden: int = 0,
-                 score: str = "sigmoid") -> None:
+                 score: str = "sigmoid", activation: str = "silu", weight_on: str = "input", correction: bool = False,
+                 groups=None, normalise: bool = False, scale: float = 1.0, shared_gate: bool = False) -> None:
         super().__init__(width, hidden, n_experts, top, vocab_size=0, shared_hidden=shared_hidden)
         if score not in kernels.ROUTER_SCORES:
             raise ValueError(f"router score {score!r} is none of {sorted(kernels.ROUTER_SCORES)}")
         self.score = score
+        if activation != "silu" and activation not in _EXPERT_ACTIVATIONS:
+            raise ValueError(f"experts' activation {activation!r} is neither 'silu' (gated) nor one of {sorted(_EXPERT_ACTIVATIONS)}")
+        self.gated = activation == "silu"
+        self.epilogue = kernels.EPI_NONE if self.gated else _EXPERT_ACTIVATIONS[activation]
+        if weight_on not in ("input", "output"):
+            raise ValueError(f"weight_on {weight_on!r} is neither 'input' nor 'output'")
+        self.weighs_output, self.has_correction = weight_on == "output", bool(correction)
+        self.groups = None if groups is None else (int(groups[0]), int(groups[1]))
+        if self.groups is not None:
+            count, keep = self.groups
+            if not 0 < keep <= count or self.n_experts % count or self.top > keep * (self.n_experts // count):
+                raise ValueError(f"{self.n_experts} experts in {count} groups of which {keep} stay: need equal groups and "
+                                 f"{self.top} experts left to choose")
+        self.normalise, self.scale = bool(normalise), float(scale)
+        self.gates_shared = bool(shared_gate) and self.shared_hidden > 0
+        self.correction = self.shared_gate_weight = None
 
     def weight_requests(self) -> Dict[str, WeightRequest]:
         req = super().weight_requests()
         del req["table"]
         req["router_weight"] = WeightRequest((self.n_experts, self.width), MATRIX)
+        if self.has_correction:
+            req["correction"] = WeightRequest((self.n_experts,), VECTOR)
+        if self.gates_shared:
+            req["shared_gate_weight"] = WeightRequest((1, self.width), MATRIX)
         return req
 
     def bind(self, tensors):
         self.router_weight = tensors["router_weight"]
+        self.correction = tensors.get("correction")
+        self.shared_gate_weight = tensors.get("shared_gate_weight")
         return self._bind_experts(tensors)
 
     def token_matrix_elements(self) -> int:
@@ -325,5 +401,10 @@ class RoutedExperts(TableExperts):
         hn = as_tensor(ctx, h)
         chosen = ws.get("router_chosen", n, self.top, torch.int32)
         weight = ws.get("router_weight", n, self.top, torch.float32)
-        kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, q_req=ctx.q_req, score=self.score)
-        self._experts_add(ctx, hn, x, n, None, chosen, weight.view(-1), 1.0)
+        gate = ws.get("router_shared_gate", n, 1, torch.float32).view(-1) if self.gates_shared else None
+        kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, q_req=ctx.q_req, score=self.score,
+                            correction=self.correction, groups=self.groups, normalise=self.normalise, scale=self.scale,
+                            extra=self.shared_gate_weight, extra_out=gate)
+        weight = weight.view(-1)
+        self._experts_add(ctx, hn, x, n, None, chosen, None if self.weighs_output else weight, 1.0,
+                          out_weight=weight if self.weighs_output else None, shared_gate=gate)

@@ -2,7 +2,8 @@
 
 from __future__ import annotations
 
-from typing import Dict, Optional, Union
+import math
+from typing import Dict, List, Optional, Union
 
 import torch
 
@@ -304,6 +305,23 @@ def _own_rotation(rotary: Optional[dict]) -> Optional[PositionEncoding]:
     return part
 
 
+def distance_buckets(n_buckets: int, bias_max: int) -> List[int]:
+    """The bucket of every distance 0, 1, .. up to the first one in the last bucket, which holds all beyond it.  With
+    h = n_buckets / 2: bucket n for n < h, then min(n_buckets - 1, h + floor(ln(n / h) / ln(bias_max / h) h)): one
+    bucket a distance nearby, buckets that widen by a factor further away."""
+    half = n_buckets // 2
+    if n_buckets < 2 or n_buckets % 2 or bias_max <= half:
+        raise ValueError(f"{n_buckets} distance buckets up to {bias_max}: need an even number, and bias_max beyond half of it")
+    out: List[int] = []
+    while not out or out[-1] < n_buckets - 1:
+        n = len(out)
+        far = n_buckets - half
+        # (1e-9: a quotient of logarithms that is an integer may come out a rounding below it)
+        step = 0.0 if n < half else math.log(n / half) / math.log(bias_max / half) * far
+        out.append(n if n < half else min(n_buckets - 1, half + math.floor(step + 1e-9)))
+    return out
+
+
 @register_mixer("gated_attention")
 class GatedAttention(Mixer):
     """Causal softmax attention over the paged cache with grouped key/value heads, a query/key size
@@ -327,7 +345,10 @@ class GatedAttention(Mixer):
     weights as long as the projection; `values_from_keys`: there is no Wv, a key head's values are its keys as
     projected (before norm and rotation), so E = D; `score_bias`: no softmax, a visible key's weight is
     sigmoid(score + b_a) with a number per head (the tensor `score_bias`), not normalised over the keys;
-    `out_bias`: the output projection has a bias.
+    `out_bias`: the output projection has a bias; `sinks`: one more term exp(sink_a) in the softmax's denominator,
+    a number per head with no key and no value; `chunked`: `window` is the size of chunks counted from position 0, and
+    a query sees the keys of its own chunk; `bias_max` = M: the number rel[bucket(i - j)][a] (the tensor `rel`
+    [B, H]) is added to the scaled score of query i and key j, with the buckets of distance_buckets(B, M).
 
     The cache keeps keys and values in pages of one head size, so both are laid out with
     max(D, E) channels a head (rounded up to what the bfloat16 attention kernels take), the
@@ -341,7 +362,8 @@ class GatedAttention(Mixer):
                  softcap: float = 0.0, head_gate: bool = False, value_mix: Optional[str] = None,
                  share: str = "values", conv_taps: int = 0, window: int = 0, keep_first: int = 0,
                  qk_norm_weights: Optional[str] = None, values_from_keys: bool = False, score_bias: bool = False,
-                 out_bias: bool = False) -> None:
+                 out_bias: bool = False, sinks: bool = False, chunked: bool = False,
+                 bias_max: Optional[int] = None) -> None:
         self.width, self.n_head, self.n_kv_head = int(width), int(n_head), int(n_kv_head)
         self.head_dim, self.value_dim, self.scale = int(head_dim), int(value_dim), float(scale)
         self.has_bias, self.has_gate = bool(bias), bool(head_gate)
@@ -369,6 +391,12 @@ class GatedAttention(Mixer):
             raise ValueError("values that are the keys have the keys' size, and are neither mixed nor convolved")
         if self.has_score_bias and self.softcap > 0.0:
             raise ValueError("sigmoid weights take no score cap")
+        self.has_sinks, self.chunked = bool(sinks), bool(chunked and self.window)
+        self.bias_max = None if bias_max is None else int(bias_max)
+        if self.has_score_bias and (self.has_sinks or self.bias_max is not None):
+            raise ValueError("sigmoid weights take neither sinks nor numbers by distance")
+        if self.bias_max is not None and self.softcap > 0.0:
+            raise ValueError("numbers by distance go with no score cap")
         size = max(self.head_dim, self.value_dim)
         self.head_stride = -(-size // 32) * 32 if size <= 128 else -(-size // 8) * 8
         if self.head_stride > 512:
@@ -378,7 +406,7 @@ class GatedAttention(Mixer):
         self.v_off = self.k_off + self.n_kv_head * s
         self.g_off = self.v_off + (0 if self.values_from_keys else self.n_kv_head * s)
         self.in_rows = -(-(self.g_off + (self.n_head if self.has_gate else 0)) // 16) * 16
-        self.in_weight = self.in_bias = self.out_padded = self.conv_weight = None
+        self.in_weight = self.in_bias = self.out_padded = self.conv_weight = self.dist_bias = None
 
     def weight_requests(self) -> Dict[str, WeightRequest]:
         H, G, D, E, W = self.n_head, self.n_kv_head, self.head_dim, self.value_dim, self.width
@@ -393,6 +421,10 @@ class GatedAttention(Mixer):
             req["score_bias"] = WeightRequest((H,), VECTOR)
         if self.has_out_bias:
             req["out_bias"] = WeightRequest((W,), VECTOR)
+        if self.has_sinks:
+            req["sink"] = WeightRequest((H,), VECTOR)
+        if self.bias_max is not None:
+            req["rel"] = WeightRequest((-1, H), VECTOR)      # (the stored table says how many buckets there are)
         if self.conv_taps > 1:
             J = self.conv_taps
             req.update(q_conv=WeightRequest((H * D, J), VECTOR), k_conv=WeightRequest((G * D, J), VECTOR),
@@ -442,6 +474,11 @@ class GatedAttention(Mixer):
                                           ("v_conv", self.v_off, G, E)):
                 taps[at:at + heads * s].view(heads, s, -1)[:, :size].copy_(tensors[name].view(heads, size, -1))
             self.conv_weight = taps
+        if self.bias_max is not None:
+            # bucket by bucket to distance by distance, head by head: what the attention kernels read
+            rel = tensors["rel"]
+            rows = torch.tensor(distance_buckets(rel.shape[0], self.bias_max), device=rel.device)
+            self.dist_bias = rel[rows].t().contiguous()
         out = tensors["out_weight"]
         padded = torch.zeros((W, H * s), dtype=out.dtype, device=out.device)
         padded.view(W, H, s)[:, :, :E].copy_(out.view(W, H, E))
@@ -452,7 +489,7 @@ class GatedAttention(Mixer):
         return views
 
     def cache_need(self) -> KVNeed:
-        return KVNeed(self.n_kv_head, self.head_stride, self.window, keep_first=self.keep_first,
+        return KVNeed(self.n_kv_head, self.head_stride, self.window, keep_first=self.keep_first, chunked=self.chunked,
                       state_numel=(self.conv_taps - 1) * self.g_off if self.conv_taps > 1 else 0)
 
     def token_matrix_elements(self) -> int:
@@ -494,7 +531,9 @@ class GatedAttention(Mixer):
         # (the gate per head is applied by the attention kernel as it stores a head's output)
         attention_ops.paged_attention(ctx, z, y, k_pool, v_pool, group, self.n_head, self.scale, self.window,
                                       softcap=self.softcap, gate=gate_rows[:, self.g_off:] if self.has_gate else None,
-                                      keep_first=self.keep_first, score_bias=self.score_bias if self.has_score_bias else None)
+                                      keep_first=self.keep_first, score_bias=self.score_bias if self.has_score_bias else None,
+                                      sinks=self.sink if self.has_sinks else None, chunked=self.chunked,
+                                      dist_bias=self.dist_bias)
         linear_add(ctx, y, self.out_padded, self.out_bias if self.has_out_bias else None, x, n)
 
 
@@ -777,4 +816,114 @@ class StateSpaceMixer(Mixer):
         y = ws.get("state_space_out", n, self.inner, ctx.dtype)
         kernels.rms_norm(sums, self.norm_weight, y, n, self.norm_eps, self.inner // self.norm_groups,
                          groups=self.norm_groups, gate=u, gate_act="silu_first")
+        linear_add(ctx, y, self.out_weight, None, x, n)
+
+
+@register_mixer("gated_delta_rule")
+class GatedDeltaRule(Mixer):
+    """Linear attention whose state, before it takes a token's value in, gives up what it holds under the token's
+    key: no softmax, and instead of a cache one float32 matrix per request and head.
+
+    q = h Wq^T, k = h Wk^T [G, D], v = h Wv^T [H, E]; each of them passes a causal convolution over time, channel
+    by channel (weights [channels, J], the last tap on the current token, zeros before the sequence's start), then
+    silu; q and k are made unit vectors per head, x / sqrt(sum(x^2) + 1e-6), q also times `q_scale`.  Head a reads
+    q and k of group a // (H / G).  beta = sigmoid(h Wb^T), g = exp(-exp(A_log) softplus(h Wa^T + dt_bias)), one
+    number per head each;  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q, S zero before the first token.
+    Each head's o is divided by its root mean square and multiplied by `norm_weight` [E] (one weight for all
+    heads), the heads by silu(h Wg^T); out = y Wo^T, added into the residual.  Kept per request: the state and the
+    convolutions' last J - 1 inputs.  From the unit vectors and the two logits on everything is float32 up to y."""
+
+    graph_safe = True
+    plan_safe = True
+
+    def __init__(self, width: int, n_head: int, n_kv_head: int, head_dim: int, value_dim: int, conv_taps: int,
+                 norm_eps: float, q_scale: Optional[float] = None) -> None:
+        self.width, self.n_head, self.n_group = int(width), int(n_head), int(n_kv_head)
+        self.head_dim, self.value_dim, self.conv_taps = int(head_dim), int(value_dim), int(conv_taps)
+        self.norm_eps = float(norm_eps)
+        self.q_scale = self.head_dim ** -0.5 if q_scale is None else float(q_scale)
+        if self.n_head % self.n_group:
+            raise ValueError("n_head must be a multiple of n_kv_head")
+        if not (0 < self.head_dim <= 256 and 0 < self.value_dim <= 256):
+            raise ValueError("the state kernel takes head sizes up to 256")
+        if not 1 <= self.conv_taps <= kernels.MAX_CONV_TAPS:
+            raise ValueError(f"the convolution takes 1 to {kernels.MAX_CONV_TAPS} taps")
+        self.qk_width, self.v_width = self.n_group * self.head_dim, self.n_head * self.value_dim
+        self.k_off, self.v_off = self.qk_width, 2 * self.qk_width
+        self.conv_width = self.v_off + self.v_width
+        self.g_off = self.conv_width
+        self.b_off = self.g_off + self.v_width
+        self.a_off = self.b_off + self.n_head
+        self.in_rows = -(-(self.a_off + self.n_head) // 16) * 16
+        self.state_numel = self.n_head * self.head_dim * self.value_dim
+        self.conv_numel = (self.conv_taps - 1) * self.conv_width
+        self.in_weight = self.conv_weight = self.head_gain = None
+
+    def weight_requests(self) -> Dict[str, WeightRequest]:
+        H, W, J = self.n_head, self.width, self.conv_taps
+        return {"q_weight": WeightRequest((self.qk_width, W), MATRIX), "k_weight": WeightRequest((self.qk_width, W), MATRIX),
+                "v_weight": WeightRequest((self.v_width, W), MATRIX), "gate_weight": WeightRequest((self.v_width, W), MATRIX),
+                "beta_weight": WeightRequest((H, W), MATRIX), "decay_weight": WeightRequest((H, W), MATRIX),
+                "q_conv": WeightRequest((self.qk_width, J), VECTOR), "k_conv": WeightRequest((self.qk_width, J), VECTOR),
+                "v_conv": WeightRequest((self.v_width, J), VECTOR), "a_log": WeightRequest((H,), VECTOR),
+                "dt_bias": WeightRequest((H,), VECTOR), "norm_weight": WeightRequest((self.value_dim,), VECTOR),
+                "out_weight": WeightRequest((W, self.v_width), MATRIX)}
+
+    def token_matrix_elements(self) -> int:
+        return self.in_weight.numel() + self.out_weight.numel() if self.in_weight is not None else 0
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        names = ["q_weight", "k_weight", "v_weight", "gate_weight", "beta_weight", "decay_weight"]
+        stacked = [tensors[n] for n in names]
+        short = self.in_rows - sum(t.shape[0] for t in stacked)
+        if short:
+            stacked.append(torch.zeros((short, self.width), dtype=stacked[0].dtype, device=stacked[0].device))
+        self.in_weight = torch.cat(stacked, dim=0).contiguous()
+        views, at = {}, 0
+        for n in names:
+            rows = tensors[n].shape[0]
+            views[n] = self.in_weight[at:at + rows]
+            setattr(self, n, views[n])
+            at += rows
+        self.conv_weight = torch.cat([tensors["q_conv"], tensors["k_conv"], tensors["v_conv"]], dim=0).contiguous()
+        self.head_gain = self.norm_weight.repeat(self.n_head).contiguous()    # the heads' one weight, head by head
+        return views
+
+    def cache_need(self) -> StateNeed:
+        return StateNeed(self.state_numel + self.conv_numel)
+
+    def forward_add(self, ctx: StepContext, h, x: torch.Tensor, binding: CacheBinding,
+                    position: PositionEncoding) -> None:
+        if binding.kind != "state":
+            raise ValueError("the gated delta rule needs a state pool")
+        plain_residual(ctx, h, x)
+        n, ws = ctx.n_rows, ctx.workspace
+        n_req = ctx.cu_q.numel() - 1
+        pool = ctx.state_pools[binding.index]
+        state = pool[:, :self.state_numel]
+        z = ws.get("delta_in", n, self.in_rows, ctx.dtype)
+        linear(ctx, h, self.in_weight, None, z, n)
+        qkv = ws.get("delta_conv", n, self.conv_width, ctx.dtype)
+        kernels.short_conv(z, 0, self.conv_weight, None, pool[:, self.state_numel:], ctx.state_slots, ctx.cu_q, ctx.q_req,
+                           ctx.positions, n_req, qkv, 0, n, activation="silu")
+        y = ws.get("delta_out", n, self.v_width, ctx.dtype)
+        sizes = (z, self.b_off, self.a_off, self.n_head, self.n_group, self.head_dim, self.value_dim, self.dt_bias,
+                 self.a_log, state, ctx.state_slots, ctx.cu_q, n_req, ctx.positions)
+        # a step with prompt portions: the recurrence a chunk of tokens at a time on the matrix cores, the heads'
+        # norm and gate in a kernel behind it; single tokens: token by token, norm and gate inside
+        chunked = False
+        if not ctx.decode_only:
+            floats = kernels.delta_image_floats(n, n_req, self.n_head, self.head_dim)
+            if floats:
+                sums = ws.get("delta_sums", n, self.v_width, torch.float32)
+                images = ws.get("delta_images", floats // 4, 4, torch.float32)
+                chunked = kernels.delta_state_chunked(qkv, 0, self.k_off, self.v_off, *sizes, images, sums, n,
+                                                      q_scale=self.q_scale)
+        if chunked:
+            kernels.rms_norm(sums, self.head_gain, y, n, self.norm_eps, self.value_dim, groups=self.n_head,
+                             gate=z[:, self.g_off:], gate_act="silu")
+        else:
+            kernels.delta_state(qkv, 0, self.k_off, self.v_off, *sizes, y, n, q_scale=self.q_scale, gate_off=self.g_off,
+                                norm_weight=self.norm_weight, eps=self.norm_eps)
         linear_add(ctx, y, self.out_weight, None, x, n)

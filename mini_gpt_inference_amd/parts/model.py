@@ -100,6 +100,7 @@ class CacheGroupSpec:
     n_pools: int       # caches (one per writing run) in the group
     joint: bool = False   # keys and values are one tensor
     keep_first: int = 0   # with a window: the first positions whose pages stay (the most any run of the group keeps)
+    chunked: bool = False   # the window is a chunk counted from position 0 (for every run of the group)
 
 
 @dataclass
@@ -124,6 +125,13 @@ class KVRun:
     window: int
     tensors: int = 2      # cached tensors a key position costs: keys and values, or one joint latent
     keep_first: int = 0   # first positions seen beside the window
+    chunked: bool = False   # the window is a chunk
+
+    def keys_seen(self, n: int) -> int:
+        """Keys that a query with n keys up to its own sees."""
+        if not self.window:
+            return n
+        return min(n, ((n - 1) % self.window + 1 if self.chunked else self.window) + self.keep_first)
 
 
 @dataclass(frozen=True)
@@ -145,8 +153,7 @@ class ModelCost:
         kv = 0.0
         for run in self.kv_runs:
             for c in context_lens:
-                reach = min(c, run.window + run.keep_first) if run.window else c
-                kv += reach * run.tensors * run.n_kv_head * run.head_dim * cache_itemsize
+                kv += run.keys_seen(c) * run.tensors * run.n_kv_head * run.head_dim * cache_itemsize
         return self.whole_tensor_bytes + n_tokens * self.table_row_bytes + kv + 4.0 * self.state_floats * len(context_lens)
 
     def prompt_flops(self, prompt_lens, n_logit_rows: int) -> float:
@@ -156,7 +163,7 @@ class ModelCost:
         flops = 2.0 * n * self.run_matrix_elements + 2.0 * n_logit_rows * self.head_matrix_elements
         for run in self.kv_runs:
             for t in prompt_lens:
-                seen = sum(min(i + 1, run.window + run.keep_first) if run.window else i + 1 for i in range(t))
+                seen = sum(run.keys_seen(i + 1) for i in range(t))
                 flops += 4.0 * seen * run.n_head * run.head_dim
         return flops
 
@@ -288,7 +295,8 @@ class DecoderModel:
                 need = part.cache_need() if hasattr(part, "cache_need") else None
                 if isinstance(need, KVNeed):
                     kv_runs.append(KVRun(int(getattr(part, "n_head", need.n_kv_head)), need.n_kv_head,
-                                         need.head_dim, need.window, 1 if need.joint else 2, need.keep_first))
+                                         need.head_dim, need.window, 1 if need.joint else 2, need.keep_first,
+                                         need.chunked))
                     state_floats += int(need.state_numel)
                 elif isinstance(need, StateNeed):
                     state_floats += int(need.numel)
@@ -299,7 +307,7 @@ class DecoderModel:
     # ------------------------------------------------------------------ cache
     def _plan_cache(self) -> CacheLayout:
         groups: List[CacheGroupSpec] = []
-        keys: List[Tuple[int, int, int, bool, int]] = []
+        keys: List[Tuple[int, int, int, bool, int, bool]] = []
         state_numels: List[int] = []
         run_bindings: List[Dict[str, CacheBinding]] = []
 
@@ -313,7 +321,8 @@ class DecoderModel:
 
         # What a writing run's pages must keep: the widest window among itself and the runs that read
         # its cache (each masks with its own window; 0, all keys, is the widest).
-        reach: Dict[Tuple[int, str], Tuple[int, int]] = {}      # (window, first positions kept beside it)
+        # (A sliding window of a chunk's size holds the chunk, so runs of both kinds need the wider as a window.)
+        reach: Dict[Tuple[int, str], Tuple[int, int, bool]] = {}     # (window, first positions kept beside it, chunked)
         for i, run in enumerate(self.spec.order):
             for role in self.spec.layers[run.layer].roles("mixer"):
                 need = need_of(i, role)
@@ -322,11 +331,12 @@ class DecoderModel:
                 key = (i if run.reads_cache_of is None else run.reads_cache_of, role)
                 seen = reach.get(key)
                 if seen is None:
-                    reach[key] = (need.window, need.keep_first if need.window else 0)
+                    reach[key] = (need.window, need.keep_first if need.window else 0, bool(need.window and need.chunked))
                 elif 0 in (seen[0], need.window):
-                    reach[key] = (0, 0)
+                    reach[key] = (0, 0, False)
                 else:
-                    reach[key] = (max(seen[0], need.window), max(seen[1], need.keep_first))
+                    reach[key] = (max(seen[0], need.window), max(seen[1], need.keep_first),
+                                  seen[2] and need.chunked and seen[0] == need.window)
 
         for i, run in enumerate(self.spec.order):
             layer_spec = self.spec.layers[run.layer]
@@ -340,17 +350,18 @@ class DecoderModel:
                         raise ValueError(f"run {i} cannot read the cache of run {run.reads_cache_of}: different needs")
                     bindings[role] = CacheBinding("kv", src.group, src.index, writes=False)
                 elif isinstance(need, KVNeed):
-                    key = (need.n_kv_head, need.head_dim, reach[(i, role)][0], need.joint, reach[(i, role)][1])
+                    window, kept_first, chunked = reach[(i, role)]
+                    key = (need.n_kv_head, need.head_dim, window, need.joint, kept_first, chunked)
                     if key not in keys:
                         keys.append(key)
-                        groups.append(CacheGroupSpec(key[0], key[1], key[2], 0, key[3], key[4]))
+                        groups.append(CacheGroupSpec(key[0], key[1], key[2], 0, *key[3:]))
                     g = keys.index(key)
                     state = -1
                     if need.state_numel:
                         state = len(state_numels)
                         state_numels.append(int(need.state_numel))
                     bindings[role] = CacheBinding("kv", g, groups[g].n_pools, writes=True, state=state)
-                    groups[g] = CacheGroupSpec(key[0], key[1], key[2], groups[g].n_pools + 1, key[3], key[4])
+                    groups[g] = CacheGroupSpec(key[0], key[1], key[2], groups[g].n_pools + 1, *key[3:])
                 elif isinstance(need, StateNeed):
                     bindings[role] = CacheBinding("state", -1, len(state_numels), writes=True)
                     state_numels.append(int(need.numel))
