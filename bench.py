@@ -368,15 +368,37 @@ def nutitar_like(layers, width, heads, vocab):
             "embedding": {"scale": 1.0}, "layers": out}
 
 
-COMPARED = {"viperax": viperax_like, "bobevik": bobevik_like, "rilavik": rilavik_like, "nutitar": nutitar_like}
+def gekopel_like(layers, width, heads, vocab):
+    """A Gekopel config.json of a GPT-2-style model's size: the same layers, width, heads and vocabulary, heads of
+    128 channels; delta and attention layers in turn, the delta rule with half as many query/key heads as value
+    heads and four taps, attention with a quarter as many key/value heads in chunks of 512; every token goes
+    through 8 width^2 feed-forward elements a layer (dense in the first layer; then 2 of 8 experts of hidden size
+    3/2 width in 4 groups of which 3 stay, beside a shared one of hidden size width)."""
+    out = []
+    for i in range(layers):
+        if i % 2:
+            kind, mixer = "attention", {"heads": heads, "kv_heads": max(heads // 4, 1), "dim": 128, "vdim": 128,
+                                        "scale": 128 ** -0.5, "bias_max": 384, "mask": {"size": 512}}
+        else:
+            kind, mixer = "delta", {"heads": heads, "kv_heads": max(heads // 2, 1), "dim": 128, "vdim": 128, "conv": 4}
+        mlp = {"kind": "dense", "ff": 4 * width} if i == 0 else {
+            "kind": "moe", "expert": {"ff": width * 3 // 2}, "shared": {"ff": width},
+            "router": {"experts": 8, "top": 2, "scale": 1.5, "groups": {"count": 4, "keep": 3}}}
+        out.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Gekopel", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": 4096,
+            "embedding": {"scale": float(width) ** 0.5}, "layers": out}
+
+
+COMPARED = {"viperax": viperax_like, "bobevik": bobevik_like, "rilavik": rilavik_like, "nutitar": nutitar_like,
+            "gekopel": gekopel_like}
 # the model a design is measured beside: the GPT-2-style model, or the design nearest to it
-BESIDE = {"rilavik": "bobevik"}
+BESIDE = {"rilavik": "bobevik", "gekopel": "rilavik"}
 
 
 def compare_run(args, name):
-    """--compare viperax | bobevik | rilavik | nutitar: prefill (2 prompts of 1,024 tokens as one step) and decode
+    """--compare viperax | bobevik | rilavik | nutitar | gekopel: prefill (2 prompts of 1,024 tokens as one step) and decode
     (batch 8, by the default run's timing rule, fewer blocks) of that design beside the GPT-2-style model
-    (Rilavik: beside Bobevik, the nearest design) at equal layers, width, heads and vocabulary, random
+    (Rilavik: beside Bobevik, Gekopel: beside Rilavik, the nearest designs) at equal layers, width, heads and vocabulary, random
     weights, at COMPARE_SIZES.  One JSON line."""
     import argparse as _argparse
     import gc
@@ -522,7 +544,8 @@ def main(argv=None) -> int:
     ap.add_argument("--prefill-requests", type=int, default=2,
                     help="prompts of 1,024 tokens in the prefill step (the default run's 2,048 tokens are 2)")
     ap.add_argument("--compare", choices=sorted(COMPARED), default=None,
-                    help="prefill and decode of that design beside the GPT-2-style model at equal sizes (COMPARE_SIZES)")
+                    help="prefill and decode of that design beside the GPT-2-style model or the design nearest to it, at "
+                         "equal sizes (COMPARE_SIZES)")
     ap.add_argument("--prefill-only", action="store_true",
                     help="run only the 2,048-token prefill and print its record (for profiling)")
     args = ap.parse_args(argv)

@@ -37,8 +37,8 @@ __device__ __forceinline__ float ds_sum_rows(float v) {
 // With `gate_off` >= 0 each head's output is then divided by its root mean square over E (eps), multiplied by
 // norm_w and by silu of the gate's row (in z, head by head), and stored in the rows' type; otherwise o is stored
 // as float32.
-template <typename T, int DQ>     // DQ: rows of S a lane holds at most
-__global__ __launch_bounds__(1024) void delta_state_kernel(
+template <typename T, int DQ, int THREADS>     // DQ: rows of S a lane holds at most; THREADS: of the workgroup, at most
+__global__ __launch_bounds__(THREADS) void delta_state_kernel(
     const T* __restrict__ x, long ldx, int q_off, int k_off, int v_off, const T* __restrict__ z, long ldz, int b_off,
     int a_off, int gate_off, int n_head, int heads_per_group, int D, int E, float q_scale,
     const float* __restrict__ dt_bias, const float* __restrict__ a_log, const float* __restrict__ norm_w, float eps,
@@ -46,7 +46,7 @@ __global__ __launch_bounds__(1024) void delta_state_kernel(
     const int* __restrict__ positions, void* __restrict__ out, long ldo) {
   constexpr int LDQ = DQ + 4;            // a quarter's stretch of a staged row
   __shared__ __attribute__((aligned(16))) float q_s[DS_TC][4 * LDQ], k_s[DS_TC][4 * LDQ];
-  __shared__ float v_s[DS_TC][DS_MAX], o_s[DS_TC][DS_MAX], g_s[DS_TC], beta_s[DS_TC], qk_s[DS_TC];
+  __shared__ float v_s[DS_TC][DS_MAX], o_s[DS_TC][DS_MAX], gate_s[DS_TC][DS_MAX], g_s[DS_TC], beta_s[DS_TC], qk_s[DS_TC];
   const int r = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int slot = state_slots[r];
   const int t_begin = cu_q[r], t_end = cu_q[r + 1];
@@ -63,7 +63,8 @@ __global__ __launch_bounds__(1024) void delta_state_kernel(
 #pragma unroll
   for (int j = 0; j < DQ; ++j) S[j] = (mine && !fresh && j < rows) ? st[(long)(d0 + j) * E + c] : 0.f;
   const float rate = expf(a_log[h]), bias = dt_bias[h];
-  for (int i = tid; i < DS_TC * 4 * LDQ; i += blockDim.x) {      // rows behind a quarter's last stay zero
+  const int staged = t_end - t_begin < DS_TC ? t_end - t_begin : DS_TC;
+  for (int i = tid; i < staged * 4 * LDQ; i += blockDim.x) {     // rows behind a quarter's last stay zero
     (&q_s[0][0])[i] = 0.f;
     (&k_s[0][0])[i] = 0.f;
   }
@@ -108,6 +109,7 @@ __global__ __launch_bounds__(1024) void delta_state_kernel(
     for (int i = tid; i < nt * E; i += blockDim.x) {
       const int tt = i / E, e = i - tt * E;
       v_s[tt][e] = to_float<T>(x[(long)(t0 + tt) * ldx + v_off + (long)h * E + e]);
+      if (gate_off >= 0) gate_s[tt][e] = to_float<T>(z[(long)(t0 + tt) * ldz + gate_off + (long)h * E + e]);
     }
     __syncthreads();
     for (int tt = 0; tt < nt; ++tt) {
@@ -140,13 +142,12 @@ __global__ __launch_bounds__(1024) void delta_state_kernel(
         for (int e = lane; e < E; e += 64) ((float*)out)[orow + e] = o_s[tt][e];
         continue;
       }
-      const T* gr = z + (long)(t0 + tt) * ldz + gate_off + (long)h * E;
       float ov[DS_MAX / 64], gv[DS_MAX / 64], ss = 0.f;
 #pragma unroll
       for (int u = 0; u < DS_MAX / 64; ++u) {
         const int e = lane + 64 * u;
         ov[u] = e < E ? o_s[tt][e] : 0.f;
-        gv[u] = e < E ? to_float<T>(gr[e]) : 0.f;
+        gv[u] = e < E ? gate_s[tt][e] : 0.f;
         ss = fmaf(ov[u], ov[u], ss);
       }
       const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)E + eps);
@@ -184,14 +185,19 @@ extern "C" int mgpt_delta_state(const void* x, int dtype, long ldx, int q_off, i
   if (n_head > 65535) return MGPT_ERR_TOO_LARGE;
   const int quarter = (D + 3) / 4;
   dim3 grid(n_req, n_head), block(64 * ((E + 15) / 16));
-#define DS_LAUNCH2(T, Q)                                                                                              \
-  hipLaunchKernelGGL((delta_state_kernel<T, Q>), grid, block, 0, stream, (const T*)x, ldx, q_off, k_off, v_off,       \
+#define DS_LAUNCH3(T, Q, N)                                                                                              \
+  hipLaunchKernelGGL((delta_state_kernel<T, Q, N>), grid, block, 0, stream, (const T*)x, ldx, q_off, k_off, v_off,       \
                      (const T*)z, ldz, b_off, a_off, gate_off, n_head, n_head / n_group, D, E, q_scale, dt_bias, a_log, \
                      norm_w, eps, state, ld_state, state_slots, cu_q, positions, out, ldo)
+#define DS_LAUNCH2(T, Q)                 \
+  {                                      \
+    if (E <= 128) DS_LAUNCH3(T, Q, 512); \
+    else DS_LAUNCH3(T, Q, 1024);         \
+  }
 #define DS_LAUNCH(Q)                     \
   {                                      \
-    if (dtype == MGPT_F32) DS_LAUNCH2(float, Q); \
-    else DS_LAUNCH2(bf16_t, Q);          \
+    if (dtype == MGPT_F32) DS_LAUNCH2(float, Q) \
+    else DS_LAUNCH2(bf16_t, Q)           \
   }
   if (quarter <= 4) DS_LAUNCH(4)
   else if (quarter <= 8) DS_LAUNCH(8)
@@ -200,6 +206,7 @@ extern "C" int mgpt_delta_state(const void* x, int dtype, long ldx, int q_off, i
   else DS_LAUNCH(64)
 #undef DS_LAUNCH
 #undef DS_LAUNCH2
+#undef DS_LAUNCH3
   return mgpt_last_error();
 }
 
@@ -238,7 +245,26 @@ __host__ __device__ __forceinline__ int ds_image_floats(int Dp) {
   return 2 * DC_C * (Dp + 4) + Dp * DC_LDP + DC_C * DC_LDP;
 }
 
-template <typename T>
+__device__ __forceinline__ void ds_load8(const float* p, float (&v)[8]) {
+  const ds_f32x4 a = *reinterpret_cast<const ds_f32x4*>(p), b = *reinterpret_cast<const ds_f32x4*>(p + 4);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    v[e] = a[e];
+    v[4 + e] = b[e];
+  }
+}
+__device__ __forceinline__ void ds_load8(const bf16_t* p, float (&v)[8]) {
+  const uint4 a = *reinterpret_cast<const uint4*>(p);
+  const unsigned words[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    v[2 * k] = __uint_as_float(words[k] << 16);
+    v[2 * k + 1] = __uint_as_float(words[k] & 0xffff0000u);
+  }
+}
+
+// VEC: D is a multiple of 8 and the rows of x are aligned for loads of eight elements
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(
     const T* __restrict__ x, long ldx, int q_off, int k_off, int v_off, const T* __restrict__ z, long ldz, int b_off,
     int a_off, int n_head, int heads_per_group, int D, int E, float q_scale, const float* __restrict__ dt_bias,
@@ -252,7 +278,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
   float* Ps = As + DC_C * DC_LDP;         // [32][LDP] q . k
   float* Ms = Ps + DC_C * DC_LDP;         // [32][LDP] the decays between tokens
   float* Rs = Ms + DC_C * DC_LDP;         // [32][LDP] R
-  float* Xs = Rs + DC_C * DC_LDP;         // [16][LDP] scratch of the block inverse
+  float* Xs = Ps;                         // [16][LDP] scratch of the block inverse (q . k is in the image by then)
   __shared__ float beta_s[DC_C], l_s[DC_C], G_s[DC_C], bg_s[DC_C];
   const int chunk = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63, r16 = lane & 15, g4 = lane >> 4;
@@ -274,12 +300,31 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     const T* xr = x + (long)(t0 + row) * ldx + (long)group * D;
     float qv[DC_DMAX / 8], kv[DC_DMAX / 8];
     float sq = 0.f, sk = 0.f;
+    // value u of a thread is channel sub + 8 u, or (VEC) channel 8 sub + u % 8 + 64 (u / 8)
+    auto channel = [&](int u) { return VEC ? 8 * sub + (u & 7) + 64 * (u >> 3) : sub + 8 * u; };
+    if (VEC) {
 #pragma unroll
-    for (int u = 0; u < DC_DMAX / 8; ++u) {
-      const int d = sub + 8 * u;
-      const bool ok = row < nt && d < D;
-      qv[u] = ok ? to_float<T>(xr[q_off + d]) : 0.f;
-      kv[u] = ok ? to_float<T>(xr[k_off + d]) : 0.f;
+      for (int u = 0; u < DC_DMAX / 64; ++u) {
+        const int d = 8 * sub + 64 * u;
+        float q8[8] = {}, k8[8] = {};
+        if (row < nt && d < D) {
+          ds_load8(xr + q_off + d, q8);
+          ds_load8(xr + k_off + d, k8);
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          qv[8 * u + e] = q8[e];
+          kv[8 * u + e] = k8[e];
+        }
+      }
+    } else {
+#pragma unroll
+      for (int u = 0; u < DC_DMAX / 8; ++u) {
+        const int d = channel(u);
+        const bool ok = row < nt && d < D;
+        qv[u] = ok ? to_float<T>(xr[q_off + d]) : 0.f;
+        kv[u] = ok ? to_float<T>(xr[k_off + d]) : 0.f;
+      }
     }
 #pragma unroll
     for (int u = 0; u < DC_DMAX / 8; ++u) {
@@ -294,7 +339,7 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     const float iq = q_scale / sqrtf(sq + DS_UNIT_EPS), ik = 1.0f / sqrtf(sk + DS_UNIT_EPS);
 #pragma unroll
     for (int u = 0; u < DC_DMAX / 8; ++u) {
-      const int d = sub + 8 * u;
+      const int d = channel(u);
       if (d < Dp) {
         Qs[row * ld + d] = qv[u] * iq;
         Ks[row * ld + d] = kv[u] * ik;
@@ -373,9 +418,10 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
     for (int i = 0; i < 16; ++i) Rs[(b * 16 + i) * DC_LDP + b * 16 + j] = col[i];
   } else if (tid >= 64) {
     // meanwhile the other waves put the queries and the keys into the image
-    for (int e = tid - 64; e < DC_C * Dp; e += 192) {
-      const int i = e / Dp, d = e - i * Dp;
-      imgQ[i * ld + d] = Qs[i * ld + d] * G_s[i];
+    for (int i = (tid - 64) >> 3; i < DC_C; i += 24) {
+      const float G = G_s[i];
+      for (int d = 4 * (tid & 7); d < Dp; d += 32)
+        *reinterpret_cast<ds_f32x4*>(imgQ + i * ld + d) = *reinterpret_cast<const ds_f32x4*>(Qs + i * ld + d) * G;
     }
     for (int e = tid - 64; e < DC_C * Dp; e += 192) {
       const int d = e >> 5, i = e & 31;
@@ -610,13 +656,19 @@ extern "C" int mgpt_delta_state_chunked(const void* x, int dtype, long ldx, int 
       allowed = bytes;                                                                                       \
     }                                                                                                        \
   }
-#define DC_PREPARE(T)                                                                                                  \
+  const size_t align = (size_t)x | (size_t)(ldx * (dtype == MGPT_F32 ? 4 : 2));
+  const bool vec = !(D & 7) && !(align & 15) && !((q_off | k_off) & 7);
+#define DC_PREPARE2(T, V)                                                                                                  \
   {                                                                                                                    \
-    const int bytes = (int)sizeof(float) * (2 * DC_C * ld + (4 * DC_C + 16) * DC_LDP);                                \
-    DC_ALLOW((delta_prepare_kernel<T>), bytes)                                                                         \
-    hipLaunchKernelGGL((delta_prepare_kernel<T>), dim3(chunks, n_head), dim3(256), bytes, stream, (const T*)x, ldx,    \
+    const int bytes = (int)sizeof(float) * (2 * DC_C * ld + 4 * DC_C * DC_LDP);                                       \
+    DC_ALLOW((delta_prepare_kernel<T, V>), bytes)                                                                         \
+    hipLaunchKernelGGL((delta_prepare_kernel<T, V>), dim3(chunks, n_head), dim3(256), bytes, stream, (const T*)x, ldx,    \
                        q_off, k_off, v_off, (const T*)z, ldz, b_off, a_off, n_head, n_head / n_group, D, E, q_scale,   \
                        dt_bias, a_log, cu_q, n_req, images, out, ldo);                                                 \
+  }
+#define DC_PREPARE(T)                                        \
+  {                                                          \
+    if (vec) DC_PREPARE2(T, true) else DC_PREPARE2(T, false) \
   }
   if (dtype == MGPT_F32) DC_PREPARE(float) else DC_PREPARE(bf16_t)
 #define DC_WALK(EB)                                                                                              \
@@ -630,6 +682,7 @@ extern "C" int mgpt_delta_state_chunked(const void* x, int dtype, long ldx, int 
   if ((long)n_req * n_head * ((E + 31) / 32) >= 256) DC_WALK(32) else DC_WALK(16)
 #undef DC_WALK
 #undef DC_PREPARE
+#undef DC_PREPARE2
 #undef DC_ALLOW
   return mgpt_last_error();
 }

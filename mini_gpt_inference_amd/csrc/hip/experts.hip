@@ -157,9 +157,9 @@ __device__ __forceinline__ void router_load8(const bf16_t* p, float (&v)[8]) {
 
 // The storage types are the kernel's parameters (a choice made load by load keeps the loads from being in flight
 // together).  VEC: the width is a multiple of 8 and the rows are aligned for loads of eight elements; then thread t
-// takes columns 8 t .. 8 t + 7 of every stretch of 2,048 columns for eight experts at a time, whose loads are all in
+// takes columns 8 t .. 8 t + 7 of every stretch of 2,048 columns for J experts at a time, whose loads are all in
 // flight together, and the sums meet through the waves in a fixed order.  Otherwise a wave takes an expert at a time.
-template <typename HT, typename WT, bool VEC>
+template <typename HT, typename WT, bool VEC, int J>     // J: rows of the matrix in flight at a time (VEC)
 __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__ h, long ldh, const WT* __restrict__ w,
                                                           const int* __restrict__ q_req, int width, int n_experts, int top,
                                                           int kind, int* __restrict__ chosen, float* __restrict__ weight,
@@ -169,19 +169,19 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
   __shared__ float logit[EX_MAX_EXPERTS + 1];    // the extra row's comes last
   __shared__ float key[EX_MAX_EXPERTS];          // what the choice goes by
   __shared__ float rank[EX_MAX_EXPERTS];         // of a group
-  __shared__ float part[4][8];
+  __shared__ float part[4][J];
   const int n_rows_w = n_experts + (extra ? 1 : 0);
   const int n = blockIdx.x;
   if (q_req && q_req[n] < 0) return;     // padded token
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   if (VEC) {
-    for (int e0 = 0; e0 < n_rows_w; e0 += 8) {
-      float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    for (int e0 = 0; e0 < n_rows_w; e0 += J) {
+      float acc[J] = {};
       for (int c = 8 * threadIdx.x; c < width; c += 8 * 256) {
         float hv[8];
         router_load8(h + (long)n * ldh + c, hv);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
+        for (int j = 0; j < J; ++j) {
           const int e = e0 + j < n_experts ? e0 + j : n_experts - 1;     // (behind the last row: loaded again, not used)
           float wv[8];
           router_load8((extra && e0 + j >= n_experts ? extra : w + (long)e * width) + c, wv);
@@ -190,12 +190,12 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
         }
       }
 #pragma unroll
-      for (int j = 0; j < 8; ++j) {
+      for (int j = 0; j < J; ++j) {
         const float sum = wave_sum(acc[j]);
         if (lane == 0) part[wave][j] = sum;
       }
       __syncthreads();
-      if (threadIdx.x < 8 && e0 + threadIdx.x < n_rows_w)
+      if (threadIdx.x < J && e0 + threadIdx.x < n_rows_w)
         logit[e0 + threadIdx.x] = (part[0][threadIdx.x] + part[1][threadIdx.x]) + (part[2][threadIdx.x] + part[3][threadIdx.x]);
       __syncthreads();
     }
@@ -288,23 +288,31 @@ extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* 
   if (n_groups > keep && keep > 0 && (n_experts % n_groups || top > keep * (n_experts / n_groups))) return MGPT_ERR_BAD_SHAPE;
   if (extra && !extra_out) return MGPT_ERR_NULL;
   const size_t h_size = dtype == MGPT_F32 ? 4 : 2, w_size = w_dtype == MGPT_F32 ? 4 : 2;
+  const int rows_w = n_experts + (extra ? 1 : 0);
   const bool vec = !(width & 7) && !(((size_t)h | (size_t)(ldh * h_size)) & 15) && !(((size_t)w | (size_t)extra) & 15);
-#define ROUTER_LAUNCH(HT, WT)                                                                                            \
+#define ROUTER_LAUNCH2(HT, WT, JJ)                                                                                            \
   {                                                                                                                      \
     if (vec)                                                                                                             \
-      hipLaunchKernelGGL((router_topk_kernel<HT, WT, true>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,      \
+      hipLaunchKernelGGL((router_topk_kernel<HT, WT, true, JJ>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,      \
                          (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
                          normalise, scale, (const WT*)extra, extra_out);                                                 \
     else                                                                                                                 \
-      hipLaunchKernelGGL((router_topk_kernel<HT, WT, false>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,     \
+      hipLaunchKernelGGL((router_topk_kernel<HT, WT, false, 8>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,     \
                          (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
                          normalise, scale, (const WT*)extra, extra_out);                                                 \
+  }
+  // up to eight rows at a time; a matrix of 9 to 12 (a few experts and the extra row) in one go
+#define ROUTER_LAUNCH(HT, WT)                                                                                            \
+  {                                                                                                                      \
+    if (rows_w > 8 && rows_w <= 12) ROUTER_LAUNCH2(HT, WT, 12)                                                           \
+    else ROUTER_LAUNCH2(HT, WT, 8)                                                                                       \
   }
   if (dtype == MGPT_F32 && w_dtype == MGPT_F32) ROUTER_LAUNCH(float, float)
   else if (dtype == MGPT_F32) ROUTER_LAUNCH(float, bf16_t)
   else if (w_dtype == MGPT_F32) ROUTER_LAUNCH(bf16_t, float)
   else ROUTER_LAUNCH(bf16_t, bf16_t)
 #undef ROUTER_LAUNCH
+#undef ROUTER_LAUNCH2
   return mgpt_last_error();
 }
 
