@@ -83,9 +83,14 @@ RAW: Dict[str, dict] = {
     "E": model(45, 48, 1e-5, 5.0, 150, [
         layer("delta", delta(4, 2, 24, 16, 4), moe(4, 2, 24, (4, 2), 1.0, 24)),
         layer("delta", delta(3, 1, 16, 32, 2), None)]),
+    # attention layers only, two of them with the same pages and different chunks: no state
+    "F": model(64, 80, 1e-5, 1.5, 260, [
+        layer("attention", attention(4, 2, 32, 32, 0.18, 70, 40), moe(7, 1, 40, (7, 4), 1.0, 24)),
+        layer("attention", attention(2, 2, 32, 24, 0.2, 7), None),
+        layer("attention", attention(6, 2, 24, 32, 0.15, 300, 64), dense(112))]),
 }
-SEEDS = {"A": 31, "B": 32, "C": 33, "D": 34, "E": 35}
-BUCKETS = {"A": 16, "B": 20, "C": 4, "D": 32, "E": 8}     # rows of the distance tables
+SEEDS = {"A": 31, "B": 32, "C": 33, "D": 34, "E": 35, "F": 36}
+BUCKETS = {"A": 16, "B": 20, "C": 4, "D": 32, "E": 8, "F": 6}     # rows of the distance tables
 STD_SCALE = 1.5
 
 

@@ -454,7 +454,7 @@ def test_scaled_embedding_with_positions(dtype):
 
 # ---------------------------------------------------------------- the model through the step function
 LENGTHS = {"A": [5, 70, 23, 41, 2, 64, 37], "B": [1, 9, 33, 17, 110], "C": [40, 3, 64, 21], "D": [75, 12, 30, 6, 49],
-           "E": [33, 4, 70, 18, 2]}
+           "E": [33, 4, 70, 18, 2], "F": [130, 1, 66, 40, 9]}
 _folders, _plain, _twin = {}, {}, {}
 
 
