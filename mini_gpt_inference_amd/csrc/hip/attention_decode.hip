@@ -15,7 +15,8 @@
 // Slots outside the visible range are never loaded.  With `keep_first` > 0 a query behind a window also sees
 // the keys at positions below keep_first; with `score_bias` a visible key's weight is
 // sigmoid(score + score_bias[head]) and nothing is normalised; with `chunked` a query sees its own chunk of
-// `window` positions; with `dist_bias` the number for a key's distance is added to its scaled score.
+// `window` positions; with `dist_bias` the number for a key's distance is added to its scaled score; with `slopes`
+// slope * distance is taken off it (behind the cap).
 #include "attention_mask.h"
 #include "common.h"
 #include "launchers.h"
@@ -30,7 +31,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_kernel(
     const int* __restrict__ seq_lens, const int* __restrict__ q_req, int n_tokens, int n_head,
     int n_kv_head, int head_dim, int page_size, float scale, int window, const float* __restrict__ sinks,
     float softcap, const bf16_t* __restrict__ gate, long ldg, int keep_first, const float* __restrict__ score_bias,
-    int chunked, const float* __restrict__ dist_bias, int bias_len) {
+    int chunked, const float* __restrict__ dist_bias, int bias_len, const float* __restrict__ slopes) {
   __shared__ float q_s[AD_MAX_DPL * 64];
   __shared__ float p_s[AD_WAVES][64];
   __shared__ int page_s[AD_WAVES][64];
@@ -61,6 +62,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_kernel(
 
   const bool weigh = score_bias != nullptr;   // sigmoid weights, no softmax
   const float bias = weigh ? score_bias[h] : 0.f;
+  const float slope = slopes ? slopes[h] : 0.f;
   // the chunks of the kept first keys (those before the window's first chunk), then the window's
   const int first_chunk = kv_begin / 64;
   const int kept_chunks = keep_first > 0 ? ((keep_first + 63) / 64 < first_chunk ? (keep_first + 63) / 64 : first_chunk) : 0;
@@ -87,6 +89,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_kernel(
       }
       s = softcap > 0.f ? softcap * tanh_fast(dot * __builtin_amdgcn_rcpf(softcap)) : dot;
       if (dist_bias) s += dist_bias[(long)h * bias_len + distance_entry(qpos - j, bias_len)];
+      if (slopes) s = fmaf(-slope, (float)(qpos - j), s);
     }
     float p = 0.f, alpha = 1.f;
     if (weigh) {
@@ -165,20 +168,20 @@ extern "C" int mgpt_paged_attention_split_bf16(
     const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int* q_req,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias,
-    int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
+    int chunked, const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !cu_q || !seq_lens || !q_req) return MGPT_ERR_NULL;
   if (n_tokens < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 || head_dim <= 0 ||
       head_dim > AD_MAX_DPL * 64 || (head_dim % 8) != 0 || page_size <= 0 || max_blocks <= 0 || window < 0 ||
       keep_first < 0 || (score_bias && (sinks || softcap > 0.f)) ||
-      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
+      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)) || (slopes && (dist_bias || score_bias)))
     return MGPT_ERR_BAD_SHAPE;
   if (window == 0) keep_first = 0;
   if (n_head > 65535) return MGPT_ERR_TOO_LARGE;
   hipLaunchKernelGGL(paged_attention_split_kernel, dim3(n_tokens, n_head), dim3(256), 0, stream,
                      (const bf16_t*)q, ldq, (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool,
                      block_tables, max_blocks, cu_q, seq_lens, q_req, n_tokens, n_head, n_kv_head, head_dim,
-                     page_size, scale, window, sinks, softcap, (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len);
+                     page_size, scale, window, sinks, softcap, (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len, slopes);
   return mgpt_last_error();
 }
 
@@ -196,7 +199,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_fast_kernel(
     const int* __restrict__ seq_lens, const int* __restrict__ q_req, int n_tokens, int n_head,
     int n_kv_head, int page_size, float scale, int window, const float* __restrict__ sinks, float softcap,
     const bf16_t* __restrict__ gate, long ldg, int keep_first, const float* __restrict__ score_bias,
-    int chunked, const float* __restrict__ dist_bias, int bias_len) {
+    int chunked, const float* __restrict__ dist_bias, int bias_len, const float* __restrict__ slopes) {
   constexpr int LPK = D / 8;     // lanes per key
   constexpr int KPI = 64 / LPK;  // keys per load instruction
   __shared__ float m_s[AD_WAVES], l_s[AD_WAVES];
@@ -234,6 +237,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_fast_kernel(
 
   const bool weigh = score_bias != nullptr;   // sigmoid weights, no softmax
   const float bias = weigh ? score_bias[h] : 0.f;
+  const float slope = slopes ? slopes[h] : 0.f;
   const int first_chunk = kv_begin / 64;
   const int kept_chunks = keep_first > 0 ? ((keep_first + 63) / 64 < first_chunk ? (keep_first + 63) / 64 : first_chunk) : 0;
   const int n_chunks = kept_chunks + (kv_end + 63) / 64 - first_chunk;
@@ -272,6 +276,7 @@ __global__ __launch_bounds__(256) void paged_attention_split_fast_kernel(
       for (int off = 1; off < LPK; off <<= 1) dot += __shfl_xor(dot, off, 64);
       if (softcap > 0.f) dot = softcap * tanh_fast(dot * __builtin_amdgcn_rcpf(softcap));
       if (dist_bias) dot += dist_bias[(long)h * bias_len + distance_entry(qpos - (c0 + i * KPI + sub), bias_len)];
+      if (slopes) dot = fmaf(-slope, (float)(qpos - (c0 + i * KPI + sub)), dot);
       s[i] = valid[i] ? dot : -INFINITY;
       cmax = fmaxf(cmax, s[i]);
     }
@@ -333,12 +338,12 @@ extern "C" int mgpt_paged_attention_split_fast_bf16(
     const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int* q_req,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias,
-    int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
+    int chunked, const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !cu_q || !seq_lens || !q_req) return MGPT_ERR_NULL;
   if (n_tokens < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 || page_size <= 0 ||
       max_blocks <= 0 || window < 0 || (ldq % 8) != 0 || keep_first < 0 || (score_bias && (sinks || softcap > 0.f)) ||
-      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
+      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)) || (slopes && (dist_bias || score_bias)))
     return MGPT_ERR_BAD_SHAPE;
   if (window == 0) keep_first = 0;
   if (n_head > 65535) return MGPT_ERR_TOO_LARGE;
@@ -347,7 +352,7 @@ extern "C" int mgpt_paged_attention_split_fast_bf16(
   hipLaunchKernelGGL(paged_attention_split_fast_kernel<DD>, grid, block, 0, stream, (const bf16_t*)q, ldq, \
                      (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool, block_tables,       \
                      max_blocks, cu_q, seq_lens, q_req, n_tokens, n_head, n_kv_head, page_size, scale, window, sinks, softcap, \
-                     (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len)
+                     (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len, slopes)
   switch (head_dim) {
     case 16: AD_LAUNCH(16); break;
     case 32: AD_LAUNCH(32); break;

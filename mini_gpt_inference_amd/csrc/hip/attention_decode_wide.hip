@@ -23,7 +23,8 @@
 //    pass then starts at key 0 and the passes behind the kept keys go on at the window's first chunk; with
 //    `score_bias` a visible key's weight is sigmoid(score + score_bias[head]) and nothing is normalised;
 //  * with `chunked` a query sees its own chunk of `window` positions; with a table of numbers by distance
-//    (BIAS) a lane asks for its keys' numbers together with the keys;
+//    (BIAS 1) a lane asks for its keys' numbers together with the keys; with a slope per head (BIAS 2) slope *
+//    distance is taken off a score, behind the cap;
 //  * the waves' partial results (maximum, sum, weighted values per key subgroup) are merged
 //    through LDS once, in a fixed order.
 #include "attention_mask.h"
@@ -69,7 +70,7 @@ __device__ __forceinline__ float aw_dot2(unsigned int a, unsigned int b, float c
 }
 
 // IDENT: token n is request n (or padded), so its block table row is known before anything is loaded
-template <int D, bool IDENT, bool BIAS>
+template <int D, bool IDENT, int BIAS>
 __global__ __launch_bounds__(AW_WAVES * 64) void paged_attention_decode_kernel(
     const bf16_t* __restrict__ q, long ldq, bf16_t* __restrict__ out, long ldo,
     const bf16_t* __restrict__ kpool, const bf16_t* __restrict__ vpool,
@@ -77,7 +78,7 @@ __global__ __launch_bounds__(AW_WAVES * 64) void paged_attention_decode_kernel(
     const int* __restrict__ q_req, const int* __restrict__ cu_q, int n_head, int n_kv_head, int page_shift,
     int num_pages, unsigned int page_bytes, float scale_log2e, int window, const float* __restrict__ sinks,
     float cap_log2e, const bf16_t* __restrict__ gate, long ldg, int keep_first, const float* __restrict__ score_bias,
-    int chunked, const float* __restrict__ dist_bias, int bias_len) {
+    int chunked, const float* __restrict__ dist_bias, int bias_len, const float* __restrict__ slopes) {
   constexpr int LPK = D / 8;     // lanes per key
   constexpr int KPI = 64 / LPK;  // keys per load instruction
   constexpr int ROWS = AW_WAVES * KPI;      // partial results: one per (key subgroup, wave)
@@ -110,6 +111,7 @@ __global__ __launch_bounds__(AW_WAVES * 64) void paged_attention_decode_kernel(
   const int* bt = block_tables + (long)r * max_blocks;
   const bool weigh = score_bias != nullptr;   // sigmoid weights, no softmax
   const float bias_log2e = weigh ? score_bias[h] * 1.4426950408889634f : 0.f;
+  const float slope_log2e = BIAS == 2 ? slopes[h] * 1.4426950408889634f : 0.f;
 
   float m = -INFINITY, l = 0.f;
   float acc[8];
@@ -150,7 +152,7 @@ __global__ __launch_bounds__(AW_WAVES * 64) void paged_attention_decode_kernel(
       const unsigned int off = follow ? row_off + lane_off : 0u;
       kraw[i] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(kpool) + off);
       vraw[i] = *reinterpret_cast<const uint4*>(reinterpret_cast<const char*>(vpool) + off);
-      if (BIAS) by_dist[i] = dist_bias[(long)h * bias_len + distance_entry(qpos - j, bias_len)];
+      if (BIAS == 1) by_dist[i] = dist_bias[(long)h * bias_len + distance_entry(qpos - j, bias_len)];
     }
 #pragma unroll
     for (int i = 0; i < LPK; ++i)
@@ -166,7 +168,8 @@ __global__ __launch_bounds__(AW_WAVES * 64) void paged_attention_decode_kernel(
       dot = aw_dot2(qraw.w, kraw[i].w, dot);
       dot = aw_group_sum<LPK>(dot) * scale_log2e;
       if (cap_log2e > 0.f) dot = cap_log2e * tanh_fast(dot * __builtin_amdgcn_rcpf(cap_log2e));   // capped scores
-      if (BIAS) dot = fmaf(by_dist[i], 1.4426950408889634f, dot);
+      if (BIAS == 1) dot = fmaf(by_dist[i], 1.4426950408889634f, dot);
+      if (BIAS == 2) dot = fmaf(-slope_log2e, (float)(qpos - (c0 + i * KPI + sub)), dot);
       s[i] = valid[i] ? dot : -INFINITY;
       cmax = fmaxf(cmax, s[i]);
     }
@@ -258,12 +261,12 @@ extern "C" int mgpt_paged_attention_decode_bf16(
     const int* block_tables, int max_blocks, const int* positions, const int* q_req, const int* cu_q,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, int num_pages, float scale, int window,
     int identity, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias,
-    int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
+    int chunked, const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !positions || !q_req) return MGPT_ERR_NULL;
   if (n_tokens < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 || page_size <= 0 ||
       max_blocks <= 0 || num_pages <= 0 || window < 0 || (ldq % 8) != 0 || (identity && cu_q) || keep_first < 0 ||
-      (score_bias && (sinks || softcap > 0.f)) || (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
+      (score_bias && (sinks || softcap > 0.f)) || (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)) || (slopes && (dist_bias || score_bias)))
     return MGPT_ERR_BAD_SHAPE;
   if (window == 0) keep_first = 0;
   if (n_head > 65535) return MGPT_ERR_TOO_LARGE;
@@ -282,11 +285,12 @@ extern "C" int mgpt_paged_attention_decode_bf16(
                      (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool, block_tables,          \
                      max_blocks, positions, q_req, cu_q, n_head, n_kv_head, page_shift, num_pages, page_bytes, \
                      scale_log2e, window, sinks, softcap > 0.f ? softcap * 1.4426950408889634f : 0.f, \
-                     (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len)
+                     (const bf16_t*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len, slopes)
 #define AW_LAUNCH2(DD, ID)                     \
   do {                                         \
-    if (dist_bias) AW_LAUNCH3(DD, ID, true);   \
-    else AW_LAUNCH3(DD, ID, false);            \
+    if (slopes) AW_LAUNCH3(DD, ID, 2);         \
+    else if (dist_bias) AW_LAUNCH3(DD, ID, 1); \
+    else AW_LAUNCH3(DD, ID, 0);                \
   } while (0)
 #define AW_LAUNCH(DD)              \
   do {                             \

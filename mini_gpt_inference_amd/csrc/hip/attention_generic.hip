@@ -16,6 +16,7 @@
 // sigmoid(score + score_bias[head]), and the weights are not normalised;
 // with `chunked` a query sees the positions of its own chunk of `window` positions instead of the last `window`;
 // with `dist_bias` ([heads][bias_len]) the number for the key's distance is added to the scaled score;
+// with `slopes` ([heads]) slope * distance is taken off the scaled (and capped) score;
 // y = P v (reference: src/minigpt_infer/model.py:61-87,
 // the rule col <= cache_len + row of src/minigpt_infer/batch.py:202-227).
 //
@@ -80,7 +81,8 @@ __global__ __launch_bounds__(64) void paged_attention_generic_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ seq_lens, const int* __restrict__ q_req,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     const float* __restrict__ sinks, float softcap, const T* __restrict__ gate, long ldg, int keep_first,
-    const float* __restrict__ score_bias, int chunked, const float* __restrict__ dist_bias, int bias_len) {
+    const float* __restrict__ score_bias, int chunked, const float* __restrict__ dist_bias, int bias_len,
+    const float* __restrict__ slopes) {
   __shared__ float q_s[MAX_DPL * MGPT_WAVE];
   __shared__ float p_s[MGPT_WAVE];
   __shared__ int page_s[MGPT_WAVE];
@@ -126,6 +128,7 @@ __global__ __launch_bounds__(64) void paged_attention_generic_kernel(
       s = dot * scale;
       if (dist_bias) s += dist_bias[(long)h * bias_len + distance_entry(qpos - j, bias_len)];
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+      if (slopes) s -= slopes[h] * (float)(qpos - j);
     }
     float p = 0.f, alpha = 1.f;
     if (weigh) {
@@ -186,12 +189,13 @@ extern "C" int mgpt_paged_attention_generic(
     const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int* q_req,
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     int dtype, int fast_exp, const float* sinks, float softcap, const void* gate, long ldg, int keep_first,
-    const float* score_bias, int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
+    const float* score_bias, int chunked, const float* dist_bias, int bias_len, const float* slopes,
+    hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !cu_q || !seq_lens || !q_req) return MGPT_ERR_NULL;
   if (n_tokens < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 || head_dim <= 0 ||
       head_dim > MAX_DPL * MGPT_WAVE || page_size <= 0 || max_blocks <= 0 || window < 0 || keep_first < 0 || (score_bias && (sinks || softcap > 0.f)) ||
-      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
+      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)) || (slopes && (dist_bias || score_bias)))
     return MGPT_ERR_BAD_SHAPE;
   if (n_head > 65535) return MGPT_ERR_TOO_LARGE;
   if (window == 0) keep_first = 0;   // every key is seen anyway
@@ -200,7 +204,7 @@ extern "C" int mgpt_paged_attention_generic(
   hipLaunchKernelGGL((paged_attention_generic_kernel<T, F>), grid, block, 0, stream, (const T*)q, ldq, \
                      (T*)out, ldo, (const T*)kpool, (const T*)vpool, block_tables, max_blocks, cu_q,  \
                      seq_lens, q_req, n_tokens, n_head, n_kv_head, head_dim, page_size, scale, window, sinks, softcap, \
-                     (const T*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len)
+                     (const T*)gate, ldg, keep_first, score_bias, chunked, dist_bias, bias_len, slopes)
   if (dtype == MGPT_F32) {
     if (fast_exp) LAUNCH(float, true); else LAUNCH(float, false);
   } else if (dtype == MGPT_BF16) {

@@ -10,7 +10,8 @@
 // sigmoid(score + score_bias[head]) and nothing is normalised.  With `chunked` a query sees its own chunk of
 // `window` positions instead of the last `window`.
 //
-// With a table of numbers by distance (BIAS; in the scores' units before log2 e) the numbers that a step's
+// With a slope per head (BIAS 2) slope * distance is taken off a score, behind the cap.
+// With a table of numbers by distance (BIAS 1; in the scores' units before log2 e) the numbers that a step's
 // stretch of keys needs for the tile's 64 queries, one per distance, lie in LDS in the order of the key, so that a
 // lane's four neighbouring keys read four neighbouring numbers.
 //
@@ -69,7 +70,7 @@ __device__ __forceinline__ float pf_sum_over_rows(float v) {
 // thread stages as much per step as with one group, and on each SIMD a wave of one group has its
 // softmax arithmetic while the other group's wave has its MFMAs.  Head sizes whose two stretches
 // do not fit LDS run with one group.
-template <int D, int G, bool BIAS>
+template <int D, int G, int BIAS>
 __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     const bf16_t* __restrict__ q, long ldq, bf16_t* __restrict__ out, long ldo,
     const bf16_t* __restrict__ kpool, const bf16_t* __restrict__ vpool,
@@ -77,7 +78,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     const int* __restrict__ seq_lens, int n_head, int n_kv_head, int page_size, float scale, int window,
     int single_below, const float* __restrict__ sinks, float softcap, const bf16_t* __restrict__ gate, long ldg,
     int keep_first, const float* __restrict__ score_bias, int chunked, const float* __restrict__ dist_bias,
-    int bias_len) {
+    int bias_len, const float* __restrict__ slopes) {
   constexpr int THREADS = 256 * G;
   constexpr int SB = PF_KT * G;    // keys staged per step
   // Key and value rows in LDS: as long as the head size where that is a power of two, the 16-byte
@@ -182,6 +183,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
   // by distance the scores are scaled when those are added)
   const float raw2 = scale * 1.4426950408889634f;
   const float sc2 = BIAS ? 1.0f : raw2;
+  const float slope2 = BIAS == 2 ? slopes[h] * 1.4426950408889634f : 0.f;
   const bool weigh = score_bias != nullptr;   // sigmoid weights, no softmax
   const float bias2 = weigh ? score_bias[h] * 1.4426950408889634f : 0.f;
   const int c_first = (kv_begin / SB) * SB;
@@ -201,7 +203,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
   __syncthreads();
   fetch(0);
   deposit(0);
-  if (BIAS) fill_bias(0);
+  if (BIAS == 1) fill_bias(0);
   if (n_steps > 1) fetch(1);
   __syncthreads();
   for (int b = 0; b < n_steps; ++b) {
@@ -210,7 +212,7 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
     int row_ahead = -1;
     if (b + 1 < n_steps) {
       deposit(buf ^ 1);   // its readers finished before the last barrier
-      if (BIAS) fill_bias(b + 1);
+      if (BIAS == 1) fill_bias(b + 1);
       if (b + 2 < n_steps) fetch(b + 2);
       // asked for now, written to the table at the end of this step's work
       if (b + 3 < n_steps && tid < SB) row_ahead = lookup(stretch_start(b + 3) + tid);
@@ -239,14 +241,26 @@ __global__ __launch_bounds__(256 * G) void prefill_attention_kernel(
           for (int kt = 0; kt < NKT; ++kt)
             s[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[kk][kt], qf[kk], s[kt], 0, 0, 0);
       }
-      if (BIAS) {
+      if (BIAS == 1) {
         const float* mine = bias_tab + buf * NB + grp * PF_KT + (PF_QT - 1 - (qwave * 16 + qi)) + g * 4;
 #pragma unroll
         for (int kt = 0; kt < NKT; ++kt)
 #pragma unroll
           for (int i = 0; i < 4; ++i) s[kt][i] = __builtin_fmaf(s[kt][i], raw2, mine[kt * 16 + i]);
       }
-      if (softcap > 0.f) {
+      if (BIAS == 2) {
+        // scaled and capped scores in units of log2 e, then minus slope * distance (the lane's first key's, and
+        // the keys' places behind it as constants)
+        const float first = slope2 * (float)(c0 + g * 4 - my_pos);
+        const float in = scale * __builtin_amdgcn_rcpf(softcap), cap2 = softcap * 1.4426950408889634f;
+#pragma unroll
+        for (int kt = 0; kt < NKT; ++kt)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float off = __builtin_fmaf(slope2, (float)(kt * 16 + i), first);
+            s[kt][i] = softcap > 0.f ? __builtin_fmaf(cap2, tanh_fast(s[kt][i] * in), off) : __builtin_fmaf(s[kt][i], raw2, off);
+          }
+      } else if (softcap > 0.f) {
         // capped scores: cap * tanh(s * scale / cap), kept in the raw scores' units (times cap / scale)
         const float in = scale * __builtin_amdgcn_rcpf(softcap), back = softcap * __builtin_amdgcn_rcpf(scale);
 #pragma unroll
@@ -401,13 +415,13 @@ extern "C" int mgpt_prefill_attention_bf16(
     const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, int n_req,
     int max_q_len, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     int single_below, const float* sinks, float softcap, const void* gate, long ldg, int keep_first,
-    const float* score_bias, int chunked, const float* dist_bias, int bias_len, hipStream_t stream) {
+    const float* score_bias, int chunked, const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream) {
   if (n_req == 0 || max_q_len == 0) return MGPT_OK;
   if (!q || !out || !kpool || !vpool || !block_tables || !cu_q || !seq_lens) return MGPT_ERR_NULL;
   if (n_req < 0 || max_q_len < 0 || n_head <= 0 || n_kv_head <= 0 || (n_head % n_kv_head) != 0 ||
       page_size <= 0 || max_blocks <= 0 || window < 0 || (ldq % 8) != 0 || (ldo % 4) != 0 ||
       (((size_t)out) & 7) != 0 || !(scale > 0.f) || keep_first < 0 || (score_bias && (sinks || softcap > 0.f)) ||
-      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)))
+      (dist_bias && (bias_len <= 0 || score_bias || softcap > 0.f)) || (slopes && (dist_bias || score_bias)))
     return MGPT_ERR_BAD_SHAPE;
   if (window == 0) keep_first = 0;
   if (n_req > 65535 || n_head > 65535) return MGPT_ERR_TOO_LARGE;
@@ -416,7 +430,7 @@ extern "C" int mgpt_prefill_attention_bf16(
   {                                                                                                                 \
     constexpr int sb = PF_KT * GG;                                                                                  \
     constexpr int kld = (DD & (DD - 1)) == 0 ? DD : DD + 8;                                                         \
-    constexpr int lds_bytes = 4 * sb * kld * (int)sizeof(bf16_t) + 4 * sb * 4 + (BI ? 2 * (sb + PF_QT) * 4 : 0);    \
+    constexpr int lds_bytes = 4 * sb * kld * (int)sizeof(bf16_t) + 4 * sb * 4 + (BI == 1 ? 2 * (sb + PF_QT) * 4 : 0);    \
     static bool allowed = false; /* more LDS than a kernel gets without asking */                                   \
     if (!allowed) {                                                                                                 \
       const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(prefill_attention_kernel<DD, GG, BI>), \
@@ -428,11 +442,13 @@ extern "C" int mgpt_prefill_attention_bf16(
                        (const bf16_t*)q, ldq, (bf16_t*)out, ldo, (const bf16_t*)kpool, (const bf16_t*)vpool,        \
                        block_tables, max_blocks, cu_q, seq_lens, n_head, n_kv_head, page_size, scale, window,       \
                        single_below, sinks, softcap, (const bf16_t*)gate, ldg, keep_first, score_bias, chunked,     \
-                       dist_bias, bias_len);                                                                        \
+                       dist_bias, bias_len, slopes);                                                                        \
   }
 #define PF_LAUNCH(DD, GG)                                               \
   {                                                                     \
-    if (dist_bias) PF_LAUNCH2(DD, GG, true) else PF_LAUNCH2(DD, GG, false) \
+    if (slopes) PF_LAUNCH2(DD, GG, 2)                                   \
+    else if (dist_bias) PF_LAUNCH2(DD, GG, 1)                           \
+    else PF_LAUNCH2(DD, GG, 0)                                          \
   }
   // Two wave groups halve the walk of a tile over its keys; one group leaves LDS for a second
   // workgroup on the compute unit.  The first serves a step with few tiles, the second one with many.

@@ -1,7 +1,9 @@
 // Gated feed-forwards and experts chosen by a table or by a router.
 //
 // gated unit: act[n][j] = silu(z[n][j]) * z[n][F + j], z = the joint product with the gate and up
-// matrices stacked, silu(v) = v * sigmoid(v), in 32-bit.
+// matrices stacked, silu(v) = v * sigmoid(v), in 32-bit.  Other units by number: relu(g) * u, gelu_tanh(g) * u, and
+// the clamped swish (number 3): with g' = min(g, limit) and u' = u held within -limit .. limit,
+// g' * sigmoid(sharpness * g') * (u' + 1).
 //
 // experts: a token's id picks a row of `top` experts from an integer table.  A (token, choice)
 // pair is one unit of work.  The route kernel sorts the pairs by expert into slots; every expert's
@@ -20,25 +22,32 @@
 #define EX_EPI_NONE 0
 #define EX_EPI_RELU2 5   // max(v, 0)^2
 
+template <bool FAST>
+__device__ __forceinline__ float gated_value(float g, float u, int kind, float limit, float sharpness) {
+  if (kind == 1) return fmaxf(g, 0.f) * u;
+  if (kind == 2) return (FAST ? gelu_tanh_fast(g) : gelu_tanh(g)) * u;
+  if (kind == 3) {
+    const float gc = fminf(g, limit), uc = fminf(fmaxf(u, -limit), limit) + 1.0f, a = sharpness * gc;
+    return (FAST ? gc * __builtin_amdgcn_rcpf(1.0f + __expf(-a)) : gc / (1.0f + expf(-a))) * uc;
+  }
+  return (FAST ? g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) : g / (1.0f + expf(-g))) * u;
+}
+
 template <typename T, bool FAST>
 __global__ void gated_unit_kernel(const T* __restrict__ z, long ldz, T* __restrict__ act, long lda, long total,
-                                  int hidden, int kind) {
+                                  int hidden, int kind, float limit, float sharpness) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= total) return;
   const long n = i / hidden;
   const int j = (int)(i - n * hidden);
   const float g = to_float<T>(z[n * ldz + j]), u = to_float<T>(z[n * ldz + hidden + j]);
-  float s;
-  if (kind == 1) s = fmaxf(g, 0.f);                                  // relu
-  else if (kind == 2) s = FAST ? gelu_tanh_fast(g) : gelu_tanh(g);
-  else s = FAST ? g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) : g / (1.0f + expf(-g));   // silu
-  act[n * lda + j] = from_float<T>(s * u);
+  act[n * lda + j] = from_float<T>(gated_value<FAST>(g, u, kind, limit, sharpness));
 }
 
 // the same for bfloat16 rows whose hidden size is a multiple of 8: a thread takes 8 units, 16 bytes a load
 template <bool FAST>
 __global__ void gated_unit_vec8_kernel(const bf16_t* __restrict__ z, long ldz, bf16_t* __restrict__ act, long lda, long total8,
-                                       int hidden8, int kind) {
+                                       int hidden8, int kind, float limit, float sharpness) {
   const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
   if (i >= total8) return;
   const long n = i / hidden8;
@@ -54,11 +63,7 @@ __global__ void gated_unit_vec8_kernel(const bf16_t* __restrict__ z, long ldz, b
     for (int half = 0; half < 2; ++half) {
       const float g = __uint_as_float(half ? (gw[e] & 0xffff0000u) : (gw[e] << 16));
       const float u = __uint_as_float(half ? (uw[e] & 0xffff0000u) : (uw[e] << 16));
-      float s;
-      if (kind == 1) s = fmaxf(g, 0.f);
-      else if (kind == 2) s = FAST ? gelu_tanh_fast(g) : gelu_tanh(g);
-      else s = FAST ? g * __builtin_amdgcn_rcpf(1.0f + __expf(-g)) : g / (1.0f + expf(-g));
-      r[half] = s * u;
+      r[half] = gated_value<FAST>(g, u, kind, limit, sharpness);
     }
     out[e] = pack_bf16x2(r[0], r[1]);
   }
@@ -66,20 +71,20 @@ __global__ void gated_unit_vec8_kernel(const bf16_t* __restrict__ z, long ldz, b
 }
 
 extern "C" int mgpt_gated_unit(const void* z, long ldz, void* act, long lda, int n_rows, int hidden, int dtype,
-                               int fast, int kind, hipStream_t stream) {
+                               int fast, int kind, float limit, float sharpness, hipStream_t stream) {
   if (n_rows == 0) return MGPT_OK;
   if (!z || !act) return MGPT_ERR_NULL;
-  if (n_rows < 0 || hidden <= 0 || ldz < 2L * hidden || lda < hidden || kind < 0 || kind > 2) return MGPT_ERR_BAD_SHAPE;
+  if (n_rows < 0 || hidden <= 0 || ldz < 2L * hidden || lda < hidden || kind < 0 || kind > 3) return MGPT_ERR_BAD_SHAPE;
   if (dtype == MGPT_BF16 && (hidden & 7) == 0 && (ldz & 7) == 0 && (lda & 7) == 0 && (((size_t)z | (size_t)act) & 15) == 0) {
     const long total8 = (long)n_rows * (hidden / 8);
     const long blocks8 = (total8 + 255) / 256;
     if (blocks8 > 0x7fffffffL) return MGPT_ERR_TOO_LARGE;
     if (fast)
       hipLaunchKernelGGL(gated_unit_vec8_kernel<true>, dim3((unsigned)blocks8), dim3(256), 0, stream, (const bf16_t*)z, ldz,
-                         (bf16_t*)act, lda, total8, hidden / 8, kind);
+                         (bf16_t*)act, lda, total8, hidden / 8, kind, limit, sharpness);
     else
       hipLaunchKernelGGL(gated_unit_vec8_kernel<false>, dim3((unsigned)blocks8), dim3(256), 0, stream, (const bf16_t*)z, ldz,
-                         (bf16_t*)act, lda, total8, hidden / 8, kind);
+                         (bf16_t*)act, lda, total8, hidden / 8, kind, limit, sharpness);
     return mgpt_last_error();
   }
   const long total = (long)n_rows * hidden;
@@ -87,7 +92,7 @@ extern "C" int mgpt_gated_unit(const void* z, long ldz, void* act, long lda, int
   if (blocks > 0x7fffffffL) return MGPT_ERR_TOO_LARGE;
   dim3 grid((unsigned)blocks), block(256);
 #define GU_LAUNCH(T, F) \
-  hipLaunchKernelGGL((gated_unit_kernel<T, F>), grid, block, 0, stream, (const T*)z, ldz, (T*)act, lda, total, hidden, kind)
+  hipLaunchKernelGGL((gated_unit_kernel<T, F>), grid, block, 0, stream, (const T*)z, ldz, (T*)act, lda, total, hidden, kind, limit, sharpness)
   if (dtype == MGPT_F32) {
     if (fast) GU_LAUNCH(float, true); else GU_LAUNCH(float, false);
   } else if (dtype == MGPT_BF16) {
@@ -128,12 +133,13 @@ extern "C" int mgpt_gather_rows(const void* src, long ld, const int* slot_token,
 }
 
 // A router: scores of every expert for a token, in float32 whatever the rows' dtype, and the `top`
-// largest.  logit[e] = w[e] . h; score = sigmoid(logit) (kind 0) or the logit itself (kind 1);
+// largest.  logit[e] = w[e] . h; score = sigmoid(logit) (kind 0), the logit itself (kind 1) or its softmax over all
+// experts (kind 2);
 // chosen[n][c] is the expert with the c-th largest score (of equal scores the lower number first) and
 // weight[n][c] its score.  Optional steps:
 //  - `correction` (a number per expert) is added to the scores that the choice goes by, not to the weights;
 //  - with n_groups > keep > 0 the experts form n_groups equal groups of neighbours, a group's rank is the sum of
-//    its two largest choice scores, and only experts of the `keep` best groups can be chosen;
+//    its `group_best` (1 or 2) largest choice scores, and only experts of the `keep` best groups can be chosen;
 //  - `normalise`: the chosen scores are divided by (their sum + 1e-20); every weight is multiplied by `scale`;
 //  - `extra` (one more row beside the matrix): extra_out[n] = sigmoid(extra . h).
 // One workgroup a token: its threads along the width in a fixed order, then the first wave picks the largest
@@ -165,7 +171,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
                                                           int kind, int* __restrict__ chosen, float* __restrict__ weight,
                                                           const float* __restrict__ correction, int n_groups, int keep,
                                                           int normalise, float scale, const WT* __restrict__ extra,
-                                                          float* __restrict__ extra_out) {
+                                                          float* __restrict__ extra_out, int group_best) {
   __shared__ float logit[EX_MAX_EXPERTS + 1];    // the extra row's comes last
   __shared__ float key[EX_MAX_EXPERTS];          // what the choice goes by
   __shared__ float rank[EX_MAX_EXPERTS];         // of a group
@@ -211,11 +217,27 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
     __syncthreads();
   }
   if (extra && threadIdx.x == 0) extra_out[n] = 1.0f / (1.0f + expf(-logit[n_experts]));
-  // (without a correction and groups the choice goes by the logits, in whose order the scores come)
+  // softmax: the largest logit and the sum over all experts, in every wave by itself (so the same in every thread)
+  float top_logit = 0.f, inv_total = 1.f;
+  if (kind == 2) {
+    float m = -INFINITY;
+    for (int e = lane; e < n_experts; e += 64) m = fmaxf(m, logit[e]);
+    top_logit = wave_max(m);
+    float total = 0.f;
+    for (int e = lane; e < n_experts; e += 64) total += expf(logit[e] - top_logit);
+    inv_total = 1.0f / wave_sum(total);
+  }
+  auto score_of = [&](float z) {
+    if (kind == 0) return 1.0f / (1.0f + expf(-z));
+    return kind == 1 ? z : expf(z - top_logit) * inv_total;
+  };
+  // (without a correction and groups, and with groups that rank by one expert, the choice goes by the logits, in
+  // whose order the scores come)
   const bool grouped = n_groups > keep && keep > 0;
+  const bool by_score = correction || (grouped && group_best > 1);
   for (int e = threadIdx.x; e < n_experts; e += 256) {
     const float z = logit[e];
-    key[e] = (correction || grouped) ? (kind == 0 ? 1.0f / (1.0f + expf(-z)) : z) + (correction ? correction[e] : 0.f) : z;
+    key[e] = by_score ? score_of(z) + (correction ? correction[e] : 0.f) : z;
   }
   __syncthreads();
   if (grouped) {
@@ -227,7 +249,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
         if (v > a) { b = a; a = v; }
         else if (v > b) b = v;
       }
-      rank[g] = size > 1 ? a + b : a;
+      rank[g] = size > 1 && group_best > 1 ? a + b : a;
     }
     __syncthreads();
     // a group stays if fewer than `keep` groups come before it (of equal ranks the lower number first)
@@ -256,7 +278,7 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
       cand = other < cand ? other : cand;
     }
     if (cand == 0x7fffffff) cand = 0;          // every score is -inf or NaN
-    const float score = kind == 0 ? 1.0f / (1.0f + expf(-logit[cand])) : logit[cand];
+    const float score = score_of(logit[cand]);
     sum += score;                                         // (the same in every lane)
     if (lane == 0) {
       chosen[(long)n * top + c] = cand;
@@ -278,12 +300,12 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
 extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
                                 int width, int n_experts, int top, int kind, int* chosen, float* weight,
                                 const float* correction, int n_groups, int keep, int normalise, float scale,
-                                const void* extra, float* extra_out, hipStream_t stream) {
+                                const void* extra, float* extra_out, int group_best, hipStream_t stream) {
   if (n_rows == 0) return MGPT_OK;
   if (!h || !w || !chosen || !weight) return MGPT_ERR_NULL;
   if (!dtype_ok(dtype) || !dtype_ok(w_dtype)) return MGPT_ERR_BAD_DTYPE;
   if (n_rows < 0 || width <= 0 || n_experts <= 0 || n_experts > EX_MAX_EXPERTS || top <= 0 || top > n_experts ||
-      (kind != 0 && kind != 1) || n_groups < 0 || keep < 0)
+      kind < 0 || kind > 2 || n_groups < 0 || keep < 0 || (group_best != 1 && group_best != 2))
     return MGPT_ERR_BAD_SHAPE;
   if (n_groups > keep && keep > 0 && (n_experts % n_groups || top > keep * (n_experts / n_groups))) return MGPT_ERR_BAD_SHAPE;
   if (extra && !extra_out) return MGPT_ERR_NULL;
@@ -295,11 +317,11 @@ extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* 
     if (vec)                                                                                                             \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, true, JJ>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,      \
                          (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
-                         normalise, scale, (const WT*)extra, extra_out);                                                 \
+                         normalise, scale, (const WT*)extra, extra_out, group_best);                                                 \
     else                                                                                                                 \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, false, 8>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,     \
                          (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
-                         normalise, scale, (const WT*)extra, extra_out);                                                 \
+                         normalise, scale, (const WT*)extra, extra_out, group_best);                                                 \
   }
   // up to eight rows at a time; a matrix of 9 to 12 (a few experts and the extra row) in one go
 #define ROUTER_LAUNCH(HT, WT)                                                                                            \

@@ -50,17 +50,20 @@ extern "C" int mgpt_rms_norm_store(const void* src, int dtype, long ld, const fl
 
 // A latent with a rotated part.  A cached row is [c: rank | kr: rot_dim | zeros up to row_width]: c as above,
 // kr one key part that all heads share, rotated by the token's position; a query head is [plain: head_dim |
-// rotated: rot_dim] and its rotated part is rotated in place.  Rotation of pairs (i, i + rot_dim / 2) by the angle
-// position * freq[i], cosine and sine both times rot_mag, in 32-bit.  One workgroup a token.  Without a pool
-// (a layer that reads another layer's latents) only the queries are rotated.
+// rotated: rot_dim] and its rotated part is rotated in place.  Rotation of pairs (i, i + rot_dim / 2), or with
+// `interleaved` (2i, 2i + 1), by the angle position * freq[i], cosine and sine both times rot_mag, in 32-bit.  One
+// workgroup a token.  Without a pool (a layer that reads another layer's latents, or queries that are projected later)
+// only the queries are rotated; with n_head 0 there are no queries to rotate.  With `cq_out` the cq_rank columns of z
+// at cq_off are RMS-normed with cq_gain into its rows: the latent that the queries are made from.
 #define LP_MAX_HALF 256
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(
     T* __restrict__ z, long ldz, int q_off, int n_head, int head_dim, int rot_dim, int c_off, int rank,
     const float* __restrict__ gain, float eps, const int* __restrict__ positions, const float* __restrict__ freq,
-    float rot_mag, T* __restrict__ pool, int row_width, const int* __restrict__ slot_mapping, int n_tokens) {
+    float rot_mag, T* __restrict__ pool, int row_width, const int* __restrict__ slot_mapping, int n_tokens, int interleaved,
+    int cq_off, int cq_rank, const float* __restrict__ cq_gain, T* __restrict__ cq_out, long ld_cq) {
   __shared__ float cos_s[LP_MAX_HALF], sin_s[LP_MAX_HALF];
-  __shared__ float red_s[4];
+  __shared__ float red_s[8];
   const int n = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int half = rot_dim / 2;
   const float p = (float)positions[n];
@@ -71,54 +74,74 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
   }
   T* row = z + (long)n * ldz;
   const int slot = pool ? slot_mapping[n] : -1;
-  float ss = 0.f;
+  float ss = 0.f, sq = 0.f;
   if (slot >= 0)
     for (int c = tid; c < rank; c += 256) {
       const float v = to_float<T>(row[c_off + c]);
       ss = fmaf(v, v, ss);
     }
+  if (cq_out)
+    for (int c = tid; c < cq_rank; c += 256) {
+      const float v = to_float<T>(row[cq_off + c]);
+      sq = fmaf(v, v, sq);
+    }
   ss = wave_sum(ss);
-  if (lane == 0) red_s[wave] = ss;
+  sq = wave_sum(sq);
+  if (lane == 0) {
+    red_s[wave] = ss;
+    red_s[4 + wave] = sq;
+  }
   __syncthreads();
+  // (the pair's channels)
+  auto lo = [&](int i) { return interleaved ? 2 * i : i; };
+  auto hi = [&](int i) { return interleaved ? 2 * i + 1 : i + half; };
   for (int idx = tid; idx < n_head * half; idx += 256) {
     const int h = idx / half, i = idx - h * half;
     T* at = row + q_off + (long)h * (head_dim + rot_dim) + head_dim;
-    const float u = to_float<T>(at[i]), w = to_float<T>(at[i + half]);
-    at[i] = from_float<T>(u * cos_s[i] - w * sin_s[i]);
-    at[i + half] = from_float<T>(w * cos_s[i] + u * sin_s[i]);
+    const float u = to_float<T>(at[lo(i)]), w = to_float<T>(at[hi(i)]);
+    at[lo(i)] = from_float<T>(u * cos_s[i] - w * sin_s[i]);
+    at[hi(i)] = from_float<T>(w * cos_s[i] + u * sin_s[i]);
+  }
+  if (cq_out) {
+    const float inv = 1.0f / sqrtf(((red_s[4] + red_s[5]) + (red_s[6] + red_s[7])) / (float)cq_rank + eps);
+    for (int c = tid; c < cq_rank; c += 256)
+      cq_out[(long)n * ld_cq + c] = from_float<T>(to_float<T>(row[cq_off + c]) * inv * cq_gain[c]);
   }
   if (slot < 0) return;
   const float inv = 1.0f / sqrtf(((red_s[0] + red_s[1]) + (red_s[2] + red_s[3])) / (float)rank + eps);
   T* dst = pool + (long)slot * row_width;
   for (int c = tid; c < rank; c += 256) dst[c] = from_float<T>(to_float<T>(row[c_off + c]) * inv * gain[c]);
   for (int i = tid; i < half; i += 256) {
-    const float u = to_float<T>(row[c_off + rank + i]), w = to_float<T>(row[c_off + rank + i + half]);
-    dst[rank + i] = from_float<T>(u * cos_s[i] - w * sin_s[i]);
-    dst[rank + i + half] = from_float<T>(w * cos_s[i] + u * sin_s[i]);
+    const float u = to_float<T>(row[c_off + rank + lo(i)]), w = to_float<T>(row[c_off + rank + hi(i)]);
+    dst[rank + lo(i)] = from_float<T>(u * cos_s[i] - w * sin_s[i]);
+    dst[rank + hi(i)] = from_float<T>(w * cos_s[i] + u * sin_s[i]);
   }
   for (int c = rank + rot_dim + tid; c < row_width; c += 256) dst[c] = from_float<T>(0.f);
 }
 
 // z: the step's projected rows (queries at q_off, n_head heads of head_dim + rot_dim; the latent's rank + rot_dim
-// columns at c_off); pool: the latent pages with rows of row_width >= rank + rot_dim values, or null.
+// columns at c_off; the cq_rank columns of the queries' latent at cq_off); pool: the latent pages with rows of
+// row_width >= rank + rot_dim values, or null; cq_out: rows of ld_cq >= cq_rank values, or null.
 extern "C" int mgpt_latent_prepare(void* z, int dtype, long ldz, int q_off, int n_head, int head_dim, int rot_dim,
                                    int c_off, int rank, const float* gain, float eps, const int* positions,
                                    const float* freq, float rot_mag, void* pool, int row_width,
-                                   const int* slot_mapping, int n_tokens, hipStream_t stream) {
+                                   const int* slot_mapping, int n_tokens, int interleaved, int cq_off, int cq_rank,
+                                   const float* cq_gain, void* cq_out, long ld_cq, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
-  if (!z || !positions || !freq || (pool && (!gain || !slot_mapping))) return MGPT_ERR_NULL;
-  if (n_tokens < 0 || n_head <= 0 || head_dim < 0 || rot_dim <= 0 || (rot_dim & 1) || rot_dim / 2 > LP_MAX_HALF ||
+  if (!z || !positions || !freq || (pool && (!gain || !slot_mapping)) || (cq_out && !cq_gain)) return MGPT_ERR_NULL;
+  if (n_tokens < 0 || n_head < 0 || head_dim < 0 || rot_dim <= 0 || (rot_dim & 1) || rot_dim / 2 > LP_MAX_HALF ||
       q_off < 0 || ldz < q_off + (long)n_head * (head_dim + rot_dim) ||
-      (pool && (rank <= 0 || row_width < rank + rot_dim || c_off < 0 || ldz < c_off + rank + rot_dim)))
+      (pool && (rank <= 0 || row_width < rank + rot_dim || c_off < 0 || ldz < c_off + rank + rot_dim)) ||
+      (cq_out && (cq_rank <= 0 || cq_off < 0 || ldz < cq_off + cq_rank || ld_cq < cq_rank || cq_out == z)))
     return MGPT_ERR_BAD_SHAPE;
   if (dtype == MGPT_F32)
     hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, (float*)z, ldz, q_off, n_head,
                        head_dim, rot_dim, c_off, rank, gain, eps, positions, freq, rot_mag, (float*)pool, row_width,
-                       slot_mapping, n_tokens);
+                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (float*)cq_out, ld_cq);
   else if (dtype == MGPT_BF16)
     hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, dim3(n_tokens), dim3(256), 0, stream, (bf16_t*)z, ldz, q_off, n_head,
                        head_dim, rot_dim, c_off, rank, gain, eps, positions, freq, rot_mag, (bf16_t*)pool, row_width,
-                       slot_mapping, n_tokens);
+                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (bf16_t*)cq_out, ld_cq);
   else
     return MGPT_ERR_BAD_DTYPE;
   return mgpt_last_error();

@@ -11,20 +11,20 @@ int mgpt_paged_attention_split_bf16(const void* q, long ldq, void* out, long ldo
     void* vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const int*
     q_req, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias, int chunked,
-    const float* dist_bias, int bias_len, hipStream_t stream);
+    const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream);
 // attention_decode.hip
 int mgpt_paged_attention_split_fast_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool,
     const void* vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, const
     int* q_req, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window,
     const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float* score_bias, int chunked,
-    const float* dist_bias, int bias_len, hipStream_t stream);
+    const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream);
 // attention_decode_wide.hip
 int mgpt_paged_attention_decode_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool, const
     void* vpool, const int* block_tables, int max_blocks, const int* positions, const int* q_req, const int*
     cu_q, int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, int num_pages, float scale,
     int window, int identity, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const
     float* score_bias, int chunked,
-    const float* dist_bias, int bias_len, hipStream_t stream);
+    const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream);
 // attention_generic.hip
 int mgpt_kv_write(const void* qkv, int dtype, long ld, int k_off, int v_off, void* kpool, void* vpool, const
     int* slot_mapping, int n_tokens, int n_kv_head, int head_dim, int page_size, hipStream_t stream);
@@ -34,14 +34,14 @@ int mgpt_paged_attention_generic(const void* q, long ldq, void* out, long ldo, c
     int n_tokens, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window, int dtype,
     int fast_exp, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float*
     score_bias, int chunked,
-    const float* dist_bias, int bias_len, hipStream_t stream);
+    const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream);
 // attention_prefill.hip
 int mgpt_prefill_attention_bf16(const void* q, long ldq, void* out, long ldo, const void* kpool, const void*
     vpool, const int* block_tables, int max_blocks, const int* cu_q, const int* seq_lens, int n_req, int
     max_q_len, int n_head, int n_kv_head, int head_dim, int page_size, float scale, int window, int
     single_below, const float* sinks, float softcap, const void* gate, long ldg, int keep_first, const float*
     score_bias, int chunked,
-    const float* dist_bias, int bias_len, hipStream_t stream);
+    const float* dist_bias, int bias_len, const float* slopes, hipStream_t stream);
 // embed_norm.hip
 int mgpt_embed(const int* ids, const int* pos, const void* tok, const void* postab, float* x, int n_tokens,
     int width, int table_dtype, hipStream_t stream);
@@ -137,7 +137,8 @@ int mgpt_rms_norm_store(const void* src, int dtype, long ld, const float* gain, 
     slot_mapping, int n_tokens, int rank, hipStream_t stream);
 int mgpt_latent_prepare(void* z, int dtype, long ldz, int q_off, int n_head, int head_dim, int rot_dim, int c_off,
     int rank, const float* gain, float eps, const int* positions, const float* freq, float rot_mag, void* pool,
-    int row_width, const int* slot_mapping, int n_tokens, hipStream_t stream);
+    int row_width, const int* slot_mapping, int n_tokens, int interleaved, int cq_off, int cq_rank, const float* cq_gain,
+    void* cq_out, long ld_cq, hipStream_t stream);
 int mgpt_heads_linear(const void* a, long lda, const void* w, void* out, long ldo, const void* gate, long ldg,
     int n_rows, int n_head, int n_out, int k_dim, int dtype, int fast, hipStream_t stream);
 int mgpt_heads_linear_mfma(const void* a, long lda, const void* w, void* out, long ldo, const void* gate, long ldg,
@@ -155,7 +156,7 @@ int mgpt_xielu(const void* z, long ldz, void* out, long ldo, int dtype, const fl
     int fast, hipStream_t stream);
 // experts.hip
 int mgpt_gated_unit(const void* z, long ldz, void* act, long lda, int n_rows, int hidden, int dtype, int fast,
-    int kind, hipStream_t stream);
+    int kind, float limit, float sharpness, hipStream_t stream);
 int mgpt_expert_route(const int* ids, const int* q_req, const int* table, int top, int n_rows, int n_experts,
     int* slot_token, int* slot_pair, int* pair_slot, int* tile_expert, int n_slots, int n_tiles, int tile_rows,
     hipStream_t stream);
@@ -163,7 +164,8 @@ int mgpt_gather_rows(const void* src, long ld, const int* slot_token, void* sort
     hipStream_t stream);
 int mgpt_router_topk(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
     int width, int n_experts, int top, int kind, int* chosen, float* weight, const float* correction, int n_groups,
-    int keep, int normalise, float scale, const void* extra, float* extra_out, hipStream_t stream);
+    int keep, int normalise, float scale, const void* extra, float* extra_out, int group_best,
+    hipStream_t stream);
 int mgpt_gather_scale_rows(const void* src, int dtype, long ld, const int* slot_token, const int* slot_pair,
     const float* pair_weight, void* sorted, long lds, int n_slots, int width, hipStream_t stream);
 int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int*
@@ -184,6 +186,7 @@ int mgpt_rms_post_norm(float* y0, float* y1, float* y2, float* y3, const float* 
     const float* g3, int n_branches, float coef, int join_unit, float* x, const float* gain_post, const float* scale_post,
     float offset, float eps, float mult, const float* gain_next, void* h, int h_dtype, int n_rows, int width,
     hipStream_t stream);
+int mgpt_cast_rows(const float* x, long ldx, void* out, int out_dtype, long ldo, int n_rows, int width, hipStream_t stream);
 // gated_state.hip
 int mgpt_gated_state(const void* z, int dtype, long ldz, int q_off, int k_off, int v_off, int n_head, int n_group,
     int head_dim, int value_dim, const void* a, int a_dtype, long lda, int a_off, int mode, float q_scale, float inv_tau,
@@ -194,6 +197,11 @@ int mgpt_gated_state_chunked(const void* z, int dtype, long ldz, int q_off, int 
                              float q_scale, float inv_tau, const float* dt_bias, const float* a_log, const float* skip,
                              float* state, long ld_state, const int* state_slots, const int* cu_q, int n_req, int n_tokens,
                              const int* positions, float* qkg, float* out, long ldo, hipStream_t stream);
+// diagonal_state.hip
+int mgpt_diagonal_state(const void* u, int u_dtype, long ldu, const void* g, int g_dtype, long ldg, const float* r_bias,
+    const float* i_bias, const float* decay, int block, const void* y, int y_dtype, long ldy, int y_off, float* state, long ld_state,
+    const int* state_slots, const int* cu_q, const int* positions, int n_req, int n_tokens, int channels, float* scratch,
+    long scratch_floats, void* out, int out_dtype, long ldo, hipStream_t stream);
 // delta_state.hip
 int mgpt_delta_state(const void* x, int dtype, long ldx, int q_off, int k_off, int v_off, const void* z, long ldz,
     int b_off, int a_off, int gate_off, int n_head, int n_group, int head_dim, int value_dim, float q_scale,
@@ -214,7 +222,7 @@ int mgpt_qk_prepare(void* z, int dtype, long ldz, int q_off, int k_off, int v_of
     int head_dim, int value_dim, int head_stride, const int* positions, const float* freq, int rot_dims, float norm_eps,
     const float* mix_lambda, void* v_other, long ld_other, int mix_mode, void* kpool, void* vpool,
     const int* slot_mapping, int page_size, int n_tokens, int norm_mode, const float* q_norm_w, const float* k_norm_w,
-    int v_from_k, float rot_mag, hipStream_t stream);
+    int v_from_k, float rot_mag, int interleaved, float temp_coef, int temp_every, hipStream_t stream);
 // decay_state.hip
 int mgpt_decay_state(const void* z, int dtype, long ldz, int q_off, int k_off, int v_off, int g_off, int n_head,
     int head_dim, int value_dim, int act, const int* positions, const float* freq, int rot_dims, float k_scale,
@@ -279,6 +287,8 @@ int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_st
   X(mgpt_linear_mfma_grouped) \
   X(mgpt_rms_norm) \
   X(mgpt_rms_post_norm) \
+  X(mgpt_cast_rows) \
+  X(mgpt_diagonal_state) \
   X(mgpt_qk_prepare) \
   X(mgpt_decay_state) \
   X(mgpt_decay_state_chunked) \

@@ -6,13 +6,14 @@
 //    a = position * freq[i].  freq is a float32 table made by the host (so base, scaling and any
 //    other rule for the frequencies are the caller's); position, angle, sine and cosine are
 //    float32, with the full-range sine and cosine.  The other channels pass unchanged.
-//    With `rot_mag` every cosine and sine is multiplied by that number;
+//    With `rot_mag` every cosine and sine is multiplied by that number; with `interleaved` the pairs are (2i, 2i + 1);
 //  - optionally each query and key head divided by its root mean square over its `head_dim` real
 //    channels (eps inside the root), after the rotation (norm_mode 0 with norm_eps >= 0);
 //  - or, before the rotation, an RMS norm with weights: head by head with one weight vector [head_dim] for all
 //    query heads and one for all key heads (norm_mode 1), or over all of a token's query channels at once (and
 //    all of its key channels) with weights [heads * head_dim] (norm_mode 2);
 //  - with `v_from_k` the values are the keys as projected (before norm and rotation), and z holds no values;
+//  - with temp_every > 0 a query at position p is multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1);
 //  - optionally values mixed with those that another layer made for the same token:
 //    v <- (1 - lambda) v + lambda v_other (mode 2), or kept for such layers (mode 1);
 //  - queries written back in place; keys and values stored into their page (slot_mapping).
@@ -37,7 +38,7 @@ __global__ __launch_bounds__(1024) void qk_prepare_kernel(
     float norm_eps, const float* __restrict__ mix_lambda, T* __restrict__ v_other, long ld_other, int mix_mode,
     T* __restrict__ kpool, T* __restrict__ vpool, const int* __restrict__ slot_mapping, int page_size,
     int n_tokens, int norm_mode, const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, int v_from_k,
-    float rot_mag, int stash) {
+    float rot_mag, int stash, int interleaved, float temp_coef, int temp_every) {
   __shared__ float cos_s[QKP_MAX_DIM / 2], sin_s[QKP_MAX_DIM / 2];
   __shared__ float red_s[2 * QKP_MAX_WAVES];
   extern __shared__ float head_s[];    // [waves][head_dim]: the head a wave is working on; with `stash` behind it
@@ -53,6 +54,7 @@ __global__ __launch_bounds__(1024) void qk_prepare_kernel(
       sin_s[i] = sinf(a) * rot_mag;
     }
   }
+  const float q_times = temp_every > 0 ? 1.0f + temp_coef * logf((float)((positions[n] + 1) / temp_every + 1)) : 1.0f;
   const long row = (long)n * ldz;
   float whole_q = 1.0f, whole_k = 1.0f;   // norm_mode 2: what all query (key) channels of the token are multiplied by
   if (norm_mode == 2) {
@@ -118,9 +120,10 @@ __global__ __launch_bounds__(1024) void qk_prepare_kernel(
     }
     if (freq) {
       for (int i = lane; i < half; i += 64) {
-        const float u = s[i], w = s[i + half], co = cos_s[i], si = sin_s[i];
-        s[i] = u * co - w * si;
-        s[i + half] = w * co + u * si;
+        const int a = interleaved ? 2 * i : i, b = interleaved ? 2 * i + 1 : i + half;
+        const float u = s[a], w = s[b], co = cos_s[i], si = sin_s[i];
+        s[a] = u * co - w * si;
+        s[b] = w * co + u * si;
       }
       __builtin_amdgcn_wave_barrier();
     }
@@ -131,6 +134,7 @@ __global__ __launch_bounds__(1024) void qk_prepare_kernel(
       r = 1.0f / sqrtf(wave_sum(ss) / (float)head_dim + norm_eps);
     }
     if (is_q) {
+      r *= q_times;
       for (int c = lane; c < head_dim; c += 64) qk_store<T>(z, src + c, s[c] * r);
     } else if (slot >= 0) {
       for (int c = lane; c < head_stride; c += 64) qk_store<T>(kpool, dst + c, c < head_dim ? s[c] * r : 0.f);
@@ -162,12 +166,12 @@ extern "C" int mgpt_qk_prepare(void* z, int dtype, long ldz, int q_off, int k_of
                                float norm_eps, const float* mix_lambda, void* v_other, long ld_other, int mix_mode,
                                void* kpool, void* vpool, const int* slot_mapping, int page_size, int n_tokens,
                                int norm_mode, const float* q_norm_w, const float* k_norm_w, int v_from_k, float rot_mag,
-                               hipStream_t stream) {
+                               int interleaved, float temp_coef, int temp_every, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
-  if (!z || (freq && !positions) || (kpool && (!vpool || !slot_mapping))) return MGPT_ERR_NULL;
+  if (!z || ((freq || temp_every > 0) && !positions) || (kpool && (!vpool || !slot_mapping))) return MGPT_ERR_NULL;
   if (!dtype_ok(dtype)) return MGPT_ERR_BAD_DTYPE;
   if (n_tokens < 0 || n_head <= 0 || n_kv_head <= 0 || head_dim <= 0 || head_dim > QKP_MAX_DIM || head_stride < head_dim || value_dim <= 0 || value_dim > head_stride ||
-      rot_dims < 0 || (rot_dims & 1) || rot_dims > head_dim || (kpool && page_size <= 0) || mix_mode < 0 || mix_mode > 2)
+      rot_dims < 0 || (rot_dims & 1) || rot_dims > head_dim || (kpool && page_size <= 0) || mix_mode < 0 || mix_mode > 2 || temp_every < 0)
     return MGPT_ERR_BAD_SHAPE;
   if (mix_mode && (!v_other || (mix_mode == 2 && !mix_lambda))) return MGPT_ERR_NULL;
   if (norm_mode < 0 || norm_mode > 2 || (norm_mode && !(norm_eps >= 0.f)) || (v_from_k && (mix_mode || value_dim != head_dim)))
@@ -184,7 +188,8 @@ extern "C" int mgpt_qk_prepare(void* z, int dtype, long ldz, int q_off, int k_of
   hipLaunchKernelGGL(qk_prepare_kernel<T>, dim3(n_tokens), dim3(64 * waves), (waves + (stash ? heads : 0)) * head_dim * sizeof(float), \
                      stream, (T*)z, ldz, q_off, k_off, v_off, n_head, n_kv_head, head_dim, value_dim, head_stride, positions,  \
                      rot_dims ? freq : nullptr, rot_dims, norm_eps, mix_lambda, (T*)v_other, ld_other, mix_mode, (T*)kpool,    \
-                     (T*)vpool, slot_mapping, page_size, n_tokens, norm_mode, q_norm_w, k_norm_w, v_from_k, rot_mag, stash)
+                     (T*)vpool, slot_mapping, page_size, n_tokens, norm_mode, q_norm_w, k_norm_w, v_from_k, rot_mag, stash, interleaved,    \
+                     temp_coef, temp_every)
   if (dtype == MGPT_F32) QKP_LAUNCH(float);
   else QKP_LAUNCH(bf16_t);
 #undef QKP_LAUNCH

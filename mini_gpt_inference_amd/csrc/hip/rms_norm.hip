@@ -14,7 +14,7 @@
 //   y = sum_b coef * unit(y_b) * gain_b          (only with several branches; else y = y_0;
 //                                                 join_unit = 0: sum_b coef * y_b * gain_b, a weighted sum)
 //   x += mult * unit(y) * (offset + gain_post) (* scale_post, a scale per channel)
-//   h = unit(x) * (offset + gain_next)           (if there is a next norm)
+//   h = unit(x) * (offset + gain_next)           (if there is a next norm; without its gain, h = x if there is an h)
 //   y_b = 0                                       (ready for the next sublayer's additions)
 // Sums of squares are taken in float32 in a fixed order (lane-strided, then across the wave, then
 // across the waves in order), so a row's result does not depend on the other rows of the step.
@@ -186,7 +186,11 @@ __global__ __launch_bounds__(256) void rms_post_norm_kernel(RmsBranches br, int 
     y0[c] = 0.f;
     sx = fmaf(v, v, sx);
   }
-  if (!gain_next) return;
+  if (!gain_next) {
+    if (h)
+      for (int c = threadIdx.x; c < width; c += 256) store_f(h, h_dtype, base + c, x[base + c]);
+    return;
+  }
   const float rx = 1.0f / sqrtf(block_sum_256(sx, scratch) / (float)width + eps);
   for (int c = threadIdx.x; c < width; c += 256)
     store_f(h, h_dtype, base + c, x[base + c] * rx * (offset + gain_next[c]));
@@ -251,7 +255,16 @@ __global__ __launch_bounds__(256) void rms_post_norm_row_kernel(RmsBranches br, 
       sx = fmaf(xv[u], xv[u], sx);
     }
   }
-  if (!gain_next) return;
+  if (!gain_next) {
+    if (h) {
+#pragma unroll
+      for (int u = 0; u < PT; ++u) {
+        const int c = threadIdx.x + u * 256;
+        if (c < width) store_f(h, h_dtype, base + c, xv[u]);
+      }
+    }
+    return;
+  }
   const float rx = 1.0f / sqrtf(block_sum_256(sx, scratch) / (float)width + eps);
 #pragma unroll
   for (int u = 0; u < PT; ++u) {
@@ -270,7 +283,7 @@ extern "C" int mgpt_rms_post_norm(float* y0, float* y1, float* y2, float* y3, co
   if (n_rows == 0) return MGPT_OK;
   if (!x || !y0 || !gain_post || (gain_next && !h)) return MGPT_ERR_NULL;
   if (n_rows < 0 || width <= 0 || n_branches < 1 || n_branches > RMS_MAX_BRANCHES) return MGPT_ERR_BAD_SHAPE;
-  if (gain_next && !dtype_ok(h_dtype)) return MGPT_ERR_BAD_DTYPE;
+  if (h && !dtype_ok(h_dtype)) return MGPT_ERR_BAD_DTYPE;
   RmsBranches br = {{y0, y1, y2, y3}, {g0, g1, g2, g3}};
   for (int b = 0; b < n_branches; ++b)
     if (!br.y[b] || (n_branches > 1 && !br.gain[b])) return MGPT_ERR_NULL;
@@ -286,5 +299,24 @@ extern "C" int mgpt_rms_post_norm(float* y0, float* y1, float* y2, float* y3, co
     hipLaunchKernelGGL(rms_post_norm_kernel, dim3(n_rows), dim3(256), 0, stream, br, n_branches, coef, join_unit, x, gain_post,
                        scale_post, offset, eps, mult, gain_next, h, h_dtype, n_rows, width);
 #undef RPN_ROW
+  return mgpt_last_error();
+}
+
+// float32 rows in another storage type (the residual as the next product's operand, where no norm stands between)
+__global__ __launch_bounds__(256) void cast_rows_kernel(const float* __restrict__ x, long ldx, void* __restrict__ out, int out_dtype,
+                                                        long ldo, int width) {
+  const int row = blockIdx.x;
+  for (int c = blockIdx.y * 256 + threadIdx.x; c < width; c += 256 * gridDim.y)
+    store_f(out, out_dtype, (long)row * ldo + c, x[(long)row * ldx + c]);
+}
+
+extern "C" int mgpt_cast_rows(const float* x, long ldx, void* out, int out_dtype, long ldo, int n_rows, int width,
+                              hipStream_t stream) {
+  if (n_rows == 0) return MGPT_OK;
+  if (!x || !out) return MGPT_ERR_NULL;
+  if (n_rows < 0 || width <= 0 || ldx < width || ldo < width) return MGPT_ERR_BAD_SHAPE;
+  if (!dtype_ok(out_dtype)) return MGPT_ERR_BAD_DTYPE;
+  const int cols = (width + 1023) / 1024;
+  hipLaunchKernelGGL(cast_rows_kernel, dim3(n_rows, cols < 64 ? cols : 64), dim3(256), 0, stream, x, ldx, out, out_dtype, ldo, width);
   return mgpt_last_error();
 }

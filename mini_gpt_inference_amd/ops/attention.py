@@ -57,21 +57,24 @@ def _padded_mixed_step(ctx, q, out, k_pool, v_pool, group, n_head: int, scale: f
 
 def paged_attention(ctx, q: torch.Tensor, out: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
                     group, n_head: int, scale: float, window: int, sinks=None, softcap: float = 0.0,
-                    gate=None, keep_first: int = 0, score_bias=None, chunked: bool = False, dist_bias=None) -> None:
+                    gate=None, keep_first: int = 0, score_bias=None, chunked: bool = False, dist_bias=None,
+                    slopes=None) -> None:
     """Attention of the step's tokens (rows of q) over their requests' pages.  softcap > 0: scores
     pass cap * tanh(score / cap) before the softmax.  gate ([tokens, >= heads], the queries' dtype): a head's
     output is multiplied by sigmoid(gate[token][head]).  keep_first: behind a window a query also sees the keys
     at positions below keep_first.  score_bias (float32 [heads]): no softmax; a visible key's weight is
     sigmoid(score + score_bias[head]).  chunked: the window is the size of chunks counted from position 0, and a
     query sees its own chunk.  dist_bias (float32 [heads, L]): the number for the key's distance (the last one for
-    every distance from L - 1 on) is added to the scaled score.
+    every distance from L - 1 on) is added to the scaled score.  slopes (float32 [heads]): slope * distance is taken off
+    the scaled and capped score.
 
     On the bfloat16 path a decode-only step (token n is request n's one token) uses the kernel
     laid out for a decode step's latency, steps with prompt portions the MFMA tile kernel and the
     rest the kernel that splits a query's keys over four waves; the 32-bit path and every shape
     those refuse use the general kernel, whose order of sums depends only on a query's position."""
     n, r = ctx.n_rows, ctx.cu_q.numel() - 1
-    mask = {"keep_first": keep_first, "score_bias": score_bias, "chunked": chunked, "dist_bias": dist_bias}
+    mask = {"keep_first": keep_first, "score_bias": score_bias, "chunked": chunked, "dist_bias": dist_bias,
+            "slopes": slopes}
     if q.dtype == torch.bfloat16 and not ctx.exact:
         if ctx.decode_only and kernels.paged_attention_decode_bf16(
                 q, out, k_pool, v_pool, group.block_tables, ctx.positions, ctx.q_req, n, n_head, scale, window,

@@ -181,11 +181,11 @@ def kv_write(qkv: torch.Tensor, k_off: int, v_off: int, k_pool: torch.Tensor, v_
 
 
 def _mask_args(keep_first: int, score_bias: Optional[torch.Tensor], n_head: int, sinks, softcap: float,
-               chunked: bool = False, dist_bias: Optional[torch.Tensor] = None):
+               chunked: bool = False, dist_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None):
     """(first positions that a window keeps, pointer of the per-head number added to a score before its sigmoid,
-    whether the window is a chunk, pointer and row length of the numbers by distance): the optional arguments
+    whether the window is a chunk, pointer and row length of the numbers by distance, pointer of the slopes): the optional arguments
     behind the gate's.  With score_bias the weights are sigmoids and not a softmax, so sinks and a score cap do not
-    go with it; numbers by distance go with neither score_bias nor a score cap."""
+    go with it; numbers by distance go with neither score_bias nor a score cap; slopes go with neither of the two."""
     _need(int(keep_first) >= 0, "keep_first must not be negative")
     if score_bias is not None:
         _need(score_bias.is_cuda and score_bias.dtype == torch.float32 and score_bias.is_contiguous()
@@ -198,7 +198,11 @@ def _mask_args(keep_first: int, score_bias: Optional[torch.Tensor], n_head: int,
               "dist_bias must be dense float32 [n_head, distances] on the GPU")
         _need(score_bias is None and not softcap > 0.0, "numbers by distance go with neither score_bias nor a score cap")
         bias_len = dist_bias.shape[1]
-    return int(keep_first), _ptr(score_bias), 1 if chunked else 0, _ptr(dist_bias), bias_len
+    if slopes is not None:
+        _need(slopes.is_cuda and slopes.dtype == torch.float32 and slopes.is_contiguous() and slopes.numel() == n_head,
+              "slopes must be float32 [n_head] on the GPU")
+        _need(score_bias is None and dist_bias is None, "slopes go with neither score_bias nor numbers by distance")
+    return int(keep_first), _ptr(score_bias), 1 if chunked else 0, _ptr(dist_bias), bias_len, _ptr(slopes)
 
 
 def _gate_args(gate: Optional[torch.Tensor], q: torch.Tensor, n_tokens: int, n_head: int):
@@ -237,14 +241,15 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Te
                             window: int = 0, fast_exp: bool = False, sinks: Optional[torch.Tensor] = None,
                             softcap: float = 0.0, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
                             score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
-                            dist_bias: Optional[torch.Tensor] = None) -> None:
+                            dist_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> None:
     """Causal attention of the step's tokens over their requests' pages (any q_len, any dtype).
     sinks: float32 [n_head], one more term exp(sinks[h]) in every softmax denominator of head h.
     softcap > 0: every score becomes softcap * tanh(score / softcap) before the softmax.
     keep_first: behind a window a query also sees the keys at positions below it.  score_bias: float32 [n_head];
     a visible key's weight is sigmoid(score + score_bias[h]), not normalised over the keys.  chunked: `window` is the
     size of chunks counted from position 0, and a query sees its own chunk.  dist_bias: float32 [n_head, L], the
-    number at [h, min(i - j, L - 1)] is added to the scaled score of query i and key j."""
+    number at [h, min(i - j, L - 1)] is added to the scaled score of query i and key j.  slopes: float32 [n_head],
+    slopes[h] * (i - j) is taken off the scaled and capped score."""
     n_kv_head, page_size, head_dim = _check_attention_args(
         q, out, k_pool, v_pool, block_tables, cu_q, seq_lens, q_req, n_tokens, n_req, n_head)
     _need(head_dim <= 1024, f"head size {head_dim} exceeds the kernel's limit of 1024")
@@ -253,7 +258,7 @@ def paged_attention_generic(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Te
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), _ptr(q_req), n_tokens, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), _dtype_code(q), int(fast_exp), _ptr(sinks), float(softcap), *_gate_args(gate, q, n_tokens, n_head),
-        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
+        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias, slopes), _stream())
     _check(rc, "paged_attention_generic")
 
 
@@ -530,7 +535,7 @@ def paged_attention_split_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch
                                window: int = 0, fast: bool = True, sinks: Optional[torch.Tensor] = None,
                                softcap: float = 0.0, gate: Optional[torch.Tensor] = None, keep_first: int = 0,
                                score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
-                               dist_bias: Optional[torch.Tensor] = None) -> bool:
+                               dist_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> bool:
     """bfloat16 attention with each (token, head)'s keys split over four waves.  False if refused.
     fast=False keeps to the variant that takes every head size."""
     if q.dtype != torch.bfloat16:
@@ -547,7 +552,7 @@ def paged_attention_split_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), _ptr(q_req), n_tokens, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), _ptr(sinks), float(softcap), *_gate_args(gate, q, n_tokens, n_head),
-        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
+        *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias, slopes), _stream())
     if rc == -2:
         return False
     _check(rc, "paged_attention_split_bf16")
@@ -561,7 +566,7 @@ def paged_attention_decode_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torc
                                 sinks: Optional[torch.Tensor] = None, softcap: float = 0.0,
                                 gate: Optional[torch.Tensor] = None, keep_first: int = 0,
                                 score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
-                                dist_bias: Optional[torch.Tensor] = None) -> bool:
+                                dist_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> bool:
     """bfloat16 attention for single tokens (one query per request and step), keys split over eight
     waves.  positions[n] is token n's absolute position, q_req[n] its block table row or -1 for a
     padded token; identity=True promises q_req[n] in (n, -1).  With cu_q (the requests' token offsets;
@@ -597,7 +602,7 @@ def paged_attention_decode_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torc
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(positions), _ptr(q_req), _ptr(cu_q), n_tokens, n_head, n_kv_head, head_dim, page_size,
         num_pages, float(scale), int(window), 1 if identity else 0, _ptr(sinks), float(softcap),
-        *_gate_args(gate, q, n_tokens, n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
+        *_gate_args(gate, q, n_tokens, n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias, slopes), _stream())
     if rc == -2:
         return False
     _check(rc, "paged_attention_decode_bf16")
@@ -740,7 +745,7 @@ def prefill_attention_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Ten
                            single_below: int = 0, sinks: Optional[torch.Tensor] = None, softcap: float = 0.0,
                            gate: Optional[torch.Tensor] = None, keep_first: int = 0,
                            score_bias: Optional[torch.Tensor] = None, chunked: bool = False,
-                           dist_bias: Optional[torch.Tensor] = None) -> bool:
+                           dist_bias: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None) -> bool:
     """MFMA tile attention for steps with prompt portions (every request's tokens are consecutive
     rows of q from cu_q; a request may bring none).  Requests that bring exactly one token, and that
     among the step's first `single_below` tokens, are left to another kernel.  False when it does
@@ -768,7 +773,7 @@ def prefill_attention_bf16(q: torch.Tensor, out: torch.Tensor, k_pool: torch.Ten
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_pool), _ptr(v_pool), _ptr(block_tables),
         block_tables.shape[1], _ptr(cu_q), _ptr(seq_lens), n_req, max_q_len, n_head, n_kv_head, head_dim,
         page_size, float(scale), int(window), int(single_below), _ptr(sinks), float(softcap),
-        *_gate_args(gate, q, q.shape[0], n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias), _stream())
+        *_gate_args(gate, q, q.shape[0], n_head), *_mask_args(keep_first, score_bias, n_head, sinks, softcap, chunked, dist_bias, slopes), _stream())
     if rc == -2:
         return False
     _check(rc, "prefill_attention_bf16")
@@ -1141,12 +1146,15 @@ def rms_norm_store(src: torch.Tensor, gain: torch.Tensor, eps: float, pool: torc
 def latent_prepare(z: torch.Tensor, q_off: int, n_head: int, head_dim: int, rot_dim: int, positions: torch.Tensor,
                    freq: torch.Tensor, n_tokens: int, rot_magnitude: float = 1.0, c_off: int = 0, rank: int = 0,
                    gain: Optional[torch.Tensor] = None, eps: float = 0.0, pool: Optional[torch.Tensor] = None,
-                   slot_mapping: Optional[torch.Tensor] = None) -> None:
+                   slot_mapping: Optional[torch.Tensor] = None, interleaved: bool = False, cq_off: int = 0,
+                   cq_gain: Optional[torch.Tensor] = None, cq_out: Optional[torch.Tensor] = None) -> None:
     """Latent attention with a rotated part: the last rot_dim channels of every query head (heads of head_dim +
     rot_dim channels at q_off of z's rows) are rotated in place by the token's position; with `pool` (latent pages
     whose rows hold at least rank + rot_dim values) the token's row becomes [rms_norm(z[c_off : c_off + rank]) * gain |
-    the next rot_dim columns of z, rotated | zeros].  freq: float32 [rot_dim / 2]."""
-    _need_cuda(z, positions, freq, gain, pool, slot_mapping)
+    the next rot_dim columns of z, rotated | zeros].  freq: float32 [rot_dim / 2]; interleaved: the pairs are (2i, 2i + 1)
+    instead of (i, i + rot_dim / 2).  n_head may be 0 (the queries are not in z).  cq_out (rows of as many columns as
+    cq_gain has): rms_norm(z[cq_off ..]) * cq_gain, the latent that queries are made from."""
+    _need_cuda(z, positions, freq, gain, pool, slot_mapping, cq_gain, cq_out)
     _rows_2d("latent_prepare z", z, n_tokens)
     _need(freq.dtype == torch.float32 and freq.is_contiguous() and freq.numel() * 2 == rot_dim, "latent_prepare: float32 frequencies [rot_dim / 2]")
     _need_i32("positions", positions, n_tokens)
@@ -1160,9 +1168,17 @@ def latent_prepare(z: torch.Tensor, q_off: int, n_head: int, head_dim: int, rot_
         _need(z.shape[1] >= c_off + rank + rot_dim, "latent_prepare: z is too narrow for the latent")
         _need_i32("slot_mapping", slot_mapping, n_tokens)
         row_width = pool.shape[3]
+    cq_rank = 0
+    if cq_out is not None:
+        _need(cq_gain is not None and cq_gain.dtype == torch.float32 and cq_gain.is_contiguous(), "latent_prepare: cq_gain must be float32")
+        cq_rank = cq_gain.numel()
+        _rows_2d("latent_prepare cq_out", cq_out, n_tokens)
+        _need(cq_out.dtype == z.dtype and cq_out.shape[1] >= cq_rank and z.shape[1] >= cq_off + cq_rank,
+              "latent_prepare: the queries' latent needs columns of z and rows in its type")
     rc = library.kernels().mgpt_latent_prepare(
         _ptr(z), _dtype_code(z), z.stride(0), int(q_off), n_head, head_dim, rot_dim, int(c_off), int(rank), _ptr(gain),
         float(eps), _ptr(positions), _ptr(freq), float(rot_magnitude), _ptr(pool), row_width, _ptr(slot_mapping), n_tokens,
+        int(interleaved), int(cq_off), cq_rank, _ptr(cq_gain), _ptr(cq_out), cq_out.stride(0) if cq_out is not None else 0,
         _stream())
     _check(rc, "latent_prepare")
 
@@ -1278,19 +1294,21 @@ EXPERT_TILES = (16, 64, 256)
 MAX_EXPERTS = 1024
 
 
-GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2}
+GATE_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "clamped_swish": 3}
 
 
 def gated_unit(z: torch.Tensor, act: torch.Tensor, n_rows: int, hidden: int, fast: bool = False,
-               activation: str = "silu") -> None:
-    """act[n][j] = f(z[n][j]) * z[n][hidden + j] with f = silu, relu or the tanh form of gelu."""
+               activation: str = "silu", limit: float = 0.0, sharpness: float = 1.0) -> None:
+    """act[n][j] = f(z[n][j]) * z[n][hidden + j] with f = silu, relu or the tanh form of gelu; "clamped_swish":
+    g sigmoid(sharpness g) (u + 1) with g = min(z[n][j], limit) and u = z[n][hidden + j] held within -limit .. limit."""
     _need(activation in GATE_ACTIVATIONS, f"gated unit: activation {activation!r} is none of {sorted(GATE_ACTIVATIONS)}")
     _need_cuda(z, act)
     _need(z.dtype == act.dtype and z.dim() == 2 and act.dim() == 2 and z.stride(1) == 1 and act.stride(1) == 1
           and z.shape[1] >= 2 * hidden and act.shape[1] >= hidden and z.shape[0] >= n_rows and act.shape[0] >= n_rows,
           "z must be [>=n_rows, >=2 * hidden] and act [>=n_rows, >=hidden], one dtype")
     rc = library.kernels().mgpt_gated_unit(_ptr(z), z.stride(0), _ptr(act), act.stride(0), n_rows, hidden,
-                                           _dtype_code(z), int(fast), GATE_ACTIVATIONS[activation], _stream())
+                                           _dtype_code(z), int(fast), GATE_ACTIVATIONS[activation], float(limit),
+                                           float(sharpness), _stream())
     _check(rc, "gated_unit")
 
 
@@ -1411,20 +1429,20 @@ def gather_rows(src: torch.Tensor, slot_token: torch.Tensor, out: torch.Tensor, 
     return True
 
 
-ROUTER_SCORES = {"sigmoid": 0, "logit": 1}
+ROUTER_SCORES = {"sigmoid": 0, "logit": 1, "softmax": 2}
 
 
 def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen: torch.Tensor, weight: torch.Tensor,
                 q_req: Optional[torch.Tensor] = None, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
                 groups=None, normalise: bool = False, scale: float = 1.0, extra: Optional[torch.Tensor] = None,
-                extra_out: Optional[torch.Tensor] = None) -> None:
+                extra_out: Optional[torch.Tensor] = None, group_best: int = 2) -> None:
     """chosen[n] = the `top` experts with the largest w[e] . h[n] (float32 sums), best first; weight[n] = their
-    scores (sigmoid of the sum, or the sum itself).  w: dense [experts, width]; chosen int32 and weight float32,
+    scores (sigmoid of the sum, the sum itself, or the sums' softmax over all experts).  w: dense [experts, width]; chosen int32 and weight float32,
     dense [>= n_rows, top].
 
     correction (float32 [experts]) is added to the scores that the choice goes by; groups = (count, keep): only the
     experts of the `keep` groups (of `count` equal groups of neighbours) whose two largest choice scores have the
-    largest sums can be chosen; normalise: the weights are the chosen scores over (their sum + 1e-20); every weight
+    largest sums (group_best 1: whose largest choice scores are the largest) can be chosen; normalise: the weights are the chosen scores over (their sum + 1e-20); every weight
     is multiplied by `scale`.  extra ([width], like w): extra_out[n] = sigmoid(extra . h[n]), float32."""
     _need_cuda(h, w, chosen, weight, q_req, correction, extra, extra_out)
     _need(score in ROUTER_SCORES, f"router score {score!r} is none of {sorted(ROUTER_SCORES)}")
@@ -1440,6 +1458,7 @@ def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen:
     if q_req is not None:
         _need_i32("q_req", q_req, n_rows)
     count, keep = (1, 1) if groups is None else (int(groups[0]), int(groups[1]))
+    _need(group_best in (1, 2), "a group ranks by its best choice score, or by its two best")
     _need(0 < keep <= count and n_experts % count == 0 and top <= keep * (n_experts // count),
           f"groups {groups}: {n_experts} experts in equal groups of which enough stay for {top} choices")
     _need(correction is None or (correction.dtype == torch.float32 and correction.is_contiguous()
@@ -1451,7 +1470,7 @@ def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen:
     rc = library.kernels().mgpt_router_topk(_ptr(h), _dtype_code(h), h.stride(0), _ptr(w), _dtype_code(w), _ptr(q_req), n_rows,
                                             width, n_experts, top, ROUTER_SCORES[score], _ptr(chosen), _ptr(weight),
                                             _ptr(correction), count, keep, 1 if normalise else 0, float(scale), _ptr(extra),
-                                            _ptr(extra_out), _stream())
+                                            _ptr(extra_out), int(group_best), _stream())
     _check(rc, "router_topk")
 
 
@@ -1555,7 +1574,7 @@ def rms_post_norm(branches, x: torch.Tensor, gain_post: torch.Tensor, n_rows: in
     """branches: [(y float32 [rows, width], gain float32 [width] or None), ...].  With several branches
     y = mean_b unit(y_b) * gain_b (join_unit False: y = sum_b y_b * gain_b, a weighted sum), else y = y_0;
     x += mult * unit(y) * (offset + gain_post) (* scale_post, float32 [width]); with gain_next
-    h = unit(x) * (offset + gain_next); every y_b is cleared.  unit(v) = v / sqrt(mean(v^2) + eps)."""
+    h = unit(x) * (offset + gain_next), with h alone h = x; every y_b is cleared.  unit(v) = v / sqrt(mean(v^2) + eps)."""
     nb = len(branches)
     _need(1 <= nb <= MAX_NORM_BRANCHES, f"rms_post_norm takes 1 to {MAX_NORM_BRANCHES} branches")
     width = x.shape[1]
@@ -1574,15 +1593,26 @@ def rms_post_norm(branches, x: torch.Tensor, gain_post: torch.Tensor, n_rows: in
     for g in (gain_post, gain_next, scale_post):
         _need(g is None or (g.dtype == torch.float32 and g.numel() == width and g.is_contiguous()), "rms_post_norm: gains are float32 [width]")
     _need(gain_post is not None, "rms_post_norm needs the gain of the norm behind the sublayer")
-    if gain_next is not None:
-        _need(h is not None and h.is_contiguous() and h.shape[1] == width and h.shape[0] >= n_rows
+    _need(gain_next is None or h is not None, "rms_post_norm: the next norm needs rows to go to")
+    if h is not None:
+        _need(h.is_contiguous() and h.shape[1] == width and h.shape[0] >= n_rows
               and h.dtype in (torch.float32, torch.bfloat16), "rms_post_norm: h must be dense rows as wide as x")
     _need_cuda(x, gain_post, gain_next, h, scale_post)
     rc = library.kernels().mgpt_rms_post_norm(
         *ys, *gs, nb, 1.0 / nb if join_unit else 1.0, int(join_unit), _ptr(x), _ptr(gain_post), _ptr(scale_post),
         float(offset), float(eps), float(mult), _ptr(gain_next),
-        _ptr(h) if gain_next is not None else None, _dtype_code(h) if gain_next is not None else 0, n_rows, width, _stream())
+        _ptr(h), _dtype_code(h) if h is not None else 0, n_rows, width, _stream())
     _check(rc, "rms_post_norm")
+
+
+def cast_rows(x: torch.Tensor, out: torch.Tensor, n_rows: int, width: int) -> None:
+    """out[:n_rows, :width] = x[:n_rows, :width] (float32) in out's type."""
+    _need_cuda(x, out)
+    _rows_2d("cast_rows input", x, n_rows)
+    _rows_2d("cast_rows output", out, n_rows)
+    _need(x.dtype == torch.float32 and x.shape[1] >= width and out.shape[1] >= width, "cast_rows: float32 rows of at least `width` columns")
+    rc = library.kernels().mgpt_cast_rows(_ptr(x), x.stride(0), _ptr(out), _dtype_code(out), out.stride(0), n_rows, width, _stream())
+    _check(rc, "cast_rows")
 
 
 QK_NORMS = {None: 0, "head": 1, "whole": 2}
@@ -1595,7 +1625,8 @@ def qk_prepare(z: torch.Tensor, q_off: int, k_off: int, v_off: int, n_head: int,
                k_pool: Optional[torch.Tensor] = None, v_pool: Optional[torch.Tensor] = None,
                slot_mapping: Optional[torch.Tensor] = None, norm: Optional[str] = None,
                q_norm_weight: Optional[torch.Tensor] = None, k_norm_weight: Optional[torch.Tensor] = None,
-               values_from_keys: bool = False, rot_magnitude: float = 1.0) -> None:
+               values_from_keys: bool = False, rot_magnitude: float = 1.0, interleaved: bool = False,
+               query_temperature=None) -> None:
     """Projected queries, keys and values of a step's tokens (rows of z; q heads at q_off, k heads at k_off, v heads
     at v_off, head_stride channels apart) made ready for attention: q and k rotated by position with the float32
     frequencies `freq` [rot_dims / 2] (pairs (i, i + rot_dims / 2)), then divided by their root mean square over
@@ -1604,7 +1635,8 @@ def qk_prepare(z: torch.Tensor, q_off: int, k_off: int, v_off: int, n_head: int,
     norm "head" / "whole" (with norm_eps and float32 weights [head_dim] / [heads * head_dim] for q and for k): an RMS
     norm with weights *before* the rotation, head by head with the heads sharing a weight vector, or over all of a
     token's query (key) channels at once.  values_from_keys: the values are the keys as projected, z holds none.
-    rot_magnitude multiplies every cosine and sine."""
+    rot_magnitude multiplies every cosine and sine; interleaved: the pairs are (2i, 2i + 1).  query_temperature =
+    (coef, every): queries at position p are multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)."""
     _need_cuda(z, positions, freq, mix_lambda, v_other, k_pool, v_pool, slot_mapping, q_norm_weight, k_norm_weight)
     _need(norm in QK_NORMS, f"qk_prepare: norm {norm!r} is none of {sorted(QK_NORMS, key=str)}")
     if norm is not None:
@@ -1619,6 +1651,11 @@ def qk_prepare(z: torch.Tensor, q_off: int, k_off: int, v_off: int, n_head: int,
         _need(freq.dtype == torch.float32 and freq.is_contiguous() and positions is not None, "rotation needs float32 frequencies and positions")
         _need_i32("positions", positions, n_tokens)
         rot_dims = 2 * freq.numel()
+    temp_coef, temp_every = 0.0, 0
+    if query_temperature is not None:
+        temp_coef, temp_every = float(query_temperature[0]), int(query_temperature[1])
+        _need(temp_every > 0 and positions is not None, "qk_prepare: a query temperature needs a positive period and positions")
+        _need_i32("positions", positions, n_tokens)
     kv_span = (n_kv_head - 1) * head_stride
     _need(z.shape[1] >= max(q_off + (n_head - 1) * head_stride + head_dim, k_off + kv_span + head_dim,
                             v_off + kv_span + head_stride if k_pool is not None and not values_from_keys else 0),
@@ -1642,7 +1679,8 @@ def qk_prepare(z: torch.Tensor, q_off: int, k_off: int, v_off: int, n_head: int,
         _ptr(positions), _ptr(freq), rot_dims, -1.0 if norm_eps is None else float(norm_eps), _ptr(mix_lambda),
         _ptr(v_other), v_other.stride(0) if v_other is not None else 0, int(mix_mode), _ptr(k_pool), _ptr(v_pool),
         _ptr(slot_mapping), page_size, n_tokens, QK_NORMS[norm], _ptr(q_norm_weight) if norm else None,
-        _ptr(k_norm_weight) if norm else None, int(values_from_keys), float(rot_magnitude), _stream())
+        _ptr(k_norm_weight) if norm else None, int(values_from_keys), float(rot_magnitude), int(interleaved), temp_coef,
+        temp_every, _stream())
     _check(rc, "qk_prepare")
 
 
@@ -1888,13 +1926,13 @@ MAX_CONV_TAPS = 9
 CONV_ACTIVATIONS = {None: 0, "silu": 1}
 
 
-def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor,
+def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
                state_slots: torch.Tensor, cu_q: torch.Tensor, q_req: torch.Tensor, positions: torch.Tensor, n_req: int,
                out: torch.Tensor, o_off: int, n_tokens: int, activation: Optional[str] = None) -> None:
     """out[t][o_off + c] = act(sum_j weight[c][j] * u_(t - taps + 1 + j)[u_off + c] (+ bias[c])) over time inside each
     request, zeros before position 0; the taps - 1 inputs before the step's first token come from the request's
     slot of `state` (float32 rows holding [taps - 1][channels], a view of a pool's columns will do), which is then
-    brought up to date.  weight: float32 [channels, taps]."""
+    brought up to date (with one tap there is none: None).  weight: float32 [channels, taps]."""
     _need_cuda(u, weight, bias, state, state_slots, cu_q, q_req, positions, out)
     _need(activation in CONV_ACTIVATIONS, f"short_conv: activation {activation!r} is none of {sorted(map(str, CONV_ACTIVATIONS))}")
     _need(weight.dtype == torch.float32 and weight.dim() == 2 and weight.is_contiguous(), "short_conv: weight must be dense float32 [channels, taps]")
@@ -1906,7 +1944,7 @@ def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional
     _rows_2d("short_conv output", out, n_tokens)
     _need(u.shape[1] >= u_off + channels and out.shape[1] >= o_off + channels, "short_conv: rows are too narrow")
     _need(u.data_ptr() != out.data_ptr(), "short_conv: the output cannot be the input's buffer")
-    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+    _need(taps == 1 if state is None else state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
           and state.shape[1] >= (taps - 1) * channels, "short_conv: state must be float32 rows of (taps - 1) * channels")
     _need_i32("state_slots", state_slots, n_req)
     _need_i32("cu_q", cu_q, n_req + 1)
@@ -1914,6 +1952,51 @@ def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional
     _need_i32("positions", positions, n_tokens)
     rc = library.kernels().mgpt_short_conv(
         _ptr(u), _dtype_code(u), u.stride(0), u_off, _ptr(weight), _ptr(bias), CONV_ACTIVATIONS[activation], _ptr(state),
-        state.stride(0), _ptr(state_slots), _ptr(cu_q), _ptr(q_req), _ptr(positions), n_req, _ptr(out), _dtype_code(out),
+        state.stride(0) if state is not None else 0, _ptr(state_slots), _ptr(cu_q), _ptr(q_req), _ptr(positions), n_req, _ptr(out), _dtype_code(out),
         out.stride(0), o_off, n_tokens, channels, taps, _stream())
     _check(rc, "short_conv", 2 if taps > 1 else 1)
+
+
+DIAGONAL_CHUNK = 32     # tokens a chunk of diagonal_state
+
+
+def diagonal_scratch_floats(n_tokens: int, n_req: int, channels: int) -> int:
+    """float32 values of scratch that diagonal_state uses for a step in which a request may bring several tokens."""
+    return 3 * (n_tokens // DIAGONAL_CHUNK + n_req) * channels
+
+
+def diagonal_state(u: torch.Tensor, gates: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, decay: torch.Tensor,
+                   block: int, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor,
+                   n_req: int, n_tokens: int, out: torch.Tensor, y: Optional[torch.Tensor] = None,
+                   scratch: Optional[torch.Tensor] = None) -> None:
+    """Over time inside each request, channel by channel: log a = decay * sigmoid(gr + r_bias),
+    S_t = a S_(t-1) + sqrt(1 - a^2) sigmoid(gi + i_bias) u_t, out_t = S_t * gelu_tanh(y_t) (without y: S_t).  The logits of
+    block b (`block` channels) are the columns 2 b block .. of `gates`, first gr, then gi.  S is zero before position 0 and
+    lives in the requests' slots of `state` (float32 rows, a view of a pool's columns will do).  r_bias, i_bias, decay
+    (<= 0): float32 [channels].  scratch (float32, diagonal_scratch_floats): the tokens of a request in chunks side by
+    side; None: one after the other (steps of single tokens)."""
+    _need_cuda(u, gates, r_bias, i_bias, decay, state, state_slots, cu_q, positions, out, y, scratch)
+    channels = decay.numel()
+    for name, t in (("r_bias", r_bias), ("i_bias", i_bias), ("decay", decay)):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == channels, f"diagonal_state: {name} must be float32 [channels]")
+    _need(block > 0 and channels % block == 0, "diagonal_state: the channels come in equal blocks")
+    for name, t, cols in (("u", u, channels), ("gates", gates, 2 * channels), ("out", out, channels), ("y", y, channels)):
+        if t is not None:
+            _rows_2d(f"diagonal_state {name}", t, n_tokens)
+            _need(t.shape[1] >= cols, f"diagonal_state: {name}'s rows are too narrow")
+    _need(out.dtype == u.dtype and (y is None or y.dtype == u.dtype) and gates.dtype in (u.dtype, torch.float32),
+          "diagonal_state: u, y and out share a type, the gates have it or float32")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] >= channels,
+          "diagonal_state: state must be float32 rows of the channels")
+    _need_i32("state_slots", state_slots, n_req)
+    _need_i32("cu_q", cu_q, n_req + 1)
+    _need_i32("positions", positions, n_tokens)
+    if scratch is not None:
+        _need(scratch.dtype == torch.float32 and scratch.is_contiguous()
+              and scratch.numel() >= diagonal_scratch_floats(n_tokens, n_req, channels), "diagonal_state: too little scratch")
+    rc = library.kernels().mgpt_diagonal_state(
+        _ptr(u), _dtype_code(u), u.stride(0), _ptr(gates), _dtype_code(gates), gates.stride(0), _ptr(r_bias), _ptr(i_bias),
+        _ptr(decay), block, _ptr(y), _dtype_code(y) if y is not None else 0, y.stride(0) if y is not None else 0, 0, _ptr(state),
+        state.stride(0), _ptr(state_slots), _ptr(cu_q), _ptr(positions), n_req, n_tokens, channels, _ptr(scratch),
+        scratch.numel() if scratch is not None else 0, _ptr(out), _dtype_code(out), out.stride(0), _stream())
+    _check(rc, "diagonal_state", 2 if scratch is not None else 1)

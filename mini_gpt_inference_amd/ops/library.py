@@ -39,7 +39,7 @@ def kernels() -> ctypes.CDLL:
         lib.mgpt_layernorm.argtypes = [P, P, P, P, P, I, I, F, I, P]
         lib.mgpt_linear_generic.argtypes = [P, I, L, P, I, P, P, I, L, I, I, I, I, P]
         lib.mgpt_kv_write.argtypes = [P, I, L, I, I, P, P, P, I, I, I, I, P]
-        lib.mgpt_paged_attention_generic.argtypes = [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, P, F, P, L, I, P, I, P, I, P]
+        lib.mgpt_paged_attention_generic.argtypes = [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, I, I, P, F, P, L, I, P, I, P, I, P, P]
         lib.mgpt_sample.argtypes = [P, L, I, I, I, P, P, P, P, P, c_ulonglong, P, P, P, I, P]
         lib.mgpt_sample_advance.argtypes = [P, L, I, I, I, P, P, P, P, P, c_ulonglong, P,
                                             P, P, P, P, P, P, P, I, I, I, I, P, P, I, I, P, P, I, P]
@@ -127,16 +127,16 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_linear_skinny_partials": [I, I, I, I, I],
         "mgpt_linear_skinny_row_groups": [I, I, I],
         "mgpt_fold_layernorm": [P, P, P, P, P, P, P, I, I, P],
-        "mgpt_paged_attention_split_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P],
-        "mgpt_paged_attention_split_fast_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P],
-        "mgpt_paged_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P],
+        "mgpt_paged_attention_split_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P, P],
+        "mgpt_paged_attention_split_fast_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, F, I, P, F, P, L, I, P, I, P, I, P, P],
+        "mgpt_paged_attention_decode_bf16": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P, P],
         "mgpt_linear_mfma": [P, L, P, P, P, I, L, I, I, I, I, P, L, P],
         "mgpt_linear_mfma_xielu": [P, L, P, P, P, L, I, I, I, P, P, L, P],
         "mgpt_linear_mfma_shape": [I, I, P, L, P, P, P, I, L, I, I, I, I, P, L, P],
         "mgpt_linear_mfma_partials": [I, I, I, I],
         "mgpt_linear_mfma_parts": [P, L, P, P, P, L, I, I, I, P],
         "mgpt_linear_mfma_qkv": [P, L, P, P, P, L, I, I, I, P, P, P, I, I, I, I, I, I, P],
-        "mgpt_prefill_attention_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P],
+        "mgpt_prefill_attention_bf16": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, I, I, P, F, P, L, I, P, I, P, I, P, P],
         # a residual that is still a sum: base, partials, n_parts, part_stride, token table, position table, ids, positions
         "mgpt_fused_attention_decode": [P, P, I, L, P, P, P, P, P, P, P, P, F, P, P, P, P, P, L, P, P, P, P, I, P, P,
                                         I, I, I, I, I, I, F, P],
@@ -157,7 +157,7 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         # latent attention
         "mgpt_rms_norm_store": [P, I, L, P, F, P, P, I, I, P],
         "mgpt_heads_linear": [P, L, P, P, L, P, L, I, I, I, I, I, I, P],
-        "mgpt_latent_prepare": [P, I, L, I, I, I, I, I, I, P, F, P, P, F, P, I, P, I, P],
+        "mgpt_latent_prepare": [P, I, L, I, I, I, I, I, I, P, F, P, P, F, P, I, P, I, I, I, I, P, P, L, P],
         # a layer whose sublayers read one norm, the mixer through a token shift; the xIELU activation
         "mgpt_parallel_norm": [P, P, F, P, F, F, P, P, I, P, P, L, P, P, P, I, I, P],
         "mgpt_token_shift": [P, P, I, P, P, L, P, P, P, P, I, I, P],
@@ -165,11 +165,12 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_xielu": [P, L, P, L, I, P, I, I, I, P],
         "mgpt_heads_linear_mfma": [P, L, P, P, L, P, L, I, I, I, I, P],
         # gated feed-forwards and experts
-        "mgpt_gated_unit": [P, L, P, L, I, I, I, I, I, P],
+        "mgpt_gated_unit": [P, L, P, L, I, I, I, I, I, F, F, P],
         # root-mean-square norms, rotation and the rest in front of attention, decaying state
         "mgpt_rms_norm": [P, I, L, P, P, F, F, F, P, I, L, I, P, I, L, I, P, L, I, I, I, I, I, I, P],
         "mgpt_rms_post_norm": [P, P, P, P, P, P, P, P, I, F, I, P, P, P, F, F, F, P, P, I, I, I, P],
-        "mgpt_qk_prepare": [P, I, L, I, I, I, I, I, I, I, I, P, P, I, F, P, P, L, I, P, P, P, I, I, I, P, P, I, F, P],
+        "mgpt_cast_rows": [P, L, P, I, L, I, I, P],
+        "mgpt_qk_prepare": [P, I, L, I, I, I, I, I, I, I, I, P, P, I, F, P, P, L, I, P, P, P, I, I, I, P, P, I, F, I, F, I, P],
         "mgpt_decay_state": [P, I, L, I, I, I, I, I, I, I, I, P, P, I, F, P, P, P, P, I, F, P, I, L, P],
         "mgpt_decay_state_chunked": [P, I, L, I, I, I, I, I, I, I, P, P, I, F, P, P, P, P, I, I, P, P, L, P],
         "mgpt_expert_route": [P, P, P, I, I, I, P, P, P, P, I, I, I, P],
@@ -178,11 +179,13 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_grouped_linear": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, I, P],
         "mgpt_grouped_linear_mfma": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, P],
         "mgpt_expert_combine": [P, P, P, P, I, I, I, F, P, P, P, P],
-        "mgpt_router_topk": [P, I, L, P, I, P, I, I, I, I, I, P, P, P, I, I, I, F, P, P, P],
+        "mgpt_router_topk": [P, I, L, P, I, P, I, I, I, I, I, P, P, P, I, I, I, F, P, P, I, P],
         "mgpt_gather_scale_rows": [P, I, L, P, P, P, P, L, I, I, P],
         # a state with a decay made from the token, short convolutions
         "mgpt_gated_state": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, P, P, L, P],
         "mgpt_gated_state_chunked": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, I, P, P, P, L, P],
+        # a diagonal state with its gates from block products
+        "mgpt_diagonal_state": [P, I, L, P, I, L, P, P, P, I, P, I, L, I, P, L, P, P, P, I, I, I, P, L, P, I, L, P],
         # the gated delta rule
         "mgpt_delta_state": [P, I, L, I, I, I, P, L, I, I, I, I, I, I, I, F, P, P, P, F, P, L, P, P, I, P, P, L, P],
         "mgpt_delta_image_floats": [I, I, I, I],

@@ -157,7 +157,8 @@ class SandwichNorm(Arrangement):
     (1 / B) * sum_b join_b(mixer_b(h)); with `join_weights` = (c_0, .., c_(B-1)) it is the weighted sum
     sum_b c_b mixer_b(h) instead, and there are no join norms.  With `layer_scale` each sublayer's normed
     output is multiplied channel by channel by a vector of the layer's own (`scale1`, `scale2`) before
-    it is added.  All norms are RMS norms (kind "rms_norm"); the norms around the sublayers share one
+    it is added.  Without `input_norm` there are no norm1 and norm2: the sublayers read x itself (rounded to
+    the compute dtype), and only their outputs are normed.  All norms are RMS norms (kind "rms_norm"); the norms around the sublayers share one
     eps and one way of storing the gain, the joins have plain gains.
 
     The sublayers are the framework's ordinary parts: they add their output into a cleared float32
@@ -168,7 +169,7 @@ class SandwichNorm(Arrangement):
     plan_safe = True
 
     def __init__(self, width: int, residual_mult: float = 1.0, feed_forward: bool = True, branches: int = 1,
-                 join_weights=None, layer_scale: bool = False) -> None:
+                 join_weights=None, layer_scale: bool = False, input_norm: bool = True) -> None:
         self.width, self.mult = int(width), float(residual_mult)
         self.has_feed_forward, self.branches = bool(feed_forward), int(branches)
         if not 1 <= self.branches <= kernels.MAX_NORM_BRANCHES:
@@ -182,9 +183,10 @@ class SandwichNorm(Arrangement):
         else:
             self.mixer_roles = tuple(f"mixer{b}" for b in range(self.branches))
             self.join_roles = () if self.join_weights is not None else tuple(f"join{b}" for b in range(self.branches))
-        self.roles = ("norm1",) + self.mixer_roles + self.join_roles + ("norm1b",)
+        self.has_input_norm = bool(input_norm)
+        self.roles = (("norm1",) if self.has_input_norm else ()) + self.mixer_roles + self.join_roles + ("norm1b",)
         if self.has_feed_forward:
-            self.roles += ("norm2", "feed_forward", "norm2b")
+            self.roles += (("norm2",) if self.has_input_norm else ()) + ("feed_forward", "norm2b")
         self._checked = False
         self.scale1 = self.scale2 = None
         self._join_gains = None
@@ -247,16 +249,19 @@ class SandwichNorm(Arrangement):
         if not self._checked:
             self._check(parts)
         n, B = ctx.n_rows, self.branches
-        norm1 = parts["norm1"]
+        norm1, norm2 = parts.get("norm1"), parts.get("norm2")
         ys = self._buffers(ctx)
         h = ctx.workspace.get("normed", n, self.width, ctx.dtype)
         left, ctx.pending_update = ctx.pending_update, None
         if left is not None and left.goes_with(norm1, x, n):
-            left.run(norm1.weight, h)       # the layer before's last addition and this layer's first norm in one kernel
+            left.run(None if norm1 is None else norm1.weight, h)       # the layer before's last addition and this layer's first norm in one kernel
         else:
             if left is not None:
                 left.run(None, None)
-            norm1.forward(ctx, x, h, n)
+            if norm1 is not None:
+                norm1.forward(ctx, x, h, n)
+            else:
+                kernels.cast_rows(x, h, n, self.width)
         for b, role in enumerate(self.mixer_roles):
             parts[role].forward_add(ctx, h, ys[b], bindings[role], position)
         joins = self._joins(ys, parts)
@@ -266,7 +271,7 @@ class SandwichNorm(Arrangement):
             return
         norm1b = parts["norm1b"]
         kernels.rms_post_norm(joins, x, norm1b.weight, n, norm1b.eps, norm1b.offset, self.mult,
-                              gain_next=parts["norm2"].weight, h=h, join_unit=join_unit, scale_post=self.scale1)
+                              gain_next=None if norm2 is None else norm2.weight, h=h, join_unit=join_unit, scale_post=self.scale1)
         parts["feed_forward"].forward_add(ctx, h, ys[0])
         ctx.pending_update = PendingSandwich([(ys[0], None)], x, parts["norm2b"], self.mult, n, True, self.scale2)
 
@@ -357,16 +362,17 @@ class PendingParallel:
 class PendingSandwich:
     """A sublayer's output that is still to be normed and added to the residual: x += mult * norm(y).  Whoever
     reads x next makes the addition: a layer of the same kind together with its first norm (run(gain, h) also
-    leaves h = norm_next(x)), anyone else through flush_update."""
+    leaves h = norm_next(x), or h = x without a norm), anyone else through flush_update."""
 
     def __init__(self, joins, x: torch.Tensor, norm: Part, mult: float, n_rows: int, join_unit: bool = True,
                  scale: Optional[torch.Tensor] = None) -> None:
         self.joins, self.x, self.norm, self.mult, self.n_rows = joins, x, norm, mult, n_rows
         self.join_unit, self.scale = join_unit, scale      # how several branches meet; the layer's scale per channel
 
-    def goes_with(self, norm_next: Part, x: torch.Tensor, n_rows: int) -> bool:
-        return (x is self.x and n_rows == self.n_rows and norm_next.eps == self.norm.eps
-                and norm_next.offset == self.norm.offset)
+    def goes_with(self, norm_next: Optional[Part], x: torch.Tensor, n_rows: int) -> bool:
+        """Whether the addition and the next layer's first norm (None: it reads x as it is) can be one kernel."""
+        return x is self.x and n_rows == self.n_rows and (
+            norm_next is None or (norm_next.eps == self.norm.eps and norm_next.offset == self.norm.offset))
 
     def run(self, gain_next: Optional[torch.Tensor], h: Optional[torch.Tensor]) -> None:
         kernels.rms_post_norm(self.joins, self.x, self.norm.weight, self.n_rows, self.norm.eps, self.norm.offset,

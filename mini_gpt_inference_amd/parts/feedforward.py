@@ -2,7 +2,7 @@
 
 from __future__ import annotations
 
-from typing import Dict
+from typing import Dict, Optional
 
 import torch
 
@@ -104,13 +104,25 @@ class DenseMLP(FeedForward):
 
 
 def _gated(ctx: StepContext, h, in_weight: torch.Tensor, down_weight: torch.Tensor, x: torch.Tensor, n: int,
-           hidden: int, activation: str = "silu") -> None:
-    """x += (act(h Wgate^T) * (h Wup^T)) Wdown^T with the gate and up matrices stacked in in_weight."""
+           hidden: int, **unit) -> None:
+    """x += (act(h Wgate^T) * (h Wup^T)) Wdown^T with the gate and up matrices stacked in in_weight; `unit`: the
+    activation and its constants, as ops.kernels.gated_unit takes them."""
     z = ctx.workspace.get("gated_z", n, 2 * hidden, ctx.dtype)
     linear(ctx, h, in_weight, None, z, n)
     act = ctx.workspace.get("gated_act", n, hidden, ctx.dtype)
-    kernels.gated_unit(z, act, n, hidden, fast=not ctx.exact, activation=activation)
+    kernels.gated_unit(z, act, n, hidden, fast=not ctx.exact, **unit)
     linear_add(ctx, act, down_weight, None, x, n)
+
+
+def _unit_options(activation: str, limit: Optional[float], sharpness: float) -> Dict[str, object]:
+    """The gated unit's activation and constants as ops.kernels.gated_unit takes them."""
+    if activation not in kernels.GATE_ACTIVATIONS:
+        raise ValueError(f"gated unit: activation {activation!r} is none of {sorted(kernels.GATE_ACTIVATIONS)}")
+    if activation != "clamped_swish":
+        return {"activation": activation}
+    if limit is None or not float(limit) > 0.0:
+        raise ValueError(f"gated unit: a clamped swish needs a positive limit, got {limit!r}")
+    return {"activation": activation, "limit": float(limit), "sharpness": float(sharpness)}
 
 
 def _stack_gate_up(part: Part, tensors, gate: str, up: str):
@@ -126,15 +138,17 @@ def _stack_gate_up(part: Part, tensors, gate: str, up: str):
 @register_feed_forward("gated_mlp")
 class GatedMLP(FeedForward):
     """m = (act(h Wgate^T) * (h Wup^T)) Wdown^T, no biases; act is silu(v) = v sigmoid(v) unless
-    `activation` names relu or gelu_tanh; the unit's nonlinearity and product in float32."""
+    `activation` names relu or gelu_tanh; the unit's nonlinearity and product in float32.  "clamped_swish" (with
+    `limit` and `sharpness`) is the unit g sigmoid(sharpness g) (u + 1), g = min(h Wgate^T, limit), u = h Wup^T held within
+    -limit .. limit."""
 
     graph_safe = True
     plan_safe = True
 
-    def __init__(self, width: int, hidden: int, activation: str = "silu") -> None:
+    def __init__(self, width: int, hidden: int, activation: str = "silu", limit: Optional[float] = None,
+                 sharpness: float = 1.0) -> None:
         self.width, self.hidden = int(width), int(hidden)
-        if activation not in kernels.GATE_ACTIVATIONS:
-            raise ValueError(f"gated unit: activation {activation!r} is none of {sorted(kernels.GATE_ACTIVATIONS)}")
+        self.unit = _unit_options(activation, limit, sharpness)
         self.activation = activation
         self.in_weight = None
 
@@ -150,7 +164,7 @@ class GatedMLP(FeedForward):
 
     def forward_add(self, ctx: StepContext, h, x: torch.Tensor) -> None:
         plain_residual(ctx, h, x)
-        _gated(ctx, h, self.in_weight, self.down_weight, x, ctx.n_rows, self.hidden, self.activation)
+        _gated(ctx, h, self.in_weight, self.down_weight, x, ctx.n_rows, self.hidden, **self.unit)
 
 
 @register_feed_forward("table_experts")
@@ -174,6 +188,7 @@ class TableExperts(FeedForward):
             raise ValueError(f"top {self.top} of {self.n_experts} experts: need 0 < top <= experts <= {kernels.MAX_EXPERTS}")
         # an expert is a gated unit; without the gate (a subclass says so) it is down(act(up h)) with this activation
         self.gated, self.epilogue = True, kernels.EPI_NONE
+        self.unit = self.shared_unit = {"activation": "silu"}     # the gated unit of the experts, and of the shared one
         self.gates_shared = False       # the shared expert's output is multiplied by a number per token
         self.in_weights = self.down_weights = self.shared_in_weight = None
 
@@ -262,7 +277,7 @@ class TableExperts(FeedForward):
             kernels.grouped_linear(rows, None, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast,
                                    self.epilogue)
         if self.gated:
-            kernels.gated_unit(z, act, slots, self.hidden, fast=not ctx.exact)
+            kernels.gated_unit(z, act, slots, self.hidden, fast=not ctx.exact, **self.unit)
         pair_out = ws.get("expert_pair_out", n * self.top, self.width, torch.float32)
         kernels.grouped_linear(act, None, self.down_weights, tile_expert, slot_token, pair_out, slot_pair, slots,
                                tile, fast)
@@ -276,13 +291,13 @@ class TableExperts(FeedForward):
         if not self.shared_hidden:
             return None
         if self.gated and not self.gates_shared:
-            _gated(ctx, hn, self.shared_in_weight, self.shared_down, x, n, self.shared_hidden)
+            _gated(ctx, hn, self.shared_in_weight, self.shared_down, x, n, self.shared_hidden, **self.shared_unit)
             return None
         act = ctx.workspace.get("shared_act", n, self.shared_hidden, ctx.dtype)
         if self.gated:
             z = ctx.workspace.get("shared_z", n, 2 * self.shared_hidden, ctx.dtype)
             linear(ctx, hn, self.shared_in_weight, None, z, n)
-            kernels.gated_unit(z, act, n, self.shared_hidden, fast=not ctx.exact)
+            kernels.gated_unit(z, act, n, self.shared_hidden, fast=not ctx.exact, **self.shared_unit)
         else:
             linear(ctx, hn, self.shared_in_weight, None, act, n, self.epilogue)
         if not self.gates_shared:
@@ -321,7 +336,7 @@ class TableExperts(FeedForward):
         if not kernels.grouped_linear_tiled(sorted_rows, self.in_weights, tile_expert, slot_token, z, slots, self.epilogue):
             return False
         if self.gated:
-            kernels.gated_unit(z, act, slots, self.hidden, fast=True)
+            kernels.gated_unit(z, act, slots, self.hidden, fast=True, **self.unit)
         slot_out = ws.get("expert_slot_out", slots, self.width, torch.float32)
         if not kernels.grouped_linear_tiled(act, self.down_weights, tile_expert, slot_token, slot_out, slots):
             return False
@@ -338,7 +353,9 @@ class RoutedExperts(TableExperts):
     expert_e(s_e h), expert(u) = (silu(u Wgate^T) * (u Wup^T)) Wdown^T: the score multiplies the expert's
     input and is not renormalised.  A shared expert (shared_hidden > 0) takes every token unweighted.
 
-    Options: `activation` "relu2": experts without a gate, expert(u) = max(u Wup^T, 0)^2 Wdown^T; `weight_on`
+    Options: `score` "softmax" (over all experts) or "logit"; `activation` "relu2": experts without a gate, expert(u) =
+    max(u Wup^T, 0)^2 Wdown^T, or another gated unit (GatedMLP's) with its constants `limit` and `sharpness` (and
+    `shared_limit` where the shared expert's differs); `group_best` 1: a group ranks by its best expert alone; `weight_on`
     "output": the weight multiplies the expert's output; `correction`: a number per expert is added to the scores
     that the choice goes by (the weights are the scores without it); `groups` = (count, keep): the experts form
     `count` equal groups of neighbours and only those of the `keep` groups whose two largest choice scores have the
@@ -354,15 +371,21 @@ class RoutedExperts(TableExperts):
 
     def __init__(self, width: int, hidden: int, n_experts: int, top: int, shared_hidden: int = 0,
                  score: str = "sigmoid", activation: str = "silu", weight_on: str = "input", correction: bool = False,
-                 groups=None, normalise: bool = False, scale: float = 1.0, shared_gate: bool = False) -> None:
+                 groups=None, normalise: bool = False, scale: float = 1.0, shared_gate: bool = False,
+                 limit: Optional[float] = None, shared_limit: Optional[float] = None, sharpness: float = 1.0,
+                 group_best: int = 2) -> None:
         super().__init__(width, hidden, n_experts, top, vocab_size=0, shared_hidden=shared_hidden)
         if score not in kernels.ROUTER_SCORES:
             raise ValueError(f"router score {score!r} is none of {sorted(kernels.ROUTER_SCORES)}")
         self.score = score
-        if activation != "silu" and activation not in _EXPERT_ACTIVATIONS:
-            raise ValueError(f"experts' activation {activation!r} is neither 'silu' (gated) nor one of {sorted(_EXPERT_ACTIVATIONS)}")
-        self.gated = activation == "silu"
+        self.gated = activation not in _EXPERT_ACTIVATIONS
         self.epilogue = kernels.EPI_NONE if self.gated else _EXPERT_ACTIVATIONS[activation]
+        if self.gated:
+            self.unit = _unit_options(activation, limit, sharpness)
+            self.shared_unit = _unit_options(activation, limit if shared_limit is None else shared_limit, sharpness)
+        if group_best not in (1, 2):
+            raise ValueError("a group of experts ranks by its best one (group_best 1) or its two best (2)")
+        self.group_best = int(group_best)
         if weight_on not in ("input", "output"):
             raise ValueError(f"weight_on {weight_on!r} is neither 'input' nor 'output'")
         self.weighs_output, self.has_correction = weight_on == "output", bool(correction)
@@ -404,7 +427,7 @@ class RoutedExperts(TableExperts):
         gate = ws.get("router_shared_gate", n, 1, torch.float32).view(-1) if self.gates_shared else None
         kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, q_req=ctx.q_req, score=self.score,
                             correction=self.correction, groups=self.groups, normalise=self.normalise, scale=self.scale,
-                            extra=self.shared_gate_weight, extra_out=gate)
+                            extra=self.shared_gate_weight, extra_out=gate, group_best=self.group_best)
         weight = weight.view(-1)
         self._experts_add(ctx, hn, x, n, None, chosen, None if self.weighs_output else weight, 1.0,
                           out_weight=weight if self.weighs_output else None, shared_gate=gate)

@@ -149,7 +149,9 @@ class LatentAttention(Mixer):
     p - window < j <= p (window 0: all j <= p); softmax in float32 with one more term exp(sink_a) in
     the denominator that has no value; y = concat_a(P v_a) * sigmoid(h Wg^T); out = y Wo^T, added
     into the residual.  The gate is a number per channel of y (`gate` "channel", Wg [H * E, W]) or a
-    number per head ("head", Wg [H, W]).
+    number per head ("head", Wg [H, W]), or there is none (None).  `sinks` False: the denominator has no such term.
+    With `q_rank` = Q > 0 the queries come from a latent of their own: q_a = Wuq_a cq with
+    cq = rms_norm(h Wdq^T) * gain, [Q], which is not cached.
 
     With `rot_dim` = P > 0 a position signal rides beside the latent: a query head is [D plain | P rotated]
     channels (Wq has H (D + P) rows), Wdkv has rank + P rows of which the last P, not normed, are one key part
@@ -168,11 +170,13 @@ class LatentAttention(Mixer):
     # up to this many rows queries, gate and latent come from one product with the matrices stacked
     # (one launch less in a decode step); beyond it from two
     JOINT_PRODUCT_MAX_ROWS = 128
+    CACHED_ROWS = (32, 64, 128)     # rows with a rotated part are padded to these where they are no longer: what the bfloat16 kernels take
     JOINT_PRODUCT_MAX_WORK = 4 << 20     # rows x (query + gate columns); a smaller product has no full round to lose
 
     def __init__(self, width: int, n_head: int, head_dim: int, value_dim: int, rank: int, scale: float,
                  window: int = 0, eps: float = 1e-6, makes_latent: bool = True, rot_dim: int = 0,
-                 rotary: Optional[dict] = None, gate: str = "channel") -> None:
+                 rotary: Optional[dict] = None, gate: Optional[str] = "channel", sinks: bool = True,
+                 q_rank: int = 0) -> None:
         self.width, self.n_head, self.head_dim = int(width), int(n_head), int(head_dim)
         self.value_dim, self.rank = int(value_dim), int(rank)
         self.scale, self.window, self.eps = float(scale), int(window), float(eps)
@@ -181,27 +185,37 @@ class LatentAttention(Mixer):
         self.rotation = _own_rotation(rotary) if self.rot_dim else None
         if self.rot_dim and (self.rotation is None or self.rotation.dims != self.rot_dim):
             raise ValueError("a latent with a rotated part needs a rotation over exactly rot_dim channels")
-        if gate not in ("channel", "head"):
-            raise ValueError(f"gate {gate!r} is neither 'channel' nor 'head'")
-        self.head_gate = gate == "head"
+        if gate not in ("channel", "head", None):
+            raise ValueError(f"gate {gate!r} is none of 'channel', 'head' and None")
+        self.has_gate, self.head_gate, self.has_sinks = gate is not None, gate == "head", bool(sinks)
+        self.q_rank = int(q_rank or 0)
+        if self.q_rank < 0 or (self.q_rank and not self.rot_dim):
+            raise ValueError("queries from a latent of their own go with a rotated part")
         # what a cached row holds: the latent alone, or the latent and the rotated key part (rows then
-        # start 16 bytes apart in bfloat16 too)
+        # start 16 bytes apart in bfloat16 too, and have a size that the matrix-core kernels take if one is near)
         self.row = self.rank if not self.rot_dim else -(-(self.rank + self.rot_dim) // 8) * 8
+        if self.rot_dim:
+            self.row = next((r for r in self.CACHED_ROWS if self.row <= r), self.row)
         if not 0 < self.row <= 1024:
             raise ValueError(f"latent size {self.row}: the attention kernels take up to 1024")
         self.q_head = self.head_dim + self.rot_dim
         self.q_width = self.n_head * self.q_head
         self.y_width = self.n_head * self.value_dim
-        self.g_width = self.n_head if self.head_gate else self.y_width
+        self.g_width = 0 if not self.has_gate else (self.n_head if self.head_gate else self.y_width)
         self.in_weight = self.uk_folded = self.uv_heads = None
 
     def weight_requests(self) -> Dict[str, WeightRequest]:
-        req = {"q_weight": WeightRequest((self.q_width, self.width), MATRIX),
-               "gate_weight": WeightRequest((self.g_width, self.width), MATRIX),
+        req = {"q_weight": WeightRequest((self.q_width, self.q_rank or self.width), MATRIX),
                "uk_weight": WeightRequest((self.n_head * self.head_dim, self.rank), MATRIX),
                "uv_weight": WeightRequest((self.y_width, self.rank), MATRIX),
-               "sink": WeightRequest((self.n_head,), VECTOR),
                "out_weight": WeightRequest((self.width, self.y_width), MATRIX)}
+        if self.q_rank:
+            req["dq_weight"] = WeightRequest((self.q_rank, self.width), MATRIX)
+            req["dq_norm"] = WeightRequest((self.q_rank,), VECTOR)
+        if self.has_gate:
+            req["gate_weight"] = WeightRequest((self.g_width, self.width), MATRIX)
+        if self.has_sinks:
+            req["sink"] = WeightRequest((self.n_head,), VECTOR)
         if self.makes_latent:
             req["dkv_weight"] = WeightRequest((self.rank + self.rot_dim, self.width), MATRIX)
             req["dkv_norm"] = WeightRequest((self.rank,), VECTOR)
@@ -210,12 +224,14 @@ class LatentAttention(Mixer):
     def token_matrix_elements(self) -> int:
         if self.in_weight is None:
             return 0
-        return self.in_weight.numel() + self.uk_folded.numel() + self.uv_heads.numel() + self.out_weight.numel()
+        own = self.q_weight.numel() if self.q_rank else 0
+        return own + self.in_weight.numel() + self.uk_folded.numel() + self.uv_heads.numel() + self.out_weight.numel()
 
     def bind(self, tensors):
         super().bind(tensors)
-        # the products that read h as one: queries, gate and (where this layer makes it) the latent
-        names = ["q_weight", "gate_weight"] + (["dkv_weight"] if self.makes_latent else [])
+        # the products that read h as one: queries (or their latent), gate and (where this layer makes it) the latent
+        names = (["dq_weight" if self.q_rank else "q_weight"] + (["gate_weight"] if self.has_gate else [])
+                 + (["dkv_weight"] if self.makes_latent else []))
         stacked = [tensors[n] for n in names]
         rows = sum(t.shape[0] for t in stacked)
         if self.rot_dim and rows % 16:      # rows of the products' output start 16 bytes apart
@@ -260,7 +276,8 @@ class LatentAttention(Mixer):
         n, ws = ctx.n_rows, ctx.workspace
         fast = not ctx.exact
         z = ws.get("latent_in", n, self.in_weight.shape[0], ctx.dtype)
-        split = self.q_width + self.g_width
+        q_cols = self.q_rank or self.q_width
+        split = q_cols + self.g_width
         if (self.makes_latent and not self.rot_dim and n > self.JOINT_PRODUCT_MAX_ROWS
                 and n * split > self.JOINT_PRODUCT_MAX_WORK):
             # many rows: the few latent columns on top of queries and gate would start another
@@ -273,21 +290,29 @@ class LatentAttention(Mixer):
             linear(ctx, h, self.in_weight, None, z, n)
         group = ctx.groups[binding.group]
         pool = group.k_pools[binding.index]
+        q = z
         if self.rot_dim:
             # the queries' rotated parts in place; the normed latent and the rotated key part into the pages
-            kernels.latent_prepare(z, 0, self.n_head, self.head_dim, self.rot_dim, ctx.positions,
-                                   self.rotation.frequencies(z.device), n, getattr(self.rotation, "magnitude", 1.0),
+            rot = (self.rot_dim, ctx.positions, self.rotation.frequencies(z.device), n, getattr(self.rotation, "magnitude", 1.0))
+            pairs = getattr(self.rotation, "interleaved", False)
+            cq = ws.get("latent_cq", n, self.q_rank, ctx.dtype) if self.q_rank else None
+            kernels.latent_prepare(z, 0, 0 if self.q_rank else self.n_head, self.head_dim, *rot,
                                    c_off=split, rank=self.rank, gain=self.dkv_norm if self.makes_latent else None,
                                    eps=self.eps, pool=pool if self.makes_latent else None,
-                                   slot_mapping=group.slot_mapping if self.makes_latent else None)
+                                   slot_mapping=group.slot_mapping if self.makes_latent else None, interleaved=pairs,
+                                   cq_gain=self.dq_norm if self.q_rank else None, cq_out=cq)
+            if self.q_rank:
+                q = ws.get("latent_queries", n, self.q_width, ctx.dtype)
+                linear(ctx, cq, self.q_weight, None, q, n)
+                kernels.latent_prepare(q, 0, self.n_head, self.head_dim, *rot, interleaved=pairs)
         elif self.makes_latent:
             kernels.rms_norm_store(z[:, split:], self.dkv_norm, self.eps, pool, group.slot_mapping, n)
         q_lat = ws.get("latent_q", n, self.n_head * self.row, ctx.dtype)
-        kernels.heads_linear(z, self.uk_folded, q_lat, n, fast=fast)
+        kernels.heads_linear(q, self.uk_folded, q_lat, n, fast=fast)
         o_lat = ws.get("latent_o", n, self.n_head * self.row, ctx.dtype)
-        gate = z[:, self.q_width:split]
+        gate = z[:, q_cols:split] if self.has_gate else None
         attention_ops.paged_attention(ctx, q_lat, o_lat, pool, pool, group, self.n_head, self.scale, self.window,
-                                      sinks=self.sink, gate=gate if self.head_gate else None)
+                                      sinks=self.sink if self.has_sinks else None, gate=gate if self.head_gate else None)
         y = ws.get("attn_out", n, self.y_width, ctx.dtype)
         kernels.heads_linear(o_lat, self.uv_heads, y, n, gate=None if self.head_gate else gate, fast=fast)
         linear_add(ctx, y, self.out_weight, None, x, n)
@@ -347,7 +372,9 @@ class GatedAttention(Mixer):
     sigmoid(score + b_a) with a number per head (the tensor `score_bias`), not normalised over the keys;
     `out_bias`: the output projection has a bias; `sinks`: one more term exp(sink_a) in the softmax's denominator,
     a number per head with no key and no value; `chunked`: `window` is the size of chunks counted from position 0, and
-    a query sees the keys of its own chunk; `bias_max` = M: the number rel[bucket(i - j)][a] (the tensor `rel`
+    a query sees the keys of its own chunk; `sink_score`: the same term with one constant score for all heads;
+    `query_temperature` = (c, n): queries at position p are multiplied by 1 + c ln(floor((p + 1) / n) + 1) behind norm
+    and rotation; `slopes` (a number per head): slopes[a] (i - j) is taken off the scaled, capped score; `bias_max` = M: the number rel[bucket(i - j)][a] (the tensor `rel`
     [B, H]) is added to the scaled score of query i and key j, with the buckets of distance_buckets(B, M).
 
     The cache keeps keys and values in pages of one head size, so both are laid out with
@@ -363,7 +390,8 @@ class GatedAttention(Mixer):
                  share: str = "values", conv_taps: int = 0, window: int = 0, keep_first: int = 0,
                  qk_norm_weights: Optional[str] = None, values_from_keys: bool = False, score_bias: bool = False,
                  out_bias: bool = False, sinks: bool = False, chunked: bool = False,
-                 bias_max: Optional[int] = None) -> None:
+                 bias_max: Optional[int] = None, sink_score: Optional[float] = None, query_temperature=None,
+                 slopes=None) -> None:
         self.width, self.n_head, self.n_kv_head = int(width), int(n_head), int(n_kv_head)
         self.head_dim, self.value_dim, self.scale = int(head_dim), int(value_dim), float(scale)
         self.has_bias, self.has_gate = bool(bias), bool(head_gate)
@@ -387,8 +415,8 @@ class GatedAttention(Mixer):
             raise ValueError("qk_norm_weights is None, 'head' or 'whole', and needs qk_norm_eps")
         self.qk_norm_weights = qk_norm_weights
         self.values_from_keys, self.has_score_bias, self.has_out_bias = bool(values_from_keys), bool(score_bias), bool(out_bias)
-        if self.values_from_keys and (self.value_dim != self.head_dim or self.value_mix is not None or self.conv_taps > 1):
-            raise ValueError("values that are the keys have the keys' size, and are neither mixed nor convolved")
+        if self.values_from_keys and (self.value_dim != self.head_dim or self.value_mix is not None):
+            raise ValueError("values that are the keys have the keys' size, and are not mixed")
         if self.has_score_bias and self.softcap > 0.0:
             raise ValueError("sigmoid weights take no score cap")
         self.has_sinks, self.chunked = bool(sinks), bool(chunked and self.window)
@@ -397,6 +425,15 @@ class GatedAttention(Mixer):
             raise ValueError("sigmoid weights take neither sinks nor numbers by distance")
         if self.bias_max is not None and self.softcap > 0.0:
             raise ValueError("numbers by distance go with no score cap")
+        self.sink_score = None if sink_score is None else float(sink_score)
+        self.query_temperature = None if query_temperature is None else (float(query_temperature[0]), int(query_temperature[1]))
+        self.slope_values = None if slopes is None else [float(v) for v in slopes]
+        if self.query_temperature is not None and self.query_temperature[1] <= 0:
+            raise ValueError("a query temperature needs a positive period")
+        if self.slope_values is not None and (len(self.slope_values) != self.n_head or self.has_score_bias or self.bias_max is not None):
+            raise ValueError("slopes are one number per head, and go with neither sigmoid weights nor numbers by distance")
+        if self.sink_score is not None and (self.has_sinks or self.has_score_bias):
+            raise ValueError("a constant sink takes the place of the heads' own, and goes with a softmax")
         size = max(self.head_dim, self.value_dim)
         self.head_stride = -(-size // 32) * 32 if size <= 128 else -(-size // 8) * 8
         if self.head_stride > 512:
@@ -406,7 +443,7 @@ class GatedAttention(Mixer):
         self.v_off = self.k_off + self.n_kv_head * s
         self.g_off = self.v_off + (0 if self.values_from_keys else self.n_kv_head * s)
         self.in_rows = -(-(self.g_off + (self.n_head if self.has_gate else 0)) // 16) * 16
-        self.in_weight = self.in_bias = self.out_padded = self.conv_weight = self.dist_bias = None
+        self.in_weight = self.in_bias = self.out_padded = self.conv_weight = self.dist_bias = self.slopes = None
 
     def weight_requests(self) -> Dict[str, WeightRequest]:
         H, G, D, E, W = self.n_head, self.n_kv_head, self.head_dim, self.value_dim, self.width
@@ -425,10 +462,11 @@ class GatedAttention(Mixer):
             req["sink"] = WeightRequest((H,), VECTOR)
         if self.bias_max is not None:
             req["rel"] = WeightRequest((-1, H), VECTOR)      # (the stored table says how many buckets there are)
-        if self.conv_taps > 1:
+        if self.conv_taps > 0:
             J = self.conv_taps
-            req.update(q_conv=WeightRequest((H * D, J), VECTOR), k_conv=WeightRequest((G * D, J), VECTOR),
-                       v_conv=WeightRequest((G * E, J), VECTOR))
+            req.update(q_conv=WeightRequest((H * D, J), VECTOR), k_conv=WeightRequest((G * D, J), VECTOR))
+            if not self.values_from_keys:
+                req["v_conv"] = WeightRequest((G * E, J), VECTOR)
         if self.has_bias:
             req.update(q_bias=WeightRequest((H * D,), VECTOR), k_bias=WeightRequest((G * D,), VECTOR))
             if not self.values_from_keys:
@@ -467,13 +505,19 @@ class GatedAttention(Mixer):
                     continue
                 bias[at:at + heads * s].view(heads, s)[:, :size].copy_(tensors[name].view(heads, size))
             self.in_bias = bias
-        if self.conv_taps > 1:
+        if self.conv_taps > 0:
             # the taps of the padded layout's channels (zeros for the channels a head does not have)
             taps = torch.zeros((self.g_off, self.conv_taps), dtype=torch.float32, device=q.device)
             for name, at, heads, size in (("q_conv", self.q_off, H, D), ("k_conv", self.k_off, G, D),
                                           ("v_conv", self.v_off, G, E)):
+                if name not in tensors:
+                    continue
                 taps[at:at + heads * s].view(heads, s, -1)[:, :size].copy_(tensors[name].view(heads, size, -1))
             self.conv_weight = taps
+        if self.sink_score is not None:
+            self.sink = torch.full((H,), self.sink_score, dtype=torch.float32, device=q.device)
+        if self.slope_values is not None:
+            self.slopes = torch.tensor(self.slope_values, dtype=torch.float64).to(torch.float32).to(q.device)
         if self.bias_max is not None:
             # bucket by bucket to distance by distance, head by head: what the attention kernels read
             rel = tensors["rel"]
@@ -503,12 +547,13 @@ class GatedAttention(Mixer):
         n, ws, s = ctx.n_rows, ctx.workspace, self.head_stride
         z = ws.get("gated_attention_in", n, self.in_rows, ctx.dtype)
         linear(ctx, h, self.in_weight, self.in_bias, z, n)
-        if self.conv_taps > 1:
+        if self.conv_taps > 0:
             # q, k and v through their short convolution into a second buffer (a token reads the inputs of the
             # tokens before it); the gate's columns, if any, stay where they are
             zc = ws.get("gated_attention_conv", n, self.in_rows, ctx.dtype)
-            kernels.short_conv(z, 0, self.conv_weight, None, ctx.state_pools[binding.state], ctx.state_slots, ctx.cu_q,
-                               ctx.q_req, ctx.positions, ctx.cu_q.numel() - 1, zc, 0, n)
+            kept = ctx.state_pools[binding.state] if self.conv_taps > 1 else None      # (one tap keeps no inputs)
+            kernels.short_conv(z, 0, self.conv_weight, None, kept, ctx.state_slots, ctx.cu_q, ctx.q_req,
+                               ctx.positions, ctx.cu_q.numel() - 1, zc, 0, n)
             gate_rows, z = z, zc
         else:
             gate_rows = z
@@ -526,15 +571,21 @@ class GatedAttention(Mixer):
                            norm=self.qk_norm_weights, q_norm_weight=self.q_norm if self.qk_norm_weights else None,
                            k_norm_weight=self.k_norm if self.qk_norm_weights else None,
                            values_from_keys=self.values_from_keys,
-                           rot_magnitude=getattr(self.rotation, "magnitude", 1.0))
+                           rot_magnitude=getattr(self.rotation, "magnitude", 1.0),
+                           interleaved=getattr(self.rotation, "interleaved", False), query_temperature=self.query_temperature)
         y = ws.get("attn_out", n, self.n_head * s, ctx.dtype)
         # (the gate per head is applied by the attention kernel as it stores a head's output)
         attention_ops.paged_attention(ctx, z, y, k_pool, v_pool, group, self.n_head, self.scale, self.window,
                                       softcap=self.softcap, gate=gate_rows[:, self.g_off:] if self.has_gate else None,
                                       keep_first=self.keep_first, score_bias=self.score_bias if self.has_score_bias else None,
-                                      sinks=self.sink if self.has_sinks else None, chunked=self.chunked,
-                                      dist_bias=self.dist_bias)
+                                      sinks=self.sink if self.has_sinks or self.sink_score is not None else None,
+                                      chunked=self.chunked, dist_bias=self.dist_bias, slopes=self.slopes)
         linear_add(ctx, y, self.out_padded, self.out_bias if self.has_out_bias else None, x, n)
+
+
+def geometric_slopes(n_head: int) -> List[float]:
+    """2^(-8 (a + 1) / H) for head a of H: slopes of a distance bias, from the steepest to 2^-8."""
+    return [2.0 ** (-8.0 * (a + 1) / n_head) for a in range(n_head)]
 
 
 @register_mixer("decay_state")
@@ -926,4 +977,95 @@ class GatedDeltaRule(Mixer):
         else:
             kernels.delta_state(qkv, 0, self.k_off, self.v_off, *sizes, y, n, q_scale=self.q_scale, gate_off=self.g_off,
                                 norm_weight=self.norm_weight, eps=self.norm_eps)
+        linear_add(ctx, y, self.out_weight, None, x, n)
+
+
+@register_mixer("gated_diagonal_state")
+class GatedDiagonalState(Mixer):
+    """A recurrence with one float32 number of state per channel, behind a short convolution and beside a gelu branch.
+
+    y = gelu_tanh(h Wy^T + by) and u = conv(h Wx^T + bx) (+ bias), both [C], the convolution causal over time, channel by
+    channel (`conv_weight` [C, J], the last tap on the current token, zeros before the sequence's start).  The channels come
+    in B equal blocks, each with square matrices of its own: r = sigmoid(Wr_b u_b + br), i = sigmoid(Wi_b u_b + bi);
+    log a = -`decay_scale` r softplus(lam), S_t = a S_(t-1) + sqrt(1 - a^2) i u_t, S zero before the first token;
+    out = (S * y) Wo^T, added into the residual.  Kept per request: S and the convolution's last J - 1 inputs.  The two
+    gates (from their products' sums on), the decay and the recurrence are float32 up to S * y."""
+
+    graph_safe = True
+    plan_safe = True
+
+    def __init__(self, width: int, channels: int, blocks: int, conv_taps: int, decay_scale: float = 8.0) -> None:
+        self.width, self.channels, self.blocks, self.conv_taps = int(width), int(channels), int(blocks), int(conv_taps)
+        self.decay_scale = float(decay_scale)
+        if self.blocks <= 0 or self.channels % self.blocks:
+            raise ValueError(f"{channels} channels do not come in {blocks} equal blocks")
+        if not 1 <= self.conv_taps <= kernels.MAX_CONV_TAPS:
+            raise ValueError(f"the convolution takes 1 to {kernels.MAX_CONV_TAPS} taps")
+        self.block = self.channels // self.blocks
+        # rows of the stacked projection: [x | y], each part padded so that the other's columns start 16 bytes apart
+        self.y_off = -(-self.channels // 16) * 16
+        self.in_rows = 2 * self.y_off
+        self.conv_numel = (self.conv_taps - 1) * self.channels
+        self.in_weight = self.in_bias = self.gate_weights = self.decay = None
+
+    def weight_requests(self) -> Dict[str, WeightRequest]:
+        C, B, S, W = self.channels, self.blocks, self.block, self.width
+        return {"y_weight": WeightRequest((C, W), MATRIX), "y_bias": WeightRequest((C,), VECTOR),
+                "x_weight": WeightRequest((C, W), MATRIX), "x_bias": WeightRequest((C,), VECTOR),
+                "conv_weight": WeightRequest((C, self.conv_taps), VECTOR), "conv_bias": WeightRequest((C,), VECTOR),
+                "r_weight": WeightRequest((B, S, S), MATRIX), "r_bias": WeightRequest((B, S), VECTOR),
+                "i_weight": WeightRequest((B, S, S), MATRIX), "i_bias": WeightRequest((B, S), VECTOR),
+                "lam": WeightRequest((C,), VECTOR), "out_weight": WeightRequest((W, C), MATRIX)}
+
+    def token_matrix_elements(self) -> int:
+        if self.in_weight is None:
+            return 0
+        return self.in_weight.numel() + self.gate_weights.numel() + self.out_weight.numel()
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        C, W, x = self.channels, self.width, tensors["x_weight"]
+        self.in_weight = torch.zeros((self.in_rows, W), dtype=x.dtype, device=x.device)
+        self.in_bias = torch.zeros(self.in_rows, dtype=torch.float32, device=x.device)
+        views = {}
+        for name, at in (("x", 0), ("y", self.y_off)):
+            self.in_weight[at:at + C].copy_(tensors[name + "_weight"])
+            self.in_bias[at:at + C].copy_(tensors[name + "_bias"])
+            views[name + "_weight"] = self.in_weight[at:at + C]
+        # block by block the two gates' matrices one under the other: one product per block makes both
+        self.gate_weights = torch.cat([tensors["r_weight"], tensors["i_weight"]], dim=1).contiguous()
+        views["r_weight"], views["i_weight"] = self.gate_weights[:, :self.block], self.gate_weights[:, self.block:]
+        for name, view in views.items():
+            setattr(self, name, view)
+        self.r_bias_flat, self.i_bias_flat = tensors["r_bias"].reshape(-1).contiguous(), tensors["i_bias"].reshape(-1).contiguous()
+        # -decay_scale softplus(lam), once, in double precision
+        lam = tensors["lam"].to(torch.float64)
+        softplus = torch.clamp(lam, min=0.0) + torch.log1p(torch.exp(-lam.abs()))
+        self.decay = (-self.decay_scale * softplus).to(torch.float32).contiguous()
+        return views
+
+    def cache_need(self) -> StateNeed:
+        return StateNeed(self.channels + self.conv_numel)
+
+    def forward_add(self, ctx: StepContext, h, x: torch.Tensor, binding: CacheBinding,
+                    position: PositionEncoding) -> None:
+        if binding.kind != "state":
+            raise ValueError("a diagonal state needs a state pool")
+        plain_residual(ctx, h, x)
+        n, ws, C = ctx.n_rows, ctx.workspace, self.channels
+        n_req, pool = ctx.cu_q.numel() - 1, ctx.state_pools[binding.index]
+        z = ws.get("diagonal_in", n, self.in_rows, ctx.dtype)
+        linear(ctx, h, self.in_weight, self.in_bias, z, n)
+        u = ws.get("diagonal_conv", n, C, ctx.dtype)
+        kernels.short_conv(z, 0, self.conv_weight, self.conv_bias, pool[:, C:] if self.conv_taps > 1 else None, ctx.state_slots,
+                           ctx.cu_q, ctx.q_req, ctx.positions, n_req, u, 0, n)
+        gates = ws.get("diagonal_gates", n, 2 * C, ctx.dtype)
+        kernels.heads_linear(u, self.gate_weights, gates, n, fast=not ctx.exact)
+        scratch = None
+        if not ctx.decode_only:
+            floats = kernels.diagonal_scratch_floats(n, n_req, C)
+            scratch = ws.get("diagonal_scratch", floats, 1, torch.float32)
+        y = ws.get("diagonal_out", n, C, ctx.dtype)
+        kernels.diagonal_state(u, gates, self.r_bias_flat, self.i_bias_flat, self.decay, self.block, pool[:, :C], ctx.state_slots,
+                               ctx.cu_q, ctx.positions, n_req, n, y, y=z[:, self.y_off:self.y_off + C], scratch=scratch)
         linear_add(ctx, y, self.out_weight, None, x, n)

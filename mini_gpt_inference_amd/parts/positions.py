@@ -82,6 +82,7 @@ class RotaryHalf(PositionEncoding):
     graph_safe = True
     plan_safe = True
     rotates = True
+    interleaved = False     # whether the pairs are neighbours (2i, 2i + 1)
 
     def __init__(self, dims: int, base: float, factor: float = 1.0, scaling: Optional[dict] = None) -> None:
         self.dims, self.base, self.factor = int(dims), float(base), float(factor)
@@ -139,3 +140,10 @@ class RotaryHalf(PositionEncoding):
             f = torch.tensor(self.frequency_values(), dtype=torch.float64).to(torch.float32).to(device)
             self._freq[device] = f
         return f
+
+
+@register_position("rotary_interleaved")
+class RotaryInterleaved(RotaryHalf):
+    """The same rotation with neighbouring channels as pairs: channel 2i with channel 2i + 1."""
+
+    interleaved = True
