@@ -389,16 +389,40 @@ def gekopel_like(layers, width, heads, vocab):
             "embedding": {"scale": float(width) ** 0.5}, "layers": out}
 
 
+def telapel_like(layers, width, heads, vocab):
+    """A Telapel config.json of a GPT-2-style model's size: the same layers, width, heads and vocabulary; recurrence,
+    latent attention, windowed attention and recurrence in turn; the recurrence over as many channels as the model is
+    wide in blocks of 256 with four taps; attention heads of 128 channels, a quarter as many key/value heads, a window of
+    512; latents of 96 values beside a rotated part of 32 (a cached row of 128), queries from a latent of 3/4 width; every
+    token goes through 8 width^2 feed-forward elements a layer (2 of 8 gated experts of hidden size width in 4 groups of
+    which 3 stay, beside a shared one of about 2/3 width)."""
+    out = []
+    for i in range(layers):
+        kind = ("rglru", "latent_attention", "attention", "rglru")[i % 4]
+        if kind == "rglru":
+            mixer = {"width": width, "blocks": max(width // 256, 1), "conv": 4}
+        elif kind == "latent_attention":
+            mixer = {"heads": heads, "dim": 96, "rot_dim": 32, "vdim": 128, "q_rank": width * 3 // 4, "kv_rank": 96,
+                     "scale": 128 ** -0.5, "rot": {"base": 1e4, "dims": 32}}
+        else:
+            mixer = {"heads": heads, "kv_heads": max(heads // 4, 1), "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "conv": 4,
+                     "softcap": 30.0, "mask": {"size": 512}, "q_temp": {"coef": 0.1, "every": 8192}}
+        out.append({"type": kind, "mixer": mixer, "mlp": {
+            "kind": "moe", "expert": {"ff": width, "limit": 7.0}, "shared": {"ff": 2 * width // 3 // 128 * 128, "limit": 7.0},
+            "router": {"experts": 8, "top": 2, "groups": {"count": 4, "keep": 3}}}})
+    return {"architecture": "Telapel", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": out}
+
+
 COMPARED = {"viperax": viperax_like, "bobevik": bobevik_like, "rilavik": rilavik_like, "nutitar": nutitar_like,
-            "gekopel": gekopel_like}
+            "gekopel": gekopel_like, "telapel": telapel_like}
 # the model a design is measured beside: the GPT-2-style model, or the design nearest to it
-BESIDE = {"rilavik": "bobevik", "gekopel": "rilavik"}
+BESIDE = {"rilavik": "bobevik", "gekopel": "rilavik", "telapel": "gekopel"}
 
 
 def compare_run(args, name):
-    """--compare viperax | bobevik | rilavik | nutitar | gekopel: prefill (2 prompts of 1,024 tokens as one step) and decode
+    """--compare viperax | bobevik | rilavik | nutitar | gekopel | telapel: prefill (2 prompts of 1,024 tokens as one step) and decode
     (batch 8, by the default run's timing rule, fewer blocks) of that design beside the GPT-2-style model
-    (Rilavik: beside Bobevik, Gekopel: beside Rilavik, the nearest designs) at equal layers, width, heads and vocabulary, random
+    (Rilavik: beside Bobevik, Gekopel: beside Rilavik, Telapel: beside Gekopel, the nearest designs) at equal layers, width, heads and vocabulary, random
     weights, at COMPARE_SIZES.  One JSON line."""
     import argparse as _argparse
     import gc

@@ -202,6 +202,10 @@ int mgpt_diagonal_state(const void* u, int u_dtype, long ldu, const void* g, int
     const float* i_bias, const float* decay, int block, const void* y, int y_dtype, long ldy, int y_off, float* state, long ld_state,
     const int* state_slots, const int* cu_q, const int* positions, int n_req, int n_tokens, int channels, float* scratch,
     long scratch_floats, void* out, int out_dtype, long ldo, hipStream_t stream);
+int mgpt_diagonal_state_fused(const void* z, long ldz, int y_off, const float* conv_w, const float* conv_b, int taps,
+    const void* w, const float* r_bias, const float* i_bias, const float* decay, int block, int channels, float* state,
+    long ld_state, const int* state_slots, const int* cu_q, const int* positions, int n_req, int n_tokens, float* scratch,
+    long scratch_floats, const void* u, void* out, long ldo, hipStream_t stream);
 // delta_state.hip
 int mgpt_delta_state(const void* x, int dtype, long ldx, int q_off, int k_off, int v_off, const void* z, long ldz,
     int b_off, int a_off, int gate_off, int n_head, int n_group, int head_dim, int value_dim, float q_scale,
@@ -216,7 +220,8 @@ int mgpt_delta_state_chunked(const void* x, int dtype, long ldx, int q_off, int 
 // short_conv.hip
 int mgpt_short_conv(const void* u, int dtype, long ldu, int u_off, const float* w, const float* bias, int act,
     float* state, long ld_state, const int* state_slots, const int* cu_q, const int* q_req, const int* positions,
-    int n_req, void* out, int out_dtype, long ldo, int o_off, int n_tokens, int channels, int taps, hipStream_t stream);
+    int n_req, void* out, int out_dtype, long ldo, int o_off, int n_tokens, int channels, int taps, int single,
+    hipStream_t stream);
 // qk_prepare.hip
 int mgpt_qk_prepare(void* z, int dtype, long ldz, int q_off, int k_off, int v_off, int n_head, int n_kv_head,
     int head_dim, int value_dim, int head_stride, const int* positions, const float* freq, int rot_dims, float norm_eps,
@@ -289,6 +294,7 @@ int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_st
   X(mgpt_rms_post_norm) \
   X(mgpt_cast_rows) \
   X(mgpt_diagonal_state) \
+  X(mgpt_diagonal_state_fused) \
   X(mgpt_qk_prepare) \
   X(mgpt_decay_state) \
   X(mgpt_decay_state_chunked) \

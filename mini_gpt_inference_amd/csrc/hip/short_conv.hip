@@ -14,20 +14,38 @@
 
 #define SC_MAX_TAPS 9
 
-// A thread a (token, channel): steps of few tokens a request (decode steps), where a run of tokens would be a chain
+// A thread a (token, channel); with `keep` (every request brings at most one token) the thread, which is then the only
+// one that reads its channel's inputs of that request, also brings them up to date.  Steps of few tokens a request (decode steps), where a run of tokens would be a chain
 // of dependent loads of one request's data after the other.
 template <typename UT, typename OT>
 __global__ __launch_bounds__(256) void short_conv_token_kernel(
     const UT* __restrict__ u, long ldu, int u_off, const float* __restrict__ w, const float* __restrict__ bias,
-    int act, const float* __restrict__ state, long ld_state, const int* __restrict__ state_slots,
+    int act, float* __restrict__ state, long ld_state, const int* __restrict__ state_slots,
     const int* __restrict__ cu_q, const int* __restrict__ q_req, const int* __restrict__ positions, OT* __restrict__ out,
-    long ldo, int o_off, int C, int J) {
+    long ldo, int o_off, int C, int J, int keep) {
   const int n = blockIdx.x;
   const int c = blockIdx.y * 256 + threadIdx.x;
   const int r = q_req[n];
   if (r < 0 || c >= C) return;      // a token of the padding
   const int start = cu_q[r], p = positions[n], slot = state_slots[r];
   float acc = bias ? bias[c] : 0.f;
+  if (keep) {
+    float* st = state + (long)(slot >= 0 ? slot : 0) * ld_state + c;
+    const float now = to_float<UT>(u[(long)n * ldu + u_off + c]);
+    float in[SC_MAX_TAPS];
+#pragma unroll
+    for (int j = 0; j < SC_MAX_TAPS; ++j)
+      if (j < J) in[j] = j == J - 1 ? now : (slot >= 0 && p - (J - 1 - j) >= 0 ? st[(long)j * C] : 0.f);
+#pragma unroll
+    for (int j = 0; j < SC_MAX_TAPS; ++j)
+      if (j < J && p - (J - 1 - j) >= 0) acc = fmaf(w[(long)c * J + j], in[j], acc);
+#pragma unroll
+    for (int j = 1; j < SC_MAX_TAPS; ++j)
+      if (j < J && slot >= 0) st[(long)(j - 1) * C] = in[j];
+    if (act == 1) acc = acc / (1.0f + expf(-acc));
+    out[(long)n * ldo + o_off + c] = from_float<OT>(acc);
+    return;
+  }
   for (int j = 0; j < J; ++j) {
     const int back = J - 1 - j;
     if (p - back < 0) continue;     // before the sequence's start
@@ -126,11 +144,11 @@ __global__ __launch_bounds__(256) void short_conv_state_kernel(
 
 // u: rows in `dtype`, the C channels at u_off; w: float32 [C][J]; bias: float32 [C] or null; act: 0 none, 1 silu.
 // state: rows of ld_state floats, (J - 1) * C of them used (with one tap none: it may be null).  out: rows in out_dtype, the C channels at o_off
-// (not the rows of u: a token reads the inputs of the tokens before it).
+// (not the rows of u: a token reads the inputs of the tokens before it).  single: no request brings more than one token.
 extern "C" int mgpt_short_conv(const void* u, int dtype, long ldu, int u_off, const float* w, const float* bias, int act,
                                float* state, long ld_state, const int* state_slots, const int* cu_q, const int* q_req,
                                const int* positions, int n_req, void* out, int out_dtype, long ldo, int o_off,
-                               int n_tokens, int channels, int taps, hipStream_t stream) {
+                               int n_tokens, int channels, int taps, int single, hipStream_t stream) {
   if (n_tokens == 0 || n_req == 0) return MGPT_OK;
   if (!u || !w || (!state && taps > 1) || !state_slots || !cu_q || !q_req || !positions || !out) return MGPT_ERR_NULL;
   if (!dtype_ok(dtype) || !dtype_ok(out_dtype)) return MGPT_ERR_BAD_DTYPE;
@@ -140,7 +158,8 @@ extern "C" int mgpt_short_conv(const void* u, int dtype, long ldu, int u_off, co
   const int cb = (channels + 255) / 256;
   if (cb > 65535) return MGPT_ERR_TOO_LARGE;
   // steps with runs of tokens (prompt portions): a workgroup a run of SC_TB tokens; few tokens a request: a token
-  const bool runs = n_tokens >= 4 * n_req && n_tokens >= 64;
+  const bool runs = !single && n_tokens >= 4 * n_req && n_tokens >= 64;
+  const int keep = single && taps > 1;
 #define SC_LAUNCH(UT, OT)                                                                                                 \
   {                                                                                                                       \
     if (runs)                                                                                                             \
@@ -150,14 +169,14 @@ extern "C" int mgpt_short_conv(const void* u, int dtype, long ldu, int u_off, co
     else                                                                                                                  \
       hipLaunchKernelGGL((short_conv_token_kernel<UT, OT>), dim3(n_tokens, cb), dim3(256), 0, stream, (const UT*)u, ldu,  \
                          u_off, w, bias, act, state, ld_state, state_slots, cu_q, q_req, positions, (OT*)out, ldo, o_off, \
-                         channels, taps);                                                                                 \
+                         channels, taps, keep);                                                                           \
   }
   if (dtype == MGPT_F32 && out_dtype == MGPT_F32) SC_LAUNCH(float, float)
   else if (dtype == MGPT_F32) SC_LAUNCH(float, bf16_t)
   else if (out_dtype == MGPT_F32) SC_LAUNCH(bf16_t, float)
   else SC_LAUNCH(bf16_t, bf16_t)
 #undef SC_LAUNCH
-  if (taps > 1)
+  if (taps > 1 && !keep)
     hipLaunchKernelGGL(short_conv_state_kernel, dim3(n_req, cb), dim3(256), 0, stream, u, dtype, ldu, u_off, state, ld_state,
                        state_slots, cu_q, channels, taps);
   return mgpt_last_error();

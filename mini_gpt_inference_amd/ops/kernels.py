@@ -1928,11 +1928,12 @@ CONV_ACTIVATIONS = {None: 0, "silu": 1}
 
 def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
                state_slots: torch.Tensor, cu_q: torch.Tensor, q_req: torch.Tensor, positions: torch.Tensor, n_req: int,
-               out: torch.Tensor, o_off: int, n_tokens: int, activation: Optional[str] = None) -> None:
+               out: torch.Tensor, o_off: int, n_tokens: int, activation: Optional[str] = None, single: bool = False) -> None:
     """out[t][o_off + c] = act(sum_j weight[c][j] * u_(t - taps + 1 + j)[u_off + c] (+ bias[c])) over time inside each
     request, zeros before position 0; the taps - 1 inputs before the step's first token come from the request's
     slot of `state` (float32 rows holding [taps - 1][channels], a view of a pool's columns will do), which is then
-    brought up to date (with one tap there is none: None).  weight: float32 [channels, taps]."""
+    brought up to date (with one tap there is none: None).  weight: float32 [channels, taps].  single promises that no
+    request brings more than one token."""
     _need_cuda(u, weight, bias, state, state_slots, cu_q, q_req, positions, out)
     _need(activation in CONV_ACTIVATIONS, f"short_conv: activation {activation!r} is none of {sorted(map(str, CONV_ACTIVATIONS))}")
     _need(weight.dtype == torch.float32 and weight.dim() == 2 and weight.is_contiguous(), "short_conv: weight must be dense float32 [channels, taps]")
@@ -1953,8 +1954,8 @@ def short_conv(u: torch.Tensor, u_off: int, weight: torch.Tensor, bias: Optional
     rc = library.kernels().mgpt_short_conv(
         _ptr(u), _dtype_code(u), u.stride(0), u_off, _ptr(weight), _ptr(bias), CONV_ACTIVATIONS[activation], _ptr(state),
         state.stride(0) if state is not None else 0, _ptr(state_slots), _ptr(cu_q), _ptr(q_req), _ptr(positions), n_req, _ptr(out), _dtype_code(out),
-        out.stride(0), o_off, n_tokens, channels, taps, _stream())
-    _check(rc, "short_conv", 2 if taps > 1 else 1)
+        out.stride(0), o_off, n_tokens, channels, taps, int(single), _stream())
+    _check(rc, "short_conv", 2 if taps > 1 and not single else 1)
 
 
 DIAGONAL_CHUNK = 32     # tokens a chunk of diagonal_state
@@ -2000,3 +2001,70 @@ def diagonal_state(u: torch.Tensor, gates: torch.Tensor, r_bias: torch.Tensor, i
         state.stride(0), _ptr(state_slots), _ptr(cu_q), _ptr(positions), n_req, n_tokens, channels, _ptr(scratch),
         scratch.numel() if scratch is not None else 0, _ptr(out), _dtype_code(out), out.stride(0), _stream())
     _check(rc, "diagonal_state", 2 if scratch is not None else 1)
+
+
+def diagonal_fused_scratch_floats(n_tokens: int, channels: int) -> int:
+    """float32 values of scratch that diagonal_state_fused uses for a step in which a request may bring several tokens."""
+    return 2 * n_tokens * channels
+
+
+def pack_diagonal_gates(r_weight: torch.Tensor, i_weight: torch.Tensor) -> Optional[torch.Tensor]:
+    """The matrices of the two gates, [blocks, block, block] each, in the order in which diagonal_state_fused takes them:
+    [channels / 16, 2, inner / 32, 64 lanes, 8], lane (g, c) with row c and inner channels 8 g .. 8 g + 7, the inner size
+    rounded up to a multiple of 32 with zeros.  None for types and block sizes that kernel does not take."""
+    blocks, block, _ = r_weight.shape
+    if r_weight.dtype != torch.bfloat16 or block % 16 or block > 512:
+        return None
+    steps = -(-block // 32)
+    both = torch.zeros((blocks, 2, block, steps * 32), dtype=r_weight.dtype, device=r_weight.device)
+    both[:, 0, :, :block], both[:, 1, :, :block] = r_weight, i_weight
+    order = both.view(blocks, 2, block // 16, 16, steps, 4, 8).permute(0, 2, 1, 4, 5, 3, 6)
+    return order.reshape(blocks * (block // 16), 2, steps, 64, 8).contiguous()
+
+
+def diagonal_state_fused(z: torch.Tensor, y_off: int, conv_weight: torch.Tensor, conv_bias: torch.Tensor, weights: torch.Tensor, block: int,
+                         r_bias: torch.Tensor, i_bias: torch.Tensor, decay: torch.Tensor, state: torch.Tensor,
+                         state_slots: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor, n_req: int, n_tokens: int,
+                         out: torch.Tensor, u: Optional[torch.Tensor] = None, scratch: Optional[torch.Tensor] = None) -> bool:
+    """diagonal_state in bfloat16 with its gates' products inside, and for steps in which requests bring several tokens
+    (scratch given: float32, diagonal_fused_scratch_floats) the short convolution in front as well.
+
+    z: rows [the convolution's input: channels | .. | y at y_off]; conv_weight: float32 [taps, channels] (the last row on
+    the current token), conv_bias float32 [channels]; weights: pack_diagonal_gates'; state: float32 rows [channels: S | (taps - 1) * channels: the
+    convolution's last inputs].  In a step of single tokens (no scratch; token n is request n) u holds the convolution's
+    output, made by short_conv: dense rows of the channels.  False, with nothing launched, for sizes and alignments it
+    does not take."""
+    if z.dtype != torch.bfloat16 or weights.dtype != torch.bfloat16:
+        return False
+    _need_cuda(z, conv_weight, conv_bias, weights, r_bias, i_bias, decay, state, state_slots, cu_q, positions, u, out, scratch)
+    channels, taps = decay.numel(), conv_weight.shape[0]
+    _need(block > 0 and block % 16 == 0 and channels % block == 0 and weights.is_contiguous()
+          and tuple(weights.shape) == (channels // 16, 2, -(-block // 32), 64, 8), "diagonal_state_fused: weights as pack_diagonal_gates makes them")
+    _need(conv_weight.dtype == torch.float32 and conv_weight.is_contiguous() and conv_weight.shape == (taps, channels),
+          "diagonal_state_fused: conv_weight must be dense float32 [taps, channels]")
+    for name, t in (("conv_bias", conv_bias), ("r_bias", r_bias), ("i_bias", i_bias), ("decay", decay)):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() == channels, f"diagonal_state_fused: {name} must be float32 [channels]")
+    _rows_2d("diagonal_state_fused z", z, n_tokens)
+    _rows_2d("diagonal_state_fused out", out, n_tokens)
+    _need(z.shape[1] >= y_off + channels and out.shape[1] >= channels and out.dtype == z.dtype,
+          "diagonal_state_fused: z and out must be bfloat16 rows of the channels")
+    _need((u is None) == (scratch is not None), "diagonal_state_fused: scratch for prompt portions, u for single tokens")
+    if u is not None:
+        _rows_2d("diagonal_state_fused u", u, n_tokens)
+        _need(u.shape[1] == channels and u.is_contiguous() and u.dtype == z.dtype, "diagonal_state_fused: u must be dense rows of the channels")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] >= taps * channels,
+          "diagonal_state_fused: state must be float32 rows of taps * channels")
+    _need_i32("state_slots", state_slots, n_req)
+    _need_i32("cu_q", cu_q, n_req + 1)
+    _need_i32("positions", positions, n_tokens)
+    if scratch is not None:
+        _need(scratch.dtype == torch.float32 and scratch.is_contiguous()
+              and scratch.numel() >= diagonal_fused_scratch_floats(n_tokens, channels), "diagonal_state_fused: too little scratch")
+    rc = library.kernels().mgpt_diagonal_state_fused(
+        _ptr(z), z.stride(0), int(y_off), _ptr(conv_weight), _ptr(conv_bias), taps, _ptr(weights), _ptr(r_bias), _ptr(i_bias),
+        _ptr(decay), int(block), channels, _ptr(state), state.stride(0), _ptr(state_slots), _ptr(cu_q), _ptr(positions),
+        n_req, n_tokens, _ptr(scratch), scratch.numel() if scratch is not None else 0, _ptr(u), _ptr(out), out.stride(0), _stream())
+    if rc == -2:
+        return False
+    _check(rc, "diagonal_state_fused", 2 if scratch is not None else 1)
+    return True

@@ -186,11 +186,12 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_gated_state_chunked": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, I, P, P, P, L, P],
         # a diagonal state with its gates from block products
         "mgpt_diagonal_state": [P, I, L, P, I, L, P, P, P, I, P, I, L, I, P, L, P, P, P, I, I, I, P, L, P, I, L, P],
+        "mgpt_diagonal_state_fused": [P, L, I, P, P, I, P, P, P, P, I, I, P, L, P, P, P, I, I, P, L, P, P, L, P],
         # the gated delta rule
         "mgpt_delta_state": [P, I, L, I, I, I, P, L, I, I, I, I, I, I, I, F, P, P, P, F, P, L, P, P, I, P, P, L, P],
         "mgpt_delta_image_floats": [I, I, I, I],
         "mgpt_delta_state_chunked": [P, I, L, I, I, I, P, L, I, I, I, I, I, I, F, P, P, P, L, P, P, I, I, P, P, L, P, L, P],
-        "mgpt_short_conv": [P, I, L, I, P, P, I, P, L, P, P, P, P, I, P, I, L, I, I, I, I, P],
+        "mgpt_short_conv": [P, I, L, I, P, P, I, P, L, P, P, P, P, I, P, I, L, I, I, I, I, I, P],
     }
     for name, argtypes in table.items():
         fn = getattr(lib, name, None)

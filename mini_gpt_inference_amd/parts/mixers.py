@@ -553,7 +553,7 @@ class GatedAttention(Mixer):
             zc = ws.get("gated_attention_conv", n, self.in_rows, ctx.dtype)
             kept = ctx.state_pools[binding.state] if self.conv_taps > 1 else None      # (one tap keeps no inputs)
             kernels.short_conv(z, 0, self.conv_weight, None, kept, ctx.state_slots, ctx.cu_q, ctx.q_req,
-                               ctx.positions, ctx.cu_q.numel() - 1, zc, 0, n)
+                               ctx.positions, ctx.cu_q.numel() - 1, zc, 0, n, single=ctx.decode_only)
             gate_rows, z = z, zc
         else:
             gate_rows = z
@@ -849,7 +849,7 @@ class StateSpaceMixer(Mixer):
         linear(ctx, h, self.in_weight, None, u, n)
         xbc = ws.get("state_space_conv", n, self.conv_width, ctx.dtype)
         kernels.short_conv(u, self.inner, self.conv_weight, self.conv_bias, pool[:, self.state_numel:], ctx.state_slots,
-                           ctx.cu_q, ctx.q_req, ctx.positions, n_req, xbc, 0, n, activation="silu")
+                           ctx.cu_q, ctx.q_req, ctx.positions, n_req, xbc, 0, n, activation="silu", single=ctx.decode_only)
         sums = ws.get("state_space_sums", n, self.inner, torch.float32)
         gn = self.n_group * self.state_dim
         state = pool[:, :self.state_numel]
@@ -957,7 +957,7 @@ class GatedDeltaRule(Mixer):
         linear(ctx, h, self.in_weight, None, z, n)
         qkv = ws.get("delta_conv", n, self.conv_width, ctx.dtype)
         kernels.short_conv(z, 0, self.conv_weight, None, pool[:, self.state_numel:], ctx.state_slots, ctx.cu_q, ctx.q_req,
-                           ctx.positions, n_req, qkv, 0, n, activation="silu")
+                           ctx.positions, n_req, qkv, 0, n, activation="silu", single=ctx.decode_only)
         y = ws.get("delta_out", n, self.v_width, ctx.dtype)
         sizes = (z, self.b_off, self.a_off, self.n_head, self.n_group, self.head_dim, self.value_dim, self.dt_bias,
                  self.a_log, state, ctx.state_slots, ctx.cu_q, n_req, ctx.positions)
@@ -1037,6 +1037,9 @@ class GatedDiagonalState(Mixer):
         views["r_weight"], views["i_weight"] = self.gate_weights[:, :self.block], self.gate_weights[:, self.block:]
         for name, view in views.items():
             setattr(self, name, view)
+        # for the kernels that multiply the gates out themselves (bfloat16): the matrices in their order
+        self.packed_gates = kernels.pack_diagonal_gates(tensors["r_weight"], tensors["i_weight"])
+        self.conv_by_tap = tensors["conv_weight"].t().contiguous()
         self.r_bias_flat, self.i_bias_flat = tensors["r_bias"].reshape(-1).contiguous(), tensors["i_bias"].reshape(-1).contiguous()
         # -decay_scale softplus(lam), once, in double precision
         lam = tensors["lam"].to(torch.float64)
@@ -1056,16 +1059,31 @@ class GatedDiagonalState(Mixer):
         n_req, pool = ctx.cu_q.numel() - 1, ctx.state_pools[binding.index]
         z = ws.get("diagonal_in", n, self.in_rows, ctx.dtype)
         linear(ctx, h, self.in_weight, self.in_bias, z, n)
-        u = ws.get("diagonal_conv", n, C, ctx.dtype)
-        kernels.short_conv(z, 0, self.conv_weight, self.conv_bias, pool[:, C:] if self.conv_taps > 1 else None, ctx.state_slots,
-                           ctx.cu_q, ctx.q_req, ctx.positions, n_req, u, 0, n)
-        gates = ws.get("diagonal_gates", n, 2 * C, ctx.dtype)
-        kernels.heads_linear(u, self.gate_weights, gates, n, fast=not ctx.exact)
-        scratch = None
-        if not ctx.decode_only:
-            floats = kernels.diagonal_scratch_floats(n, n_req, C)
-            scratch = ws.get("diagonal_scratch", floats, 1, torch.float32)
         y = ws.get("diagonal_out", n, C, ctx.dtype)
-        kernels.diagonal_state(u, gates, self.r_bias_flat, self.i_bias_flat, self.decay, self.block, pool[:, :C], ctx.state_slots,
-                               ctx.cu_q, ctx.positions, n_req, n, y, y=z[:, self.y_off:self.y_off + C], scratch=scratch)
+        single = ctx.decode_only
+        kept = pool[:, C:] if self.conv_taps > 1 else None
+        fused = False
+        fusable = self.packed_gates is not None and not ctx.exact and ctx.dtype == torch.bfloat16
+        if fusable and not single:
+            # a step with prompt portions: convolution, gates and recurrence in two kernels
+            scratch = ws.get("diagonal_scratch", kernels.diagonal_fused_scratch_floats(n, C) // C, C, torch.float32)
+            fused = self._fused(ctx, z, pool, n_req, n, y, None, scratch)
+        if not fused:
+            u = ws.get("diagonal_conv", n, C, ctx.dtype)
+            kernels.short_conv(z, 0, self.conv_weight, self.conv_bias, kept, ctx.state_slots, ctx.cu_q, ctx.q_req, ctx.positions,
+                               n_req, u, 0, n, single=single)
+            if fusable and single:
+                fused = self._fused(ctx, z, pool, n_req, n, y, u, None)
+        if not fused:
+            gates = ws.get("diagonal_gates", n, 2 * C, ctx.dtype)
+            kernels.heads_linear(u, self.gate_weights, gates, n, fast=not ctx.exact)
+            scratch = None if single else ws.get("diagonal_chunks", kernels.diagonal_scratch_floats(n, n_req, C), 1, torch.float32)
+            kernels.diagonal_state(u, gates, self.r_bias_flat, self.i_bias_flat, self.decay, self.block, pool[:, :C],
+                                   ctx.state_slots, ctx.cu_q, ctx.positions, n_req, n, y,
+                                   y=z[:, self.y_off:self.y_off + C], scratch=scratch)
         linear_add(ctx, y, self.out_weight, None, x, n)
+
+    def _fused(self, ctx: StepContext, z, pool, n_req: int, n: int, y, u, scratch) -> bool:
+        return kernels.diagonal_state_fused(z, self.y_off, self.conv_by_tap, self.conv_bias, self.packed_gates, self.block,
+                                            self.r_bias_flat, self.i_bias_flat, self.decay, pool, ctx.state_slots, ctx.cu_q, ctx.positions,
+                                            n_req, n, y, u=u, scratch=scratch)
