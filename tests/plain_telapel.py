@@ -225,7 +225,7 @@ def grouped_choice(scores: torch.Tensor, top: int, count: int, keep: int) -> tor
     open_to = scores.masked_fill(~allowed, -math.inf)
     if ROUTER_GAPS is not None:
         # (of logarithms: by how much the logits differ)
-        srt = torch.sort(torch.log(open_to), dim=-1, descending=True).values
+        srt = torch.sort(torch.log(scores).masked_fill(~allowed, -math.inf), dim=-1, descending=True).values
         gap = srt[:, top - 1] - srt[:, top] if top < X else torch.full((T,), math.inf, dtype=DTYPE)
         if keep < count:
             ranks = torch.sort(torch.log(rank), dim=-1, descending=True).values
