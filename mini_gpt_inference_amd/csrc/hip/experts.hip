@@ -643,6 +643,108 @@ extern "C" int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_ro
   return mgpt_last_error();
 }
 
+// The same product for tiles of 16 slots (a decode step), laid out for the matrices' way from memory: a workgroup owns a
+// tile x 16 columns, its four waves take the inner size 32 at a time in turn, EXD loads each on their way at once, and
+// their sums meet in LDS in wave order.  With a unit (kind >= 0) the expert's matrix is its gate's rows over its up
+// rows, a workgroup owns 16 columns of both, and what it stores is the gated unit of the two sums: n_out is then the
+// hidden size.  tile_expert null: one matrix for all rows, of which the first n_rows are used (slot_token null).
+#define EXD 4
+
+template <typename OT, bool GATED>
+__global__ __launch_bounds__(256) void grouped_few_rows_kernel(
+    const bf16_t* __restrict__ A, long lda, const int* __restrict__ a_rows, const bf16_t* __restrict__ W, long w_stride,
+    const int* __restrict__ tile_expert, const int* __restrict__ slot_token, OT* __restrict__ out, long ldo,
+    const int* __restrict__ out_rows, int n_rows, int n_out, int k_dim, int epilogue, int kind, float limit, float sharpness) {
+  constexpr int NJ = GATED ? 2 : 1;
+  __shared__ ex_f32x4_t part[4][NJ][64];
+  const int tile = blockIdx.y;
+  const int e = tile_expert ? tile_expert[tile] : 0;
+  if (e < 0) return;      // (the whole workgroup)
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, li = lane & 15, lg = lane >> 4;
+  const int col0 = blockIdx.x * 16;
+  const int slot = tile * 16 + li;
+  const bool a_ok = slot_token ? slot_token[slot] >= 0 : slot < n_rows;
+  const bf16_t* ap = A + (a_ok ? (long)(a_rows ? a_rows[slot] : slot) : 0L) * lda + lg * 8;
+  const bf16_t* wp = W + (long)e * w_stride + (long)(col0 + li < n_out ? col0 + li : n_out - 1) * k_dim + lg * 8;
+  const long up = (long)n_out * k_dim;
+  const ex_bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  ex_f32x4_t acc[NJ];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) acc[j] = ex_f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int steps = k_dim / 32;      // whole ones
+  int st = wave;
+  for (; st + 4 * (EXD - 1) < steps; st += 4 * EXD) {
+    ex_bf16x8_t wf[NJ][EXD], af[EXD];
+#pragma unroll
+    for (int d = 0; d < EXD; ++d) {
+      const long k = (long)(st + 4 * d) * 32;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) wf[j][d] = *reinterpret_cast<const ex_bf16x8_t*>(wp + j * up + k);
+      af[d] = *reinterpret_cast<const ex_bf16x8_t*>(ap + k);
+    }
+#pragma unroll
+    for (int d = 0; d < EXD; ++d) {
+      const ex_bf16x8_t a = a_ok ? af[d] : zero;
+#pragma unroll
+      for (int j = 0; j < NJ; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[j][d], a, acc[j], 0, 0, 0);
+    }
+  }
+  for (; st * 32 < k_dim; st += 4) {      // what is left, the last step perhaps not whole
+    const long k = (long)st * 32;
+    const bool k_ok = k + lg * 8 < k_dim;
+    const ex_bf16x8_t a = a_ok && k_ok ? *reinterpret_cast<const ex_bf16x8_t*>(ap + k) : zero;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+      const ex_bf16x8_t w = k_ok ? *reinterpret_cast<const ex_bf16x8_t*>(wp + j * up + k) : zero;
+      acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w, a, acc[j], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) part[wave][j][lane] = acc[j];
+  __syncthreads();
+  // a thread a (slot, column): lane (g, slot) of a wave holds columns 4 g .. 4 g + 3
+  const int s = tid >> 4, c = tid & 15, at = (c >> 2) * 16 + s, v = c & 3;
+  const int mine = tile * 16 + s;
+  if (col0 + c >= n_out || !(slot_token ? slot_token[mine] >= 0 : mine < n_rows)) return;
+  float sum[NJ];
+#pragma unroll
+  for (int j = 0; j < NJ; ++j) sum[j] = (part[0][j][at][v] + part[1][j][at][v]) + (part[2][j][at][v] + part[3][j][at][v]);
+  float r = sum[0];
+  if (GATED) r = gated_value<true>(sum[0], sum[NJ - 1], kind, limit, sharpness);
+  else if (epilogue == EX_EPI_RELU2) r = relu_squared(r);
+  out[(long)(out_rows ? out_rows[mine] : mine) * ldo + col0 + c] = from_float<OT>(r);
+}
+
+// bfloat16 operands, bfloat16 or float32 out; kind: a gated unit's number (mgpt_gated_unit), -1: none.  Refuses
+// (MGPT_ERR_BAD_SHAPE) inner sizes that are no multiple of 8 and rows or bases that do not take 16-byte loads.
+extern "C" int mgpt_grouped_few_rows(const void* a, long lda, const int* a_rows, const void* w, long w_stride,
+                                     const int* tile_expert, const int* slot_token, void* out, int out_dtype, long ldo,
+                                     const int* out_rows, int n_tiles, int n_rows, int n_out, int k_dim, int epilogue, int kind,
+                                     float limit, float sharpness, hipStream_t stream) {
+  if (n_tiles == 0 || n_out == 0) return MGPT_OK;
+  if (!a || !w || !out || (tile_expert && !slot_token)) return MGPT_ERR_NULL;
+  if ((epilogue != EX_EPI_NONE && epilogue != EX_EPI_RELU2) || kind < -1 || kind > 3 || (kind >= 0 && epilogue != EX_EPI_NONE))
+    return MGPT_ERR_BAD_SHAPE;
+  if (n_tiles < 0 || n_out < 0 || k_dim <= 0 || lda < k_dim || ldo < n_out || (!slot_token && (n_rows < 0 || n_rows > n_tiles * 16)))
+    return MGPT_ERR_BAD_SHAPE;
+  if ((k_dim & 7) || (lda & 7) || (w_stride & 7) || (((size_t)a | (size_t)w) & 15)) return MGPT_ERR_BAD_SHAPE;
+  if (n_tiles > 65535) return MGPT_ERR_TOO_LARGE;
+  dim3 grid((n_out + 15) / 16, n_tiles), block(256);
+#define GF_LAUNCH(OT, G)                                                                                              \
+  hipLaunchKernelGGL((grouped_few_rows_kernel<OT, G>), grid, block, 0, stream, (const bf16_t*)a, lda, a_rows,         \
+                     (const bf16_t*)w, w_stride, tile_expert, slot_token, (OT*)out, ldo, out_rows, n_rows, n_out,     \
+                     k_dim, epilogue, kind, limit, sharpness)
+  if (out_dtype == MGPT_F32) {
+    if (kind >= 0) GF_LAUNCH(float, true); else GF_LAUNCH(float, false);
+  } else if (out_dtype == MGPT_BF16) {
+    if (kind >= 0) GF_LAUNCH(bf16_t, true); else GF_LAUNCH(bf16_t, false);
+  } else {
+    return MGPT_ERR_BAD_DTYPE;
+  }
+#undef GF_LAUNCH
+  return mgpt_last_error();
+}
+
 __global__ void expert_combine_kernel(const float* __restrict__ pair_out, const int* __restrict__ pair_slot,
                                       const int* __restrict__ q_req, float* __restrict__ y, long total, int width,
                                       int top, float weight, const float* __restrict__ pair_weight,

@@ -174,6 +174,9 @@ int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, const void* 
 int mgpt_grouped_linear_mfma(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int*
     tile_expert, const int* slot_token, void* out, int out_dtype, long ldo, const int* out_rows, int n_tiles,
     int tile_rows, int n_out, int k_dim, int epilogue, hipStream_t stream);
+int mgpt_grouped_few_rows(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int* tile_expert,
+    const int* slot_token, void* out, int out_dtype, long ldo, const int* out_rows, int n_tiles, int n_rows, int n_out,
+    int k_dim, int epilogue, int kind, float limit, float sharpness, hipStream_t stream);
 int mgpt_expert_combine(const float* pair_out, const int* pair_slot, const int* q_req, float* y, int n_rows, int
     width, int top, float weight, const float* pair_weight, const float* extra, const float* extra_gate,
     hipStream_t stream);
@@ -284,6 +287,7 @@ int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_st
   X(mgpt_heads_linear) \
   X(mgpt_heads_linear_mfma) \
   X(mgpt_grouped_linear_mfma) \
+  X(mgpt_grouped_few_rows) \
   X(mgpt_gated_unit) \
   X(mgpt_expert_route) \
   X(mgpt_grouped_linear) \

@@ -1368,6 +1368,13 @@ def grouped_linear(a: torch.Tensor, a_rows: Optional[torch.Tensor], w: torch.Ten
     for t in (a_rows, out_rows):
         if t is not None:
             _need_i32("row index", t, n_slots)
+    if fast and tile == 16 and a.dtype == torch.bfloat16:
+        rc = library.kernels().mgpt_grouped_few_rows(_ptr(a), a.stride(0), _ptr(a_rows), _ptr(w), w.stride(0), _ptr(tile_expert),
+                                                     _ptr(slot_token), _ptr(out), _dtype_code(out), out.stride(0), _ptr(out_rows),
+                                                     n_slots // tile, 0, n_out, k_dim, epilogue, -1, 0.0, 0.0, _stream())
+        if rc != -2:
+            _check(rc, "grouped_few_rows")
+            return
     if fast and tile in (16, 64) and a.dtype == torch.bfloat16:
         # the MFMA kernel; it refuses sizes and alignments that its 16-byte loads do not take
         rc = library.kernels().mgpt_grouped_linear_mfma(_ptr(a), a.stride(0), _ptr(a_rows), _ptr(w), w.stride(0),
@@ -1382,6 +1389,48 @@ def grouped_linear(a: torch.Tensor, a_rows: Optional[torch.Tensor], w: torch.Ten
                                                out.stride(0), _ptr(out_rows), n_slots // tile, tile, n_out, k_dim,
                                                _dtype_code(a), epilogue, _stream())
     _check(rc, "grouped_linear")
+
+
+GATED_FEW_ROWS = 16      # rows that gated_few_rows takes: one tile
+
+
+def gated_few_rows(a: torch.Tensor, w: torch.Tensor, act: torch.Tensor, n_rows: int, hidden: int, a_rows: Optional[torch.Tensor] = None,
+                   tile_expert: Optional[torch.Tensor] = None, slot_token: Optional[torch.Tensor] = None, n_slots: int = 0,
+                   activation: str = "silu", limit: float = 0.0, sharpness: float = 1.0) -> bool:
+    """The product with a gate's and an up matrix, one over the other in w, and the gated unit of the two results
+    (gated_unit's) in one bfloat16 kernel.  Either act[:n_rows] from a[:n_rows] (up to GATED_FEW_ROWS rows) and one w
+    [2 * hidden, width]; or, with tile_expert, slot_token and n_slots in tiles of 16, act[s] from row a_rows[s] (or s) and the
+    tile's expert's matrix of w [experts, 2 * hidden, width].  False, with nothing launched, where it does not apply."""
+    if a.dtype != torch.bfloat16 or w.dtype != torch.bfloat16 or act.dtype != torch.bfloat16 or w.shape[-1] % 8:
+        return False
+    _need(activation in GATE_ACTIVATIONS, f"gated unit: activation {activation!r} is none of {sorted(GATE_ACTIVATIONS)}")
+    _need_cuda(a, w, act, a_rows, tile_expert, slot_token)
+    width = w.shape[-1]
+    _need(w.is_contiguous() and w.dim() == (2 if tile_expert is None else 3) and w.shape[-2] == 2 * hidden,
+          "gated_few_rows: w must be dense, gate rows over up rows")
+    _need(a.dim() == 2 and a.stride(1) == 1 and a.shape[1] >= width and act.dim() == 2 and act.stride(1) == 1 and act.shape[1] >= hidden,
+          "gated_few_rows: rows of the width and of the hidden size")
+    if tile_expert is None:
+        if n_rows > GATED_FEW_ROWS:
+            return False
+        _need(a.shape[0] >= n_rows and act.shape[0] >= n_rows, "gated_few_rows: too few rows")
+        n_tiles, stride = 1, 0
+    else:
+        _need(n_slots % 16 == 0 and act.shape[0] >= n_slots, "gated_few_rows: tiles of 16 slots")
+        n_tiles, stride = n_slots // 16, w.stride(0)
+        _need_i32("tile_expert", tile_expert, n_tiles)
+        _need_i32("slot_token", slot_token, n_slots)
+        if a_rows is not None:
+            _need_i32("a_rows", a_rows, n_slots)
+        else:
+            _need(a.shape[0] >= n_slots, "gated_few_rows: a row per slot")
+    rc = library.kernels().mgpt_grouped_few_rows(_ptr(a), a.stride(0), _ptr(a_rows), _ptr(w), stride, _ptr(tile_expert), _ptr(slot_token),
+                                                 _ptr(act), _dtype_code(act), act.stride(0), None, n_tiles, n_rows, hidden, width, 0,
+                                                 GATE_ACTIVATIONS[activation], float(limit), float(sharpness), _stream())
+    if rc == -2:
+        return False
+    _check(rc, "grouped_few_rows")
+    return True
 
 
 def expert_combine(pair_out: torch.Tensor, y: torch.Tensor, n_rows: int, top: int, weight: float,

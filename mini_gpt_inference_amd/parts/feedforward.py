@@ -107,10 +107,12 @@ def _gated(ctx: StepContext, h, in_weight: torch.Tensor, down_weight: torch.Tens
            hidden: int, **unit) -> None:
     """x += (act(h Wgate^T) * (h Wup^T)) Wdown^T with the gate and up matrices stacked in in_weight; `unit`: the
     activation and its constants, as ops.kernels.gated_unit takes them."""
-    z = ctx.workspace.get("gated_z", n, 2 * hidden, ctx.dtype)
-    linear(ctx, h, in_weight, None, z, n)
     act = ctx.workspace.get("gated_act", n, hidden, ctx.dtype)
-    kernels.gated_unit(z, act, n, hidden, fast=not ctx.exact, **unit)
+    few = not ctx.exact and n <= kernels.GATED_FEW_ROWS and kernels.gated_few_rows(as_tensor(ctx, h), in_weight, act, n, hidden, **unit)
+    if not few:
+        z = ctx.workspace.get("gated_z", n, 2 * hidden, ctx.dtype)
+        linear(ctx, h, in_weight, None, z, n)
+        kernels.gated_unit(z, act, n, hidden, fast=not ctx.exact, **unit)
     linear_add(ctx, act, down_weight, None, x, n)
 
 
@@ -266,17 +268,19 @@ class TableExperts(FeedForward):
         tile_expert = ws.get("expert_tile", slots // tile, 1, torch.int32).view(-1)
         kernels.expert_route(ids, ctx.q_req, table, n, self.n_experts, slot_token, slot_pair, tile_expert, tile)
         act = ws.get("expert_act", slots, self.hidden, ctx.dtype)
-        z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype) if self.gated else act
-        if pair_weight is None:
-            kernels.grouped_linear(hn, slot_token, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast,
-                                   self.epilogue)
-        else:
+        rows, places = hn, slot_token
+        if pair_weight is not None:
             # the weight multiplies the expert's input: every pair's row is made first, scaled, in the experts' order
-            rows = ws.get("expert_rows", slots, self.width, ctx.dtype)
+            rows, places = ws.get("expert_rows", slots, self.width, ctx.dtype), None
             kernels.gather_scale_rows(hn, slot_token, slot_pair, pair_weight, rows, slots)
-            kernels.grouped_linear(rows, None, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast,
-                                   self.epilogue)
-        if self.gated:
+        # few pairs an expert: the unit is made where the gate's and the up product's sums meet
+        done = (self.gated and fast and tile == 16
+                and kernels.gated_few_rows(rows, self.in_weights, act, 0, self.hidden, a_rows=places, tile_expert=tile_expert,
+                                           slot_token=slot_token, n_slots=slots, **self.unit))
+        if not done:
+            z = ws.get("expert_z", slots, 2 * self.hidden, ctx.dtype) if self.gated else act
+            kernels.grouped_linear(rows, places, self.in_weights, tile_expert, slot_token, z, None, slots, tile, fast, self.epilogue)
+        if self.gated and not done:
             kernels.gated_unit(z, act, slots, self.hidden, fast=not ctx.exact, **self.unit)
         pair_out = ws.get("expert_pair_out", n * self.top, self.width, torch.float32)
         kernels.grouped_linear(act, None, self.down_weights, tile_expert, slot_token, pair_out, slot_pair, slots,

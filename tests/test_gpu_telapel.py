@@ -522,6 +522,54 @@ def test_clamped_swish_unit(dtype, n, hidden, limit, sharpness):
         helpers.assert_close(act[:n], want, dtype, f"unit, fast {fast}")
 
 
+UNITS = {"silu": lambda g, u: g * P.sigmoid(g) * u, "relu": lambda g, u: torch.clamp(g, min=0.0) * u,
+         "gelu_tanh": lambda g, u: P.gelu_tanh(g) * u, "clamped_swish": lambda g, u: P.clamped_swish_unit(g, u, 0.9)}
+
+
+@pytest.mark.parametrize("activation", sorted(UNITS))
+@pytest.mark.parametrize("n,width,hidden", [(1, 64, 48), (5, 40, 37), (16, 2048, 1360), (7, 520, 16), (3, 1000, 100)])
+def test_gated_products_of_few_rows_with_their_unit(activation, n, width, hidden):
+    """One matrix pair for all rows, and pairs of four experts in tiles of 16 slots, gathered and in order; inner sizes with
+    and without a rest of less than 32; and the product without a unit, float32 out at places of its own."""
+    g = torch.Generator().manual_seed(n + width)
+    extra = {"limit": 0.9, "sharpness": 1.702} if activation == "clamped_swish" else {}
+    h = _rnd(g, n + 1, width + 8, dtype="bfloat16")
+    w = _rnd(g, 4, 2 * hidden, width, dtype="bfloat16", scale=width ** -0.5)
+    rows = _d(h[:n, :width])
+    want = torch.stack([UNITS[activation](rows @ _d(w[e, :hidden]).T, rows @ _d(w[e, hidden:]).T) for e in range(4)])
+    act = torch.full((n + 1, hidden), 9.0, dtype=torch.bfloat16, device=DEV)
+    assert kernels.gated_few_rows(h.to(DEV), w[2].to(DEV), act, n, hidden, activation=activation, **extra)
+    assert (act[n] == 9.0).all()
+    helpers.assert_close(act[:n], want[2], "bfloat16", "one matrix pair")
+    table = torch.stack([torch.randperm(4, generator=g)[:2] for _ in range(n)]).to(torch.int32)
+    slots = kernels.expert_slots(n, 2, 4, 16)
+    st, sp, te = (torch.zeros(k, dtype=torch.int32, device=DEV) for k in (slots, slots, slots // 16))
+    kernels.expert_route(None, None, table.to(DEV), n, 4, st, sp, te, 16)
+    used = (st >= 0).nonzero().flatten().tolist()
+    ref = torch.stack([want[table[st[s], sp[s] % 2], st[s]] for s in used])
+    ordered = torch.zeros(slots, width, dtype=torch.bfloat16, device=DEV)
+    ordered[used] = h[st[used].cpu().long(), :width].to(DEV)
+    for a, a_rows in ((h.to(DEV), st), (ordered, None)):
+        act = torch.full((slots, hidden), 9.0, dtype=torch.bfloat16, device=DEV)
+        assert kernels.gated_few_rows(a, w.to(DEV), act, 0, hidden, a_rows=a_rows, tile_expert=te, slot_token=st, n_slots=slots,
+                                      activation=activation, **extra)
+        helpers.assert_close(act[used], ref, "bfloat16", "experts")
+        assert (act[[s for s in range(slots) if s not in used]] == 9.0).all()
+    # tiles of 16 without a unit
+    down = _rnd(g, 4, 24, width, dtype="bfloat16", scale=width ** -0.5)
+    out = torch.full((2 * n, 24), 9.0, device=DEV)
+    kernels.grouped_linear(h.to(DEV), st, down.to(DEV), te, st, out, sp, slots, 16, True)
+    ref = torch.stack([rows[t] @ _d(down[table[t, c]]).T for t in range(n) for c in range(2)])
+    helpers.assert_close(out, ref, "bfloat16", "without a unit")
+
+
+def test_gated_products_of_more_rows_are_left_to_other_kernels():
+    h, w = torch.zeros(17, 64, dtype=torch.bfloat16, device=DEV), torch.zeros(32, 64, dtype=torch.bfloat16, device=DEV)
+    act = torch.zeros(17, 16, dtype=torch.bfloat16, device=DEV)
+    assert not kernels.gated_few_rows(h, w, act, 17, 16)
+    assert not kernels.gated_few_rows(h.float(), w.float(), act.float(), 4, 16)
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("width", [40, 1024, 3000, 5000])
 def test_norm_behind_a_sublayer_hands_the_residual_on(dtype, width):
