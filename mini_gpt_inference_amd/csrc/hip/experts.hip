@@ -161,21 +161,112 @@ __device__ __forceinline__ void router_load8(const bf16_t* p, float (&v)[8]) {
   }
 }
 
+struct RouterRule {
+  int n_experts, top, kind;
+  const float* correction;
+  int n_groups, keep, group_best, normalise;
+  float scale;
+};
+
+// One wave's choice among the logits of a token: `key` and `rank` are scratch of n_experts entries each.
+__device__ __forceinline__ void router_choose(const RouterRule& rule, const float* logit, float* key, float* rank, int lane,
+                                              int* __restrict__ chosen, float* __restrict__ weight) {
+  const int n_experts = rule.n_experts;
+  // softmax: the largest logit and the sum over all experts
+  float top_logit = 0.f, inv_total = 1.f;
+  if (rule.kind == 2) {
+    float m = -INFINITY;
+    for (int e = lane; e < n_experts; e += 64) m = fmaxf(m, logit[e]);
+    top_logit = wave_max(m);
+    float total = 0.f;
+    for (int e = lane; e < n_experts; e += 64) total += expf(logit[e] - top_logit);
+    inv_total = 1.0f / wave_sum(total);
+  }
+  auto score_of = [&](float z) {
+    if (rule.kind == 0) return 1.0f / (1.0f + expf(-z));
+    return rule.kind == 1 ? z : expf(z - top_logit) * inv_total;
+  };
+  // (without a correction and groups, and with groups that rank by one expert, the choice goes by the logits, in
+  // whose order the scores come)
+  const bool grouped = rule.n_groups > rule.keep && rule.keep > 0;
+  const bool by_score = rule.correction || (grouped && rule.group_best > 1);
+  for (int e = lane; e < n_experts; e += 64) {
+    const float z = logit[e];
+    key[e] = by_score ? score_of(z) + (rule.correction ? rule.correction[e] : 0.f) : z;
+  }
+  __builtin_amdgcn_wave_barrier();
+  if (grouped) {
+    const int size = n_experts / rule.n_groups;
+    for (int g = lane; g < rule.n_groups; g += 64) {
+      float a = -INFINITY, b = -INFINITY;     // the two largest
+      for (int i = 0; i < size; ++i) {
+        const float v = key[g * size + i];
+        if (v > a) { b = a; a = v; }
+        else if (v > b) b = v;
+      }
+      rank[g] = size > 1 && rule.group_best > 1 ? a + b : a;
+    }
+    __builtin_amdgcn_wave_barrier();
+    // a group stays if fewer than `keep` groups come before it (of equal ranks the lower number first)
+    for (int e = lane; e < n_experts; e += 64) {
+      const int mine = e / size;
+      int before = 0;
+      for (int g = 0; g < rule.n_groups; ++g) before += rank[g] > rank[mine] || (rank[g] == rank[mine] && g < mine);
+      if (before >= rule.keep) key[e] = -INFINITY;
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+  float sum = 0.f;
+  for (int c = 0; c < rule.top; ++c) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < n_experts; e += 64) {
+      const float v = key[e];
+      if (v > best) { best = v; at = e; }      // a lane's experts rise, so the lower number stays at a tie
+    }
+    const float all = wave_max(best);
+    // the lowest number among the lanes that hold the maximum: of one expert a lane the lowest lane
+    int cand = (best == all) ? at : 0x7fffffff;
+    if (n_experts <= 64) {
+      const unsigned long long held = __ballot(cand != 0x7fffffff);
+      cand = held ? __ffsll(held) - 1 : 0x7fffffff;
+    } else {
+      for (int off = 32; off > 0; off >>= 1) {
+        const int other = __shfl_xor(cand, off);
+        cand = other < cand ? other : cand;
+      }
+    }
+    if (cand == 0x7fffffff) cand = 0;          // every score is -inf or NaN
+    const float score = score_of(logit[cand]);
+    sum += score;                                         // (the same in every lane)
+    if (lane == 0) {
+      chosen[c] = cand;
+      weight[c] = score * rule.scale;
+      rank[c] = score;                                    // (the groups' ranks are done with)
+    }
+    if ((cand & 63) == lane) key[cand] = -INFINITY;       // the lane that reads this expert takes it out
+    __builtin_amdgcn_wave_barrier();
+  }
+  if (!rule.normalise) return;
+  const float by = rule.scale / (sum + 1e-20f);
+  if (lane == 0)
+    for (int c = 0; c < rule.top; ++c) weight[c] = rank[c] * by;
+}
+
 // The storage types are the kernel's parameters (a choice made load by load keeps the loads from being in flight
 // together).  VEC: the width is a multiple of 8 and the rows are aligned for loads of eight elements; then thread t
 // takes columns 8 t .. 8 t + 7 of every stretch of 2,048 columns for J experts at a time, whose loads are all in
 // flight together, and the sums meet through the waves in a fixed order.  Otherwise a wave takes an expert at a time.
 template <typename HT, typename WT, bool VEC, int J>     // J: rows of the matrix in flight at a time (VEC)
 __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__ h, long ldh, const WT* __restrict__ w,
-                                                          const int* __restrict__ q_req, int width, int n_experts, int top,
-                                                          int kind, int* __restrict__ chosen, float* __restrict__ weight,
-                                                          const float* __restrict__ correction, int n_groups, int keep,
-                                                          int normalise, float scale, const WT* __restrict__ extra,
-                                                          float* __restrict__ extra_out, int group_best) {
+                                                          const int* __restrict__ q_req, int width, RouterRule rule,
+                                                          int* __restrict__ chosen, float* __restrict__ weight,
+                                                          const WT* __restrict__ extra, float* __restrict__ extra_out) {
   __shared__ float logit[EX_MAX_EXPERTS + 1];    // the extra row's comes last
   __shared__ float key[EX_MAX_EXPERTS];          // what the choice goes by
   __shared__ float rank[EX_MAX_EXPERTS];         // of a group
   __shared__ float part[4][J];
+  const int n_experts = rule.n_experts;
   const int n_rows_w = n_experts + (extra ? 1 : 0);
   const int n = blockIdx.x;
   if (q_req && q_req[n] < 0) return;     // padded token
@@ -217,81 +308,92 @@ __global__ __launch_bounds__(256) void router_topk_kernel(const HT* __restrict__
     __syncthreads();
   }
   if (extra && threadIdx.x == 0) extra_out[n] = 1.0f / (1.0f + expf(-logit[n_experts]));
-  // softmax: the largest logit and the sum over all experts, in every wave by itself (so the same in every thread)
-  float top_logit = 0.f, inv_total = 1.f;
-  if (kind == 2) {
-    float m = -INFINITY;
-    for (int e = lane; e < n_experts; e += 64) m = fmaxf(m, logit[e]);
-    top_logit = wave_max(m);
-    float total = 0.f;
-    for (int e = lane; e < n_experts; e += 64) total += expf(logit[e] - top_logit);
-    inv_total = 1.0f / wave_sum(total);
+  if (wave == 0) router_choose(rule, logit, key, rank, lane, chosen + (long)n * rule.top, weight + (long)n * rule.top);
+}
+
+#define RR_MAX_EXPERTS 64
+#define RR_MAX_ROWS 16
+
+typedef __attribute__((__vector_size__(8 * sizeof(short)))) short ex_bf16x8_t;
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float ex_f32x4_t;
+
+// The router and the experts' slots (expert_route_kernel) of a step of few tokens in bfloat16 in one kernel of one
+// workgroup: the logits of 16 experts at a time as matrix products (products of two bfloat16 numbers are exact in the
+// float32 they are summed in), the inner size dealt out to 16 waves whose sums meet in LDS in wave order; a wave a token's
+// choice; then all threads sort the pairs.
+__global__ __launch_bounds__(1024) void router_route_kernel(const bf16_t* __restrict__ h, long ldh, const bf16_t* __restrict__ w,
+                                                            const int* __restrict__ q_req, int n_rows, int width, RouterRule rule,
+                                                            int* __restrict__ chosen, float* __restrict__ weight,
+                                                            const bf16_t* __restrict__ extra, float* __restrict__ extra_out,
+                                                            int* __restrict__ slot_token, int* __restrict__ slot_pair,
+                                                            int* __restrict__ tile_expert, int n_slots, int n_tiles, int tile_rows) {
+  __shared__ float logit[RR_MAX_ROWS][RR_MAX_EXPERTS + 1], key[RR_MAX_ROWS][RR_MAX_EXPERTS], rank[RR_MAX_ROWS][RR_MAX_EXPERTS];
+  __shared__ int pick[RR_MAX_ROWS * RR_MAX_EXPERTS];
+  __shared__ float times[RR_MAX_ROWS * RR_MAX_EXPERTS];
+  __shared__ int count[RR_MAX_EXPERTS], start[RR_MAX_EXPERTS];
+  __shared__ ex_f32x4_t part[16][64];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n_experts = rule.n_experts, top = rule.top;
+  for (int e = tid; e < n_experts; e += blockDim.x) count[e] = 0;
+  for (int s = tid; s < n_slots; s += blockDim.x) slot_token[s] = -1;
+  for (int t = tid; t < n_tiles; t += blockDim.x) tile_expert[t] = -1;
+  const int n_rows_w = n_experts + (extra ? 1 : 0);
+  const int li = lane & 15, lg = lane >> 4;
+  const ex_bf16x8_t zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  const bf16_t* hp = h + (long)(li < n_rows ? li : 0) * ldh + lg * 8;
+  for (int e0 = 0; e0 < n_rows_w; e0 += 16) {
+    const int e = e0 + li;
+    const bf16_t* wp = (e < n_experts ? w + (long)e * width : (e == n_experts && extra ? extra : w)) + lg * 8;
+    ex_f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k0 = wave * 32; k0 < width; k0 += 16 * 32) {
+      const bool k_ok = k0 + lg * 8 < width;
+      const ex_bf16x8_t hf = k_ok && li < n_rows ? *reinterpret_cast<const ex_bf16x8_t*>(hp + k0) : zero;
+      const ex_bf16x8_t wf = k_ok ? *reinterpret_cast<const ex_bf16x8_t*>(wp + k0) : zero;
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hf, wf, acc, 0, 0, 0);
+    }
+    part[wave][lane] = acc;
+    __syncthreads();
+    if (tid < 256) {
+      const int t = tid >> 4, c = tid & 15, at = (t >> 2) * 16 + c, v = t & 3;
+      float sum = 0.f;
+#pragma unroll
+      for (int i = 0; i < 16; ++i) sum += part[i][at][v];
+      if (e0 + c < n_rows_w) logit[t][e0 + c] = sum;
+    }
+    __syncthreads();
   }
-  auto score_of = [&](float z) {
-    if (kind == 0) return 1.0f / (1.0f + expf(-z));
-    return kind == 1 ? z : expf(z - top_logit) * inv_total;
-  };
-  // (without a correction and groups, and with groups that rank by one expert, the choice goes by the logits, in
-  // whose order the scores come)
-  const bool grouped = n_groups > keep && keep > 0;
-  const bool by_score = correction || (grouped && group_best > 1);
-  for (int e = threadIdx.x; e < n_experts; e += 256) {
-    const float z = logit[e];
-    key[e] = by_score ? score_of(z) + (correction ? correction[e] : 0.f) : z;
+  const bool live = wave < n_rows && (!q_req || q_req[wave] >= 0);
+  if (live) {
+    if (extra && lane == 0) extra_out[wave] = 1.0f / (1.0f + expf(-logit[wave][n_experts]));
+    router_choose(rule, logit[wave], key[wave], rank[wave], lane, pick + wave * top, times + wave * top);
   }
   __syncthreads();
-  if (grouped) {
-    const int size = n_experts / n_groups;
-    for (int g = threadIdx.x; g < n_groups; g += 256) {
-      float a = -INFINITY, b = -INFINITY;     // the two largest
-      for (int i = 0; i < size; ++i) {
-        const float v = key[g * size + i];
-        if (v > a) { b = a; a = v; }
-        else if (v > b) b = v;
-      }
-      rank[g] = size > 1 && group_best > 1 ? a + b : a;
+  const int n_pairs = n_rows * top;
+  auto used = [&](int p) { return !q_req || q_req[p / top] >= 0; };      // not a token of the padding
+  for (int p = tid; p < n_pairs; p += blockDim.x)
+    if (used(p)) {
+      chosen[p] = pick[p];
+      weight[p] = times[p];
+      atomicAdd(&count[pick[p]], 1);
     }
-    __syncthreads();
-    // a group stays if fewer than `keep` groups come before it (of equal ranks the lower number first)
-    for (int e = threadIdx.x; e < n_experts; e += 256) {
-      const int mine = e / size;
-      int before = 0;
-      for (int g = 0; g < n_groups; ++g) before += rank[g] > rank[mine] || (rank[g] == rank[mine] && g < mine);
-      if (before >= keep) key[e] = -INFINITY;
+  __syncthreads();
+  if (tid == 0) {
+    int at = 0;
+    for (int e = 0; e < n_experts; ++e) {
+      start[e] = at;
+      const int tiles = (count[e] + tile_rows - 1) / tile_rows;
+      for (int t = 0; t < tiles; ++t) tile_expert[at / tile_rows + t] = e;
+      at += tiles * tile_rows;
+      count[e] = 0;
     }
-    __syncthreads();
   }
-  if (wave != 0) return;
-  float sum = 0.f;
-  for (int c = 0; c < top; ++c) {
-    float best = -INFINITY;
-    int at = 0x7fffffff;
-    for (int e = lane; e < n_experts; e += 64) {
-      const float v = key[e];
-      if (v > best) { best = v; at = e; }      // a lane's experts rise, so the lower number stays at a tie
+  __syncthreads();
+  for (int p = tid; p < n_pairs; p += blockDim.x)
+    if (used(p)) {
+      const int s = start[pick[p]] + atomicAdd(&count[pick[p]], 1);
+      slot_token[s] = p / top;
+      slot_pair[s] = p;
     }
-    const float all = wave_max(best);
-    int cand = (best == all) ? at : 0x7fffffff;
-    // the lowest number among the lanes that hold the maximum
-    for (int off = 32; off > 0; off >>= 1) {
-      const int other = __shfl_xor(cand, off);
-      cand = other < cand ? other : cand;
-    }
-    if (cand == 0x7fffffff) cand = 0;          // every score is -inf or NaN
-    const float score = score_of(logit[cand]);
-    sum += score;                                         // (the same in every lane)
-    if (lane == 0) {
-      chosen[(long)n * top + c] = cand;
-      weight[(long)n * top + c] = score * scale;
-      rank[c] = score;                                    // (the groups' ranks are done with)
-    }
-    if ((cand & 63) == lane) key[cand] = -INFINITY;       // the lane that reads this expert takes it out
-  }
-  if (!normalise) return;
-  __builtin_amdgcn_wave_barrier();
-  const float by = scale / (sum + 1e-20f);
-  if (lane == 0)
-    for (int c = 0; c < top; ++c) weight[(long)n * top + c] = rank[c] * by;
 }
 
 // h: [n_rows, ldh] rows in `dtype`; w: dense [n_experts, width] in w_dtype; chosen: int32 [n_rows, top]; weight:
@@ -310,18 +412,17 @@ extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* 
   if (n_groups > keep && keep > 0 && (n_experts % n_groups || top > keep * (n_experts / n_groups))) return MGPT_ERR_BAD_SHAPE;
   if (extra && !extra_out) return MGPT_ERR_NULL;
   const size_t h_size = dtype == MGPT_F32 ? 4 : 2, w_size = w_dtype == MGPT_F32 ? 4 : 2;
+  const RouterRule rule = {n_experts, top, kind, correction, n_groups, keep, group_best, normalise, scale};
   const int rows_w = n_experts + (extra ? 1 : 0);
   const bool vec = !(width & 7) && !(((size_t)h | (size_t)(ldh * h_size)) & 15) && !(((size_t)w | (size_t)extra) & 15);
 #define ROUTER_LAUNCH2(HT, WT, JJ)                                                                                            \
   {                                                                                                                      \
     if (vec)                                                                                                             \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, true, JJ>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,      \
-                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
-                         normalise, scale, (const WT*)extra, extra_out, group_best);                                                 \
+                         (const WT*)w, q_req, width, rule, chosen, weight, (const WT*)extra, extra_out);                                                 \
     else                                                                                                                 \
       hipLaunchKernelGGL((router_topk_kernel<HT, WT, false, 8>), dim3(n_rows), dim3(256), 0, stream, (const HT*)h, ldh,     \
-                         (const WT*)w, q_req, width, n_experts, top, kind, chosen, weight, correction, n_groups, keep,   \
-                         normalise, scale, (const WT*)extra, extra_out, group_best);                                                 \
+                         (const WT*)w, q_req, width, rule, chosen, weight, (const WT*)extra, extra_out);                                                 \
   }
   // up to eight rows at a time; a matrix of 9 to 12 (a few experts and the extra row) in one go
 #define ROUTER_LAUNCH(HT, WT)                                                                                            \
@@ -335,6 +436,34 @@ extern "C" int mgpt_router_topk(const void* h, int dtype, long ldh, const void* 
   else ROUTER_LAUNCH(bf16_t, bf16_t)
 #undef ROUTER_LAUNCH
 #undef ROUTER_LAUNCH2
+  return mgpt_last_error();
+}
+
+// mgpt_router_topk and mgpt_expert_route in one launch for steps of up to RR_MAX_ROWS rows and RR_MAX_EXPERTS experts.
+// Refuses (MGPT_ERR_BAD_SHAPE) others, other types than bfloat16, and rows that do not take 16-byte loads.
+extern "C" int mgpt_router_route(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
+                                 int width, int n_experts, int top, int kind, int* chosen, float* weight,
+                                 const float* correction, int n_groups, int keep, int normalise, float scale,
+                                 const void* extra, float* extra_out, int group_best, int* slot_token, int* slot_pair,
+                                 int* tile_expert, int n_slots, int n_tiles, int tile_rows, hipStream_t stream) {
+  if (n_rows == 0) return MGPT_OK;
+  if (!h || !w || !chosen || !weight || !slot_token || !slot_pair || !tile_expert) return MGPT_ERR_NULL;
+  if (extra && !extra_out) return MGPT_ERR_NULL;
+  if (!dtype_ok(dtype) || !dtype_ok(w_dtype)) return MGPT_ERR_BAD_DTYPE;
+  if (n_rows < 0 || n_rows > RR_MAX_ROWS || width <= 0 || n_experts <= 0 || n_experts > RR_MAX_EXPERTS || top <= 0 || top > n_experts ||
+      kind < 0 || kind > 2 || n_groups < 0 || keep < 0 || (group_best != 1 && group_best != 2) ||
+      (tile_rows != 16 && tile_rows != 64 && tile_rows != 256) || n_slots != n_tiles * tile_rows)
+    return MGPT_ERR_BAD_SHAPE;
+  if (n_groups > keep && keep > 0 && (n_experts % n_groups || top > keep * (n_experts / n_groups))) return MGPT_ERR_BAD_SHAPE;
+  const long pairs = (long)n_rows * top;
+  const long worst = pairs + (n_experts < pairs ? n_experts : pairs) * (long)(tile_rows - 1);
+  if ((long)n_slots < worst / tile_rows * tile_rows) return MGPT_ERR_BAD_SHAPE;
+  if (dtype != MGPT_BF16 || w_dtype != MGPT_BF16 || (width & 7) || (ldh & 7) || (((size_t)h | (size_t)w | (size_t)extra) & 15))
+    return MGPT_ERR_BAD_SHAPE;
+  const RouterRule rule = {n_experts, top, kind, correction, n_groups, keep, group_best, normalise, scale};
+  hipLaunchKernelGGL(router_route_kernel, dim3(1), dim3(1024), 0, stream, (const bf16_t*)h, ldh, (const bf16_t*)w, q_req, n_rows,
+                     width, rule, chosen, weight, (const bf16_t*)extra, extra_out, slot_token, slot_pair, tile_expert, n_slots,
+                     n_tiles, tile_rows);
   return mgpt_last_error();
 }
 
@@ -527,8 +656,6 @@ extern "C" int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, c
 // tile x 64 (or 256) columns, a wave 16 (or 64) of the columns for all of the tile's slots: per 32 k one
 // (or four) slices of the expert's matrix (first operand) and four slices of gathered rows (one for a
 // tile of 16 slots: a decode step's few pairs an expert), 16 bytes a lane straight from memory.
-typedef __attribute__((__vector_size__(8 * sizeof(short)))) short ex_bf16x8_t;
-typedef __attribute__((__vector_size__(4 * sizeof(float)))) float ex_f32x4_t;
 
 template <typename OT, int NJ, int NT>     // NT: slices of 16 slots a tile
 __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(

@@ -166,6 +166,10 @@ int mgpt_router_topk(const void* h, int dtype, long ldh, const void* w, int w_dt
     int width, int n_experts, int top, int kind, int* chosen, float* weight, const float* correction, int n_groups,
     int keep, int normalise, float scale, const void* extra, float* extra_out, int group_best,
     hipStream_t stream);
+int mgpt_router_route(const void* h, int dtype, long ldh, const void* w, int w_dtype, const int* q_req, int n_rows,
+    int width, int n_experts, int top, int kind, int* chosen, float* weight, const float* correction, int n_groups,
+    int keep, int normalise, float scale, const void* extra, float* extra_out, int group_best, int* slot_token,
+    int* slot_pair, int* tile_expert, int n_slots, int n_tiles, int tile_rows, hipStream_t stream);
 int mgpt_gather_scale_rows(const void* src, int dtype, long ld, const int* slot_token, const int* slot_pair,
     const float* pair_weight, void* sorted, long lds, int n_slots, int width, hipStream_t stream);
 int mgpt_grouped_linear(const void* a, long lda, const int* a_rows, const void* w, long w_stride, const int*
@@ -303,6 +307,7 @@ int mgpt_linear_mfma_grouped(const void* act, long lda, const void* w, long w_st
   X(mgpt_decay_state) \
   X(mgpt_decay_state_chunked) \
   X(mgpt_router_topk) \
+  X(mgpt_router_route) \
   X(mgpt_gather_scale_rows) \
   X(mgpt_gated_state) \
   X(mgpt_gated_state_chunked) \

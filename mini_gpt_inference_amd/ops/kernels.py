@@ -1478,13 +1478,15 @@ def gather_rows(src: torch.Tensor, slot_token: torch.Tensor, out: torch.Tensor, 
     return True
 
 
+# a step's router and the sorting of its pairs are one workgroup's work up to these numbers (and this many matrix elements)
+ROUTE_MAX_ROWS, ROUTE_MAX_EXPERTS, ROUTE_MAX_WORK = 16, 64, 1 << 17
 ROUTER_SCORES = {"sigmoid": 0, "logit": 1, "softmax": 2}
 
 
 def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen: torch.Tensor, weight: torch.Tensor,
                 q_req: Optional[torch.Tensor] = None, score: str = "sigmoid", correction: Optional[torch.Tensor] = None,
                 groups=None, normalise: bool = False, scale: float = 1.0, extra: Optional[torch.Tensor] = None,
-                extra_out: Optional[torch.Tensor] = None, group_best: int = 2) -> None:
+                extra_out: Optional[torch.Tensor] = None, group_best: int = 2, slots=None) -> bool:
     """chosen[n] = the `top` experts with the largest w[e] . h[n] (float32 sums), best first; weight[n] = their
     scores (sigmoid of the sum, the sum itself, or the sums' softmax over all experts).  w: dense [experts, width]; chosen int32 and weight float32,
     dense [>= n_rows, top].
@@ -1492,7 +1494,11 @@ def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen:
     correction (float32 [experts]) is added to the scores that the choice goes by; groups = (count, keep): only the
     experts of the `keep` groups (of `count` equal groups of neighbours) whose two largest choice scores have the
     largest sums (group_best 1: whose largest choice scores are the largest) can be chosen; normalise: the weights are the chosen scores over (their sum + 1e-20); every weight
-    is multiplied by `scale`.  extra ([width], like w): extra_out[n] = sigmoid(extra . h[n]), float32."""
+    is multiplied by `scale`.  extra ([width], like w): extra_out[n] = sigmoid(extra . h[n]), float32.
+
+    slots = (slot_token, slot_pair, tile_expert, n_slots, tile): the pairs are also sorted into the experts' slots as
+    expert_route does, in the same launch; False, with nothing launched, where that does not apply (many rows or experts,
+    32-bit)."""
     _need_cuda(h, w, chosen, weight, q_req, correction, extra, extra_out)
     _need(score in ROUTER_SCORES, f"router score {score!r} is none of {sorted(ROUTER_SCORES)}")
     _need(w.dim() == 2 and w.is_contiguous() and w.dtype in (torch.float32, torch.bfloat16), "the router's matrix must be dense")
@@ -1516,11 +1522,28 @@ def router_topk(h: torch.Tensor, w: torch.Tensor, n_rows: int, top: int, chosen:
         _need(extra.dtype == w.dtype and extra.is_contiguous() and extra.numel() == width, "extra must be a row like w's")
         _need(extra_out is not None and extra_out.dtype == torch.float32 and extra_out.is_contiguous()
               and extra_out.numel() >= n_rows, "extra_out must be dense float32 of n_rows entries")
-    rc = library.kernels().mgpt_router_topk(_ptr(h), _dtype_code(h), h.stride(0), _ptr(w), _dtype_code(w), _ptr(q_req), n_rows,
-                                            width, n_experts, top, ROUTER_SCORES[score], _ptr(chosen), _ptr(weight),
-                                            _ptr(correction), count, keep, 1 if normalise else 0, float(scale), _ptr(extra),
-                                            _ptr(extra_out), int(group_best), _stream())
+    args = (_ptr(h), _dtype_code(h), h.stride(0), _ptr(w), _dtype_code(w), _ptr(q_req), n_rows, width, n_experts, top,
+            ROUTER_SCORES[score], _ptr(chosen), _ptr(weight), _ptr(correction), count, keep, 1 if normalise else 0, float(scale),
+            _ptr(extra), _ptr(extra_out), int(group_best))
+    if slots is not None:
+        slot_token, slot_pair, tile_expert, n_slots, tile = slots
+        if n_rows > ROUTE_MAX_ROWS or n_experts > ROUTE_MAX_EXPERTS or n_experts * width > ROUTE_MAX_WORK:
+            return False
+        _need_cuda(slot_token, slot_pair, tile_expert)
+        _need(tile in EXPERT_TILES and n_slots % tile == 0 and n_slots >= expert_slots(n_rows, top, n_experts, tile),
+              "router_topk: too few slots for the pairs")
+        _need_i32("slot_token", slot_token, n_slots)
+        _need_i32("slot_pair", slot_pair, n_slots)
+        _need_i32("tile_expert", tile_expert, n_slots // tile)
+        rc = library.kernels().mgpt_router_route(*args, _ptr(slot_token), _ptr(slot_pair), _ptr(tile_expert), n_slots, n_slots // tile,
+                                                 tile, _stream())
+        if rc == -2:
+            return False
+        _check(rc, "router_route")
+        return True
+    rc = library.kernels().mgpt_router_topk(*args, _stream())
     _check(rc, "router_topk")
+    return True
 
 
 def gather_scale_rows(src: torch.Tensor, slot_token: torch.Tensor, slot_pair: torch.Tensor, pair_weight: torch.Tensor,

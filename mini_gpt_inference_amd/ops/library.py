@@ -181,6 +181,7 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         "mgpt_grouped_few_rows": [P, L, P, P, L, P, P, P, I, L, P, I, I, I, I, I, I, F, F, P],
         "mgpt_expert_combine": [P, P, P, P, I, I, I, F, P, P, P, P],
         "mgpt_router_topk": [P, I, L, P, I, P, I, I, I, I, I, P, P, P, I, I, I, F, P, P, I, P],
+        "mgpt_router_route": [P, I, L, P, I, P, I, I, I, I, I, P, P, P, I, I, I, F, P, P, I, P, P, P, I, I, I, P],
         "mgpt_gather_scale_rows": [P, I, L, P, P, P, P, L, I, I, P],
         # a state with a decay made from the token, short convolutions
         "mgpt_gated_state": [P, I, L, I, I, I, I, I, I, I, P, I, L, I, I, F, F, P, P, P, P, L, P, P, I, P, P, L, P],

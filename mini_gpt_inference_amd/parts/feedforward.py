@@ -249,24 +249,18 @@ class TableExperts(FeedForward):
         self._experts_add(ctx, hn, x, ctx.n_rows, ctx.token_ids, self.table, None, 1.0 / self.top)
 
     def _experts_add(self, ctx: StepContext, hn: torch.Tensor, x: torch.Tensor, n: int, ids, table: torch.Tensor,
-                     pair_weight, combine_weight: float, out_weight=None, shared_gate=None) -> None:
+                     pair_weight, combine_weight: float, out_weight=None, shared_gate=None, routed=None) -> None:
         """x += combine_weight * sum over token n's experts (row ids[n] of the table, or row n without ids) of
         v expert(w h), w = pair_weight[n][choice] and v = out_weight[n][choice] (None: 1), plus the shared expert
-        (times shared_gate[n])."""
+        (times shared_gate[n]).  routed: the slots of _slots, if the pairs are sorted already."""
         ws = ctx.workspace
         fast = not ctx.exact and ctx.dtype == torch.bfloat16
-        if fast and n * self.top >= self.TILED_FROM_PAIRS and self.width % 16 == 0 and self.hidden % 16 == 0 \
+        if routed is None and fast and n * self.top >= self.TILED_FROM_PAIRS and self.width % 16 == 0 and self.hidden % 16 == 0 \
                 and self._forward_tiled(ctx, hn, x, n, ids, table, pair_weight, combine_weight, out_weight, shared_gate):
             return
-        # tiles of 64 slots for the MFMA kernel of few rows, of 16 for the general one, and for the MFMA kernel too
-        # where an expert gets 16 pairs at most on average (a decode step): a tile's empty slots are loaded and
-        # multiplied like the used ones
-        tile = 64 if fast and n * self.top > 16 * self.n_experts else 16
-        slots = kernels.expert_slots(n, self.top, self.n_experts, tile)
-        slot_token = ws.get("expert_slot_token", slots, 1, torch.int32).view(-1)
-        slot_pair = ws.get("expert_slot_pair", slots, 1, torch.int32).view(-1)
-        tile_expert = ws.get("expert_tile", slots // tile, 1, torch.int32).view(-1)
-        kernels.expert_route(ids, ctx.q_req, table, n, self.n_experts, slot_token, slot_pair, tile_expert, tile)
+        slot_token, slot_pair, tile_expert, slots, tile = routed or self._slots(ctx, n)
+        if routed is None:
+            kernels.expert_route(ids, ctx.q_req, table, n, self.n_experts, slot_token, slot_pair, tile_expert, tile)
         act = ws.get("expert_act", slots, self.hidden, ctx.dtype)
         rows, places = hn, slot_token
         if pair_weight is not None:
@@ -288,6 +282,18 @@ class TableExperts(FeedForward):
         extra = self._shared_add(ctx, hn, x, n)
         kernels.expert_combine(pair_out, x, n, self.top, combine_weight, q_req=ctx.q_req, pair_weight=out_weight,
                                extra=extra, extra_gate=shared_gate)
+
+    def _slots(self, ctx: StepContext, n: int):
+        """Buffers for the sorted pairs of n tokens: (slot_token, slot_pair, tile_expert, slots, slots a tile)."""
+        # tiles of 64 slots for the MFMA kernel of few rows, of 16 for the general one, and for the MFMA kernels too
+        # where an expert gets 16 pairs at most on average (a decode step): a tile's empty slots are loaded and
+        # multiplied like the used ones
+        ws = ctx.workspace
+        fast = not ctx.exact and ctx.dtype == torch.bfloat16
+        tile = 64 if fast and n * self.top > 16 * self.n_experts else 16
+        slots = kernels.expert_slots(n, self.top, self.n_experts, tile)
+        return (ws.get("expert_slot_token", slots, 1, torch.int32).view(-1), ws.get("expert_slot_pair", slots, 1, torch.int32).view(-1),
+                ws.get("expert_tile", slots // tile, 1, torch.int32).view(-1), slots, tile)
 
     def _shared_add(self, ctx: StepContext, hn: torch.Tensor, x: torch.Tensor, n: int):
         """The shared expert: added into x (returns None), or, if a number per token multiplies it, as rows of its own
@@ -429,9 +435,16 @@ class RoutedExperts(TableExperts):
         chosen = ws.get("router_chosen", n, self.top, torch.int32)
         weight = ws.get("router_weight", n, self.top, torch.float32)
         gate = ws.get("router_shared_gate", n, 1, torch.float32).view(-1) if self.gates_shared else None
-        kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, q_req=ctx.q_req, score=self.score,
-                            correction=self.correction, groups=self.groups, normalise=self.normalise, scale=self.scale,
-                            extra=self.shared_gate_weight, extra_out=gate, group_best=self.group_best)
+        rule = dict(q_req=ctx.q_req, score=self.score, correction=self.correction, groups=self.groups, normalise=self.normalise,
+                    scale=self.scale, extra=self.shared_gate_weight, extra_out=gate, group_best=self.group_best)
+        # few tokens: the same launch sorts the pairs
+        routed = None
+        if n <= kernels.ROUTE_MAX_ROWS and n * self.top < self.TILED_FROM_PAIRS:
+            routed = self._slots(ctx, n)
+            if not kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, slots=routed, **rule):
+                routed = None
+        if routed is None:
+            kernels.router_topk(hn, self.router_weight, n, self.top, chosen, weight, **rule)
         weight = weight.view(-1)
         self._experts_add(ctx, hn, x, n, None, chosen, None if self.weighs_output else weight, 1.0,
-                          out_weight=weight if self.weighs_output else None, shared_gate=gate)
+                          out_weight=weight if self.weighs_output else None, shared_gate=gate, routed=routed)

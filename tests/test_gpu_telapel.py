@@ -482,6 +482,44 @@ def test_router_with_softmax_scores_and_groups_by_their_best(dtype, n, width, ex
         helpers.assert_close(weight[:n].cpu()[firm], ref[firm], "float32", f"weights, normalise {normalise}")
 
 
+@pytest.mark.parametrize("dtype", ["bfloat16"])
+@pytest.mark.parametrize("n,width,experts,top,tile", [(1, 64, 4, 2, 16), (8, 2048, 8, 2, 16), (16, 264, 64, 5, 16), (5, 40, 12, 3, 64), (3, 24, 1, 1, 16)])
+def test_router_that_sorts_its_pairs_in_the_same_launch(dtype, n, width, experts, top, tile):
+    """Choice and weights are the separate kernels' (with softmax, sigmoid scores with a correction, a shared expert's
+    number), every pair has a slot in a tile of its expert, and a token of the padding has none."""
+    g = torch.Generator().manual_seed(n + experts)
+    h, w = _rnd(g, n, width, dtype=dtype).to(DEV), _rnd(g, experts, width, dtype=dtype, scale=2.0 * width ** -0.5).to(DEV)
+    extra, correction = _rnd(g, 1, width, dtype=dtype).to(DEV), _rnd(g, experts).to(DEV)
+    q_req = _i32([-1 if i == n // 2 and n > 1 else i for i in range(n)])
+    live = [i for i in range(n) if not (i == n // 2 and n > 1)]
+    slots = kernels.expert_slots(n, top, experts, tile)
+    for rule in (dict(score="softmax", normalise=True, group_best=1, groups=(experts, experts)),
+                 dict(score="sigmoid", correction=correction, normalise=True, scale=1.5),
+                 dict(score="softmax", group_best=1, groups=(2, 1)) if experts % 2 == 0 and top <= experts // 2 else dict(score="logit")):
+        outs = []
+        for sort in (False, True):
+            chosen, weight = torch.full((n, top), -7, dtype=torch.int32, device=DEV), torch.full((n, top), -7.0, device=DEV)
+            gate = torch.full((n,), -7.0, device=DEV)
+            st, sp, te = (torch.full((k,), -9, dtype=torch.int32, device=DEV) for k in (slots, slots, slots // tile))
+            assert kernels.router_topk(h, w, n, top, chosen, weight, q_req=q_req, extra=extra, extra_out=gate,
+                                       slots=(st, sp, te, slots, tile) if sort else None, **rule)
+            outs.append((chosen, weight, gate))
+        assert torch.equal(outs[0][0], outs[1][0])
+        for a, b in zip(outs[0][1:], outs[1][1:]):
+            helpers.assert_close(a, b, "float32", str(rule))
+        st, sp, te = st.tolist(), sp.tolist(), te.tolist()
+        used = [s for s in range(slots) if st[s] >= 0]
+        assert sorted(sp[s] for s in used) == [i * top + c for i in live for c in range(top)]
+        for s in used:
+            assert st[s] == sp[s] // top and te[s // tile] == int(outs[1][0][st[s], sp[s] % top])
+        assert all(te[t] == -1 for t in range(slots // tile) if all(st[s] < 0 for s in range(t * tile, (t + 1) * tile)))
+    assert not kernels.router_topk(h.float(), w.float(), n, top, chosen, weight, slots=(*(torch.zeros(k, dtype=torch.int32, device=DEV) for k in
+                                                                                         (slots, slots, slots // tile)), slots, tile))
+    assert not kernels.router_topk(h.repeat(17, 1), w, 17, top, torch.zeros(17, top, dtype=torch.int32, device=DEV), torch.zeros(17, top, device=DEV),
+                                   slots=(torch.zeros(17 * top * tile, dtype=torch.int32, device=DEV),) * 2
+                                   + (torch.zeros(17 * top, dtype=torch.int32, device=DEV), 17 * top * tile, tile))
+
+
 def test_a_group_by_its_best_and_by_its_two_best_differ():
     """Group 0 has the best expert and nothing else, groups 1 and 2 two good ones each."""
     logits = torch.tensor([[3.0, -9.0, 2.5, 2.4, 2.45, 2.3]])
@@ -558,7 +596,7 @@ def test_gated_products_of_few_rows_with_their_unit(activation, n, width, hidden
     # tiles of 16 without a unit
     down = _rnd(g, 4, 24, width, dtype="bfloat16", scale=width ** -0.5)
     out = torch.full((2 * n, 24), 9.0, device=DEV)
-    kernels.grouped_linear(h.to(DEV), st, down.to(DEV), te, st, out, sp, slots, 16, True)
+    kernels.grouped_linear(h.to(DEV)[:, :width], st, down.to(DEV), te, st, out, sp, slots, 16, True)
     ref = torch.stack([rows[t] @ _d(down[table[t, c]]).T for t in range(n) for c in range(2)])
     helpers.assert_close(out, ref, "bfloat16", "without a unit")
 
