@@ -54,14 +54,15 @@ extern "C" int mgpt_rms_norm_store(const void* src, int dtype, long ld, const fl
 // `interleaved` (2i, 2i + 1), by the angle position * freq[i], cosine and sine both times rot_mag, in 32-bit.  One
 // workgroup a token.  Without a pool (a layer that reads another layer's latents, or queries that are projected later)
 // only the queries are rotated; with n_head 0 there are no queries to rotate.  With `cq_out` the cq_rank columns of z
-// at cq_off are RMS-normed with cq_gain into its rows: the latent that the queries are made from.
+// at cq_off are RMS-normed with cq_gain into its rows: the latent that the queries are made from.  With `turns` the token's
+// cosines and sines, [rot_dim / 2] each, are left in its rows for a later kernel.
 #define LP_MAX_HALF 256
 template <typename T>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(
     T* __restrict__ z, long ldz, int q_off, int n_head, int head_dim, int rot_dim, int c_off, int rank,
     const float* __restrict__ gain, float eps, const int* __restrict__ positions, const float* __restrict__ freq,
     float rot_mag, T* __restrict__ pool, int row_width, const int* __restrict__ slot_mapping, int n_tokens, int interleaved,
-    int cq_off, int cq_rank, const float* __restrict__ cq_gain, T* __restrict__ cq_out, long ld_cq) {
+    int cq_off, int cq_rank, const float* __restrict__ cq_gain, T* __restrict__ cq_out, long ld_cq, float* __restrict__ turns) {
   __shared__ float cos_s[LP_MAX_HALF], sin_s[LP_MAX_HALF];
   __shared__ float red_s[8];
   const int n = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -71,6 +72,10 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     const float a = p * freq[i];
     cos_s[i] = cosf(a) * rot_mag;
     sin_s[i] = sinf(a) * rot_mag;
+    if (turns) {
+      turns[(long)n * rot_dim + i] = cos_s[i];
+      turns[(long)n * rot_dim + half + i] = sin_s[i];
+    }
   }
   T* row = z + (long)n * ldz;
   const int slot = pool ? slot_mapping[n] : -1;
@@ -120,13 +125,13 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
 }
 
 // z: the step's projected rows (queries at q_off, n_head heads of head_dim + rot_dim; the latent's rank + rot_dim
-// columns at c_off; the cq_rank columns of the queries' latent at cq_off); pool: the latent pages with rows of
+// columns at c_off; the cq_rank columns of the queries' latent at cq_off); turns: dense float32 rows of rot_dim, or null; pool: the latent pages with rows of
 // row_width >= rank + rot_dim values, or null; cq_out: rows of ld_cq >= cq_rank values, or null.
 extern "C" int mgpt_latent_prepare(void* z, int dtype, long ldz, int q_off, int n_head, int head_dim, int rot_dim,
                                    int c_off, int rank, const float* gain, float eps, const int* positions,
                                    const float* freq, float rot_mag, void* pool, int row_width,
                                    const int* slot_mapping, int n_tokens, int interleaved, int cq_off, int cq_rank,
-                                   const float* cq_gain, void* cq_out, long ld_cq, hipStream_t stream) {
+                                   const float* cq_gain, void* cq_out, long ld_cq, float* turns, hipStream_t stream) {
   if (n_tokens == 0) return MGPT_OK;
   if (!z || !positions || !freq || (pool && (!gain || !slot_mapping)) || (cq_out && !cq_gain)) return MGPT_ERR_NULL;
   if (n_tokens < 0 || n_head < 0 || head_dim < 0 || rot_dim <= 0 || (rot_dim & 1) || rot_dim / 2 > LP_MAX_HALF ||
@@ -137,11 +142,11 @@ extern "C" int mgpt_latent_prepare(void* z, int dtype, long ldz, int q_off, int 
   if (dtype == MGPT_F32)
     hipLaunchKernelGGL(latent_prepare_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, (float*)z, ldz, q_off, n_head,
                        head_dim, rot_dim, c_off, rank, gain, eps, positions, freq, rot_mag, (float*)pool, row_width,
-                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (float*)cq_out, ld_cq);
+                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (float*)cq_out, ld_cq, turns);
   else if (dtype == MGPT_BF16)
     hipLaunchKernelGGL(latent_prepare_kernel<bf16_t>, dim3(n_tokens), dim3(256), 0, stream, (bf16_t*)z, ldz, q_off, n_head,
                        head_dim, rot_dim, c_off, rank, gain, eps, positions, freq, rot_mag, (bf16_t*)pool, row_width,
-                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (bf16_t*)cq_out, ld_cq);
+                       slot_mapping, n_tokens, interleaved, cq_off, cq_rank, cq_gain, (bf16_t*)cq_out, ld_cq, turns);
   else
     return MGPT_ERR_BAD_DTYPE;
   return mgpt_last_error();
@@ -221,10 +226,12 @@ extern "C" int mgpt_heads_linear(const void* a, long lda, const void* w, void* o
 typedef __attribute__((__vector_size__(8 * sizeof(short)))) short hl_bf16x8_t;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float hl_f32x4_t;
 
-template <int NJ>
+// With TURN the inner channels from rot_from on are a rotated part whose rotation is made here: neighbouring channels
+// (2i, 2i + 1) of it are pairs, turned by the row's cosines and sines ([rot_dim / 2] each in a row of `turns`).
+template <int NJ, bool TURN>
 __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(
     const bf16_t* __restrict__ A, long lda, const bf16_t* __restrict__ W, bf16_t* __restrict__ out, long ldo,
-    const bf16_t* __restrict__ gate, long ldg, int n_rows, int n_out, int k_dim) {
+    const bf16_t* __restrict__ gate, long ldg, int n_rows, int n_out, int k_dim, const float* __restrict__ turns, int rot_from) {
   // a wave owns 64 rows x NJ * 16 columns of one head: the rows are read once for all those columns
   const int head = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int row0 = (blockIdx.y * 4 + wave) * 64, col0 = blockIdx.x * (NJ * 16);
@@ -261,6 +268,22 @@ __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(
 #pragma unroll
     for (int t = 0; t < 4; ++t)
       af[t] = (a_ok[t] && k_ok) ? *reinterpret_cast<const hl_bf16x8_t*>(arow[t] + k) : zero;
+    if (TURN && k_ok && k >= rot_from) {
+      const int rot = k_dim - rot_from;
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        if (!a_ok[t]) continue;
+        const float* cs = turns + (long)(row0 + 16 * t + li) * rot + (k - rot_from) / 2;
+        const float4 co = *reinterpret_cast<const float4*>(cs), si = *reinterpret_cast<const float4*>(cs + rot / 2);
+        const float c4[4] = {co.x, co.y, co.z, co.w}, s4[4] = {si.x, si.y, si.z, si.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float u = bf16_to_float((bf16_t)af[t][2 * i]), w = bf16_to_float((bf16_t)af[t][2 * i + 1]);
+          af[t][2 * i] = (short)float_to_bf16(u * c4[i] - w * s4[i]);
+          af[t][2 * i + 1] = (short)float_to_bf16(w * c4[i] + u * s4[i]);
+        }
+      }
+    }
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
 #pragma unroll
@@ -291,15 +314,20 @@ __global__ __launch_bounds__(256) void heads_linear_mfma_kernel(
   }
 }
 
-// bfloat16 only.  Refuses (MGPT_ERR_BAD_SHAPE) inner sizes that are no multiple of 8, outputs
+// bfloat16 only.  turns: float32 rows of k_dim - rot_from values (cosines, then sines), or null.  Refuses
+// (MGPT_ERR_BAD_SHAPE) inner sizes (and rotated parts) that are no multiple of 8, outputs
 // that are no multiple of 4 and rows or bases that are not aligned for 16-byte loads and 8-byte
 // stores; the caller then takes mgpt_heads_linear.
 extern "C" int mgpt_heads_linear_mfma(const void* a, long lda, const void* w, void* out, long ldo, const void* gate,
-                                      long ldg, int n_rows, int n_head, int n_out, int k_dim, hipStream_t stream) {
+                                      long ldg, int n_rows, int n_head, int n_out, int k_dim, const float* turns,
+                                      int rot_from, hipStream_t stream) {
   if (n_rows == 0) return MGPT_OK;
   if (!a || !w || !out) return MGPT_ERR_NULL;
   if (n_rows < 0 || n_head <= 0 || n_out <= 0 || k_dim <= 0 || lda < (long)n_head * k_dim ||
       ldo < (long)n_head * n_out || (gate && ldg < (long)n_head * n_out))
+    return MGPT_ERR_BAD_SHAPE;
+  // (eight inner channels at a time are plain or rotated; four cosines at a time are one load)
+  if (turns && (rot_from < 0 || rot_from >= k_dim || (rot_from & 7) || ((k_dim - rot_from) & 7) || (((size_t)turns) & 15)))
     return MGPT_ERR_BAD_SHAPE;
   if ((k_dim & 7) || (n_out & 3) || (lda & 7) || (ldo & 3) || (gate && (ldg & 3)) || (((size_t)a | (size_t)w) & 15) ||
       (((size_t)out | (size_t)gate) & 7))
@@ -312,13 +340,19 @@ extern "C" int mgpt_heads_linear_mfma(const void* a, long lda, const void* w, vo
                     (long)((n_rows + 63) / 64) * ((n_out + nj * 16 - 1) / (nj * 16)) * n_head < 1024))
     nj >>= 1;
   dim3 grid((n_out + nj * 16 - 1) / (nj * 16), (n_rows + 255) / 256, n_head), block(256);
-#define HM_LAUNCH(NJ)                                                                                        \
-  hipLaunchKernelGGL(heads_linear_mfma_kernel<NJ>, grid, block, 0, stream, (const bf16_t*)a, lda,            \
-                     (const bf16_t*)w, (bf16_t*)out, ldo, (const bf16_t*)gate, ldg, n_rows, n_out, k_dim)
+#define HM_LAUNCH2(NJ, T)                                                                                    \
+  hipLaunchKernelGGL((heads_linear_mfma_kernel<NJ, T>), grid, block, 0, stream, (const bf16_t*)a, lda,       \
+                     (const bf16_t*)w, (bf16_t*)out, ldo, (const bf16_t*)gate, ldg, n_rows, n_out, k_dim, turns, rot_from)
+#define HM_LAUNCH(NJ)                             \
+  do {                                            \
+    if (turns) HM_LAUNCH2(NJ, true);              \
+    else HM_LAUNCH2(NJ, false);                   \
+  } while (0)
   if (nj == 1) HM_LAUNCH(1);
   else if (nj == 2) HM_LAUNCH(2);
   else if (nj == 4) HM_LAUNCH(4);
   else HM_LAUNCH(8);
 #undef HM_LAUNCH
+#undef HM_LAUNCH2
   return mgpt_last_error();
 }

@@ -138,11 +138,11 @@ int mgpt_rms_norm_store(const void* src, int dtype, long ld, const float* gain, 
 int mgpt_latent_prepare(void* z, int dtype, long ldz, int q_off, int n_head, int head_dim, int rot_dim, int c_off,
     int rank, const float* gain, float eps, const int* positions, const float* freq, float rot_mag, void* pool,
     int row_width, const int* slot_mapping, int n_tokens, int interleaved, int cq_off, int cq_rank, const float* cq_gain,
-    void* cq_out, long ld_cq, hipStream_t stream);
+    void* cq_out, long ld_cq, float* turns, hipStream_t stream);
 int mgpt_heads_linear(const void* a, long lda, const void* w, void* out, long ldo, const void* gate, long ldg,
     int n_rows, int n_head, int n_out, int k_dim, int dtype, int fast, hipStream_t stream);
 int mgpt_heads_linear_mfma(const void* a, long lda, const void* w, void* out, long ldo, const void* gate, long ldg,
-    int n_rows, int n_head, int n_out, int k_dim, hipStream_t stream);
+    int n_rows, int n_head, int n_out, int k_dim, const float* turns, int rot_from, hipStream_t stream);
 // token_shift.hip
 int mgpt_parallel_norm(float* x, float* y, float mult, const float* gain, float offset, float eps, void* h, void* hs,
     int dtype, const float* shift, float* state, long ld_state, const int* state_slots, const int* q_req,

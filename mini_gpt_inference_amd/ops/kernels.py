@@ -1147,14 +1147,18 @@ def latent_prepare(z: torch.Tensor, q_off: int, n_head: int, head_dim: int, rot_
                    freq: torch.Tensor, n_tokens: int, rot_magnitude: float = 1.0, c_off: int = 0, rank: int = 0,
                    gain: Optional[torch.Tensor] = None, eps: float = 0.0, pool: Optional[torch.Tensor] = None,
                    slot_mapping: Optional[torch.Tensor] = None, interleaved: bool = False, cq_off: int = 0,
-                   cq_gain: Optional[torch.Tensor] = None, cq_out: Optional[torch.Tensor] = None) -> None:
+                   cq_gain: Optional[torch.Tensor] = None, cq_out: Optional[torch.Tensor] = None,
+                   turns: Optional[torch.Tensor] = None) -> None:
     """Latent attention with a rotated part: the last rot_dim channels of every query head (heads of head_dim +
     rot_dim channels at q_off of z's rows) are rotated in place by the token's position; with `pool` (latent pages
     whose rows hold at least rank + rot_dim values) the token's row becomes [rms_norm(z[c_off : c_off + rank]) * gain |
     the next rot_dim columns of z, rotated | zeros].  freq: float32 [rot_dim / 2]; interleaved: the pairs are (2i, 2i + 1)
     instead of (i, i + rot_dim / 2).  n_head may be 0 (the queries are not in z).  cq_out (rows of as many columns as
-    cq_gain has): rms_norm(z[cq_off ..]) * cq_gain, the latent that queries are made from."""
-    _need_cuda(z, positions, freq, gain, pool, slot_mapping, cq_gain, cq_out)
+    cq_gain has): rms_norm(z[cq_off ..]) * cq_gain, the latent that queries are made from.  turns (float32 rows of
+    rot_dim): the tokens' cosines and sines, for heads_linear."""
+    _need_cuda(z, positions, freq, gain, pool, slot_mapping, cq_gain, cq_out, turns)
+    _need(turns is None or (turns.dtype == torch.float32 and turns.dim() == 2 and turns.is_contiguous() and turns.shape[1] == rot_dim
+                            and turns.shape[0] >= n_tokens), "latent_prepare: turns must be dense float32 rows of rot_dim")
     _rows_2d("latent_prepare z", z, n_tokens)
     _need(freq.dtype == torch.float32 and freq.is_contiguous() and freq.numel() * 2 == rot_dim, "latent_prepare: float32 frequencies [rot_dim / 2]")
     _need_i32("positions", positions, n_tokens)
@@ -1179,7 +1183,7 @@ def latent_prepare(z: torch.Tensor, q_off: int, n_head: int, head_dim: int, rot_
         _ptr(z), _dtype_code(z), z.stride(0), int(q_off), n_head, head_dim, rot_dim, int(c_off), int(rank), _ptr(gain),
         float(eps), _ptr(positions), _ptr(freq), float(rot_magnitude), _ptr(pool), row_width, _ptr(slot_mapping), n_tokens,
         int(interleaved), int(cq_off), cq_rank, _ptr(cq_gain), _ptr(cq_out), cq_out.stride(0) if cq_out is not None else 0,
-        _stream())
+        _ptr(turns), _stream())
     _check(rc, "latent_prepare")
 
 
@@ -1262,10 +1266,13 @@ def xielu(z: torch.Tensor, out: torch.Tensor, coef: torch.Tensor, n_rows: int, h
 
 
 def heads_linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, n_rows: int,
-                 gate: Optional[torch.Tensor] = None, fast: bool = False) -> None:
+                 gate: Optional[torch.Tensor] = None, fast: bool = False, turns: Optional[torch.Tensor] = None) -> bool:
     """out[n][h] = a[n][h] @ w[h].T for every head h, optionally times sigmoid(gate[n][h]).
-    w: [heads, n_out, k_dim]; a: [>=n_rows, >=heads * k_dim]; out, gate: [>=n_rows, >=heads * n_out]."""
-    _need_cuda(a, w, out, gate)
+    w: [heads, n_out, k_dim]; a: [>=n_rows, >=heads * k_dim]; out, gate: [>=n_rows, >=heads * n_out].
+
+    turns (float32 rows, latent_prepare's): the last channels of every head of a, as many as a row of turns has, are
+    rotated first (neighbours as pairs, in registers).  False, with nothing launched, where no kernel does that."""
+    _need_cuda(a, w, out, gate, turns)
     _need(w.dim() == 3 and w.is_contiguous(), "the heads' matrices must be dense [heads, out, in]")
     n_head, n_out, k_dim = w.shape
     _need(a.dtype == w.dtype == out.dtype and (gate is None or gate.dtype == a.dtype), "operands must share a dtype")
@@ -1275,17 +1282,26 @@ def heads_linear(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, n_rows: in
         _need(t is None or (t.dim() == 2 and t.stride(1) == 1 and t.shape[1] >= n_head * n_out and t.shape[0] >= n_rows),
               f"{name} must be [>=n_rows, >=heads * out] with unit inner stride")
     ldg = 0 if gate is None else gate.stride(0)
+    rot = 0
+    if turns is not None:
+        _need(turns.dtype == torch.float32 and turns.is_contiguous() and turns.dim() == 2 and turns.shape[0] >= n_rows,
+              "heads_linear: turns must be dense float32 rows")
+        rot = turns.shape[1]
     if fast and a.dtype == torch.bfloat16:
         # the MFMA kernel; it refuses sizes and alignments that its 16-byte loads do not take
         rc = library.kernels().mgpt_heads_linear_mfma(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0),
-                                                      _ptr(gate), ldg, n_rows, n_head, n_out, k_dim, _stream())
+                                                      _ptr(gate), ldg, n_rows, n_head, n_out, k_dim, _ptr(turns), k_dim - rot,
+                                                      _stream())
         if rc != -2:
             _check(rc, "heads_linear_mfma")
-            return
+            return True
+    if turns is not None:
+        return False
     rc = library.kernels().mgpt_heads_linear(_ptr(a), a.stride(0), _ptr(w), _ptr(out), out.stride(0), _ptr(gate),
                                              0 if gate is None else gate.stride(0), n_rows, n_head, n_out, k_dim,
                                              _dtype_code(a), int(fast), _stream())
     _check(rc, "heads_linear")
+    return True
 
 
 # ---------------------------------------------------------------- gated feed-forwards and experts

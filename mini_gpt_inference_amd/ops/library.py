@@ -157,13 +157,13 @@ def _declare_optional(lib: ctypes.CDLL) -> None:
         # latent attention
         "mgpt_rms_norm_store": [P, I, L, P, F, P, P, I, I, P],
         "mgpt_heads_linear": [P, L, P, P, L, P, L, I, I, I, I, I, I, P],
-        "mgpt_latent_prepare": [P, I, L, I, I, I, I, I, I, P, F, P, P, F, P, I, P, I, I, I, I, P, P, L, P],
+        "mgpt_latent_prepare": [P, I, L, I, I, I, I, I, I, P, F, P, P, F, P, I, P, I, I, I, I, P, P, L, P, P],
         # a layer whose sublayers read one norm, the mixer through a token shift; the xIELU activation
         "mgpt_parallel_norm": [P, P, F, P, F, F, P, P, I, P, P, L, P, P, P, I, I, P],
         "mgpt_token_shift": [P, P, I, P, P, L, P, P, P, P, I, I, P],
         "mgpt_token_shift_keep": [P, I, P, L, P, P, I, I, P],
         "mgpt_xielu": [P, L, P, L, I, P, I, I, I, P],
-        "mgpt_heads_linear_mfma": [P, L, P, P, L, P, L, I, I, I, I, P],
+        "mgpt_heads_linear_mfma": [P, L, P, P, L, P, L, I, I, I, I, P, I, P],
         # gated feed-forwards and experts
         "mgpt_gated_unit": [P, L, P, L, I, I, I, I, I, F, F, P],
         # root-mean-square norms, rotation and the rest in front of attention, decaying state

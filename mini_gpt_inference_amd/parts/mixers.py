@@ -296,19 +296,23 @@ class LatentAttention(Mixer):
             rot = (self.rot_dim, ctx.positions, self.rotation.frequencies(z.device), n, getattr(self.rotation, "magnitude", 1.0))
             pairs = getattr(self.rotation, "interleaved", False)
             cq = ws.get("latent_cq", n, self.q_rank, ctx.dtype) if self.q_rank else None
+            # queries that are made later are turned inside the product that folds them, if its kernel can
+            turns = ws.get("latent_turns", n, self.rot_dim, torch.float32) if self.q_rank and pairs and fast else None
             kernels.latent_prepare(z, 0, 0 if self.q_rank else self.n_head, self.head_dim, *rot,
                                    c_off=split, rank=self.rank, gain=self.dkv_norm if self.makes_latent else None,
                                    eps=self.eps, pool=pool if self.makes_latent else None,
                                    slot_mapping=group.slot_mapping if self.makes_latent else None, interleaved=pairs,
-                                   cq_gain=self.dq_norm if self.q_rank else None, cq_out=cq)
+                                   cq_gain=self.dq_norm if self.q_rank else None, cq_out=cq, turns=turns)
             if self.q_rank:
                 q = ws.get("latent_queries", n, self.q_width, ctx.dtype)
                 linear(ctx, cq, self.q_weight, None, q, n)
-                kernels.latent_prepare(q, 0, self.n_head, self.head_dim, *rot, interleaved=pairs)
         elif self.makes_latent:
             kernels.rms_norm_store(z[:, split:], self.dkv_norm, self.eps, pool, group.slot_mapping, n)
         q_lat = ws.get("latent_q", n, self.n_head * self.row, ctx.dtype)
-        kernels.heads_linear(q, self.uk_folded, q_lat, n, fast=fast)
+        if not (self.rot_dim and turns is not None and kernels.heads_linear(q, self.uk_folded, q_lat, n, fast=True, turns=turns)):
+            if self.rot_dim and self.q_rank:
+                kernels.latent_prepare(q, 0, self.n_head, self.head_dim, *rot, interleaved=pairs)
+            kernels.heads_linear(q, self.uk_folded, q_lat, n, fast=fast)
         o_lat = ws.get("latent_o", n, self.n_head * self.row, ctx.dtype)
         gate = z[:, q_cols:split] if self.has_gate else None
         attention_ops.paged_attention(ctx, q_lat, o_lat, pool, pool, group, self.n_head, self.scale, self.window,

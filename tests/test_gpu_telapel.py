@@ -455,6 +455,28 @@ def test_latents_of_keys_and_of_queries_with_interleaved_pairs(dtype, n, H, D, R
     helpers.assert_close(qd[:, 2:], want.reshape(n, -1), dtype, "queries")
 
 
+@pytest.mark.parametrize("n,H,D,R2,row", [(1, 2, 16, 8, 64), (8, 16, 96, 32, 128), (70, 3, 8, 16, 32), (300, 4, 40, 64, 128)])
+def test_folding_product_turns_the_queries_rotated_part(n, H, D, R2, row):
+    g = torch.Generator().manual_seed(n)
+    base = 30.0
+    q, w = _rnd(g, n, H * (D + R2) + 8, dtype="bfloat16"), _rnd(g, H, row, D + R2, dtype="bfloat16", scale=(D + R2) ** -0.5)
+    freq = torch.tensor([base ** (-2.0 * i / R2) for i in range(R2 // 2)], dtype=torch.float64).float().to(DEV)
+    turns = torch.full((n, R2), 9.0, device=DEV)
+    kernels.latent_prepare(q.to(DEV), 0, 0, D, R2, _i32(list(range(n))), freq, n, turns=turns, interleaved=True)
+    a = torch.arange(n, dtype=P.DTYPE)[:, None] * _d(freq.cpu())
+    helpers.assert_close(turns, torch.cat([torch.cos(a), torch.sin(a)], dim=1), "float32", "cosines and sines")
+    out = torch.full((n, H * row), 9.0, dtype=torch.bfloat16, device=DEV)
+    assert kernels.heads_linear(q.to(DEV), w.to(DEV), out, n, fast=True, turns=turns)
+    heads = _d(q[:, :H * (D + R2)]).view(n, H, D + R2)
+    heads = torch.cat([heads[..., :D], P.rotate_pairs(heads[..., D:], base)], dim=-1)
+    want = torch.einsum("nhi,hoi->nho", heads, _d(w)).reshape(n, H * row)
+    helpers.assert_close(out, want, "bfloat16", "folded queries")
+    # parts that are not eight channels at a time are left to others
+    odd = torch.zeros(n, 6, device=DEV)
+    assert not kernels.heads_linear(q.to(DEV), w[:, :, :D + R2].contiguous().to(DEV), out, n, fast=True, turns=odd)
+    assert not kernels.heads_linear(q.float().to(DEV), w.float().to(DEV), out.float(), n, turns=turns)
+
+
 # ---------------------------------------------------------------- the router, the unit, the norm behind a sublayer
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("n,width,experts,top,groups", [(9, 40, 6, 2, (3, 2)), (70, 264, 12, 3, (4, 1)), (5, 2048, 8, 2, (8, 5)), (4, 24, 3, 3, (1, 1)),
