@@ -59,22 +59,12 @@ def _find(tool: str, extra_dirs: tuple[str, ...] = ()) -> str:
 
 
 def _run(cmd: list[str], what: str) -> None:
-    """Runs one compiler command, printing a line now and then while it works."""
-    done = threading.Event()
-
-    def ticker() -> None:
-        start = time.time()
-        while not done.wait(10.0):
-            _say(f"still compiling {what} ({time.time() - start:.0f} s)")
-
-    t = threading.Thread(target=ticker, daemon=True)
-    t.start()
-    try:
-        proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    finally:
-        done.set()
+    """Runs one compiler command and says when it is done."""
+    start = time.time()
+    proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
     if proc.returncode != 0:
         raise BuildError(f"compiling {what} failed:\n{' '.join(cmd)}\n{proc.stdout}")
+    _say(f"compiled {what} ({time.time() - start:.0f} s)")
 
 
 def _writable_target(path: str) -> str:
