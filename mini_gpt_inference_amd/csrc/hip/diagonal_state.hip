@@ -1,12 +1,12 @@
 // A linear recurrence with a float32 state of one number per channel, whose decay and input gate come from the token:
 //
-//   r = sigmoid(gr + r_bias), i = sigmoid(gi + i_bias), log a = decay[c] * r, a = exp(log a)
-//   S_t = a S_(t-1) + sqrt(1 - a^2) i u_t;   out_t = S_t * gelu_tanh(y_t)      (without y: S_t)
+//   a = exp(decay[c] * sigmoid(gr + r_bias)),   i = sigmoid(gi + i_bias)
+//   S <- a S + i u sqrt(1 - a^2);   out = S * gelu_tanh(y)      (without y: S)
 //
 // decay[c] <= 0 is a number per channel.  The two gates' logits lie block by block in the rows of g: for the channels of
 // block b (`block` of them) gr at columns 2 b block .., gi at (2 b + 1) block ...  S is zero before a request's first
 // token and comes from, and goes back to, the request's slot of a pool; from the loaded numbers on everything is float32.
-// sqrt(1 - a^2) is taken as sqrt(-expm1(2 log a)), which is exact where a is nearly 1.
+// That root is taken as sqrt(-expm1(2 log a)), which is exact where a is nearly 1.
 #include "common.h"
 #include "dtype_io.h"
 #include "launchers.h"

@@ -17,13 +17,13 @@ What the design fixes, and is therefore set here and handed to the parts as para
   times the distance taken off; a window of `mask.size` positions; a sink of score 0;
 - feed-forward `moe`: `router.experts` experts with the clamped swish unit (sharpness 1.702, `expert.limit`), softmax
   scores, the `router.top` best of the `router.groups.keep` groups (of `router.groups.count`) with the best experts,
-  weights the chosen scores divided by their sum, on the experts' outputs; a shared expert (`shared.ff`, `shared.limit`);
-- a layer with `weights_of: j` runs layer j's parts once more with a cache or state of its own.
+  weights the chosen scores divided by their sum, on the experts' outputs; beside them a shared one (`shared.ff`, `shared.limit`);
+- a layer with `weights_of: j` runs layer j's parts once more; its cache or state is separate.
 
 Tensor names: `embed`, `l<i>.norm1|norm2`, `l<i>.mix.{y,y.b,x,x.b,conv,conv.b,ra,ra.b,ri,ri.b,lam,o}` (rglru),
 `l<i>.mix.{dq,dq.norm,uq,dkv,dkv.norm,uk,uv,o}` (latent_attention), `l<i>.mix.{q,k,q.b,k.b,q.conv,k.conv,q.norm,k.norm,o}`
-(attention), `l<i>.mlp.router`, `l<i>.mlp.e<j>.{gate,up,down}`, `l<i>.mlp.shared.{gate,up,down}`, `final.norm`; linear
-weights are stored [out, in].
+(attention), `l<i>.mlp.router`, `l<i>.mlp.e<j>.{gate,up,down}`, `l<i>.mlp.shared.{gate,up,down}`, `final.norm`; matrices
+are [out, in].
 """
 
 from __future__ import annotations

@@ -2059,7 +2059,7 @@ def diagonal_state(u: torch.Tensor, gates: torch.Tensor, r_bias: torch.Tensor, i
                    n_req: int, n_tokens: int, out: torch.Tensor, y: Optional[torch.Tensor] = None,
                    scratch: Optional[torch.Tensor] = None) -> None:
     """Over time inside each request, channel by channel: log a = decay * sigmoid(gr + r_bias),
-    S_t = a S_(t-1) + sqrt(1 - a^2) sigmoid(gi + i_bias) u_t, out_t = S_t * gelu_tanh(y_t) (without y: S_t).  The logits of
+    S <- a S + sigmoid(gi + i_bias) u sqrt(1 - a^2), out = S * gelu_tanh(y) (without y: S).  The logits of
     block b (`block` channels) are the columns 2 b block .. of `gates`, first gr, then gi.  S is zero before position 0 and
     lives in the requests' slots of `state` (float32 rows, a view of a pool's columns will do).  r_bias, i_bias, decay
     (<= 0): float32 [channels].  scratch (float32, diagonal_scratch_floats): the tokens of a request in chunks side by

@@ -991,7 +991,7 @@ class GatedDiagonalState(Mixer):
     y = gelu_tanh(h Wy^T + by) and u = conv(h Wx^T + bx) (+ bias), both [C], the convolution causal over time, channel by
     channel (`conv_weight` [C, J], the last tap on the current token, zeros before the sequence's start).  The channels come
     in B equal blocks, each with square matrices of its own: r = sigmoid(Wr_b u_b + br), i = sigmoid(Wi_b u_b + bi);
-    log a = -`decay_scale` r softplus(lam), S_t = a S_(t-1) + sqrt(1 - a^2) i u_t, S zero before the first token;
+    log a = -`decay_scale` r softplus(lam), S <- a S + i u sqrt(1 - a^2), S zero before the first token;
     out = (S * y) Wo^T, added into the residual.  Kept per request: S and the convolution's last J - 1 inputs.  The two
     gates (from their products' sums on), the decay and the recurrence are float32 up to S * y."""
 

@@ -76,7 +76,7 @@ def clamped_swish_unit(gate: torch.Tensor, up: torch.Tensor, limit: float) -> to
 
 # ---------------------------------------------------------------- short convolution
 def short_conv(u: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """u [T, C], w [C, J]: y_t = sum_j w[:, j] u_(t - J + 1 + j) (+ bias), with zeros before the first token: the
+    """u [T, C], w [C, J]: y[t] = w[:, 0] u[t - J + 1] + ... + w[:, J - 1] u[t] (+ bias), with zeros before the first token: the
     last column of w multiplies the current token."""
     T, J = u.shape[0], w.shape[1]
     u, w = _r(u), _r(w)
@@ -99,7 +99,7 @@ def block_product(u: torch.Tensor, w: torch.Tensor, bias: torch.Tensor) -> torch
 
 
 def gated_recurrence(u: torch.Tensor, r: torch.Tensor, i: torch.Tensor, lam: torch.Tensor) -> torch.Tensor:
-    """log a = -8 r softplus(lam); S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t, S zero before the first token.
+    """a = exp(-8 r softplus(lam)); S <- a S + i u sqrt(1 - a^2), S zero before the first token.
     All of [T, C]; returns every S_t."""
     log_a = -8.0 * r * softplus(lam)
     a = torch.exp(log_a)
@@ -216,7 +216,7 @@ ROUTER_GAPS: Optional[list] = None
 
 def grouped_choice(scores: torch.Tensor, top: int, count: int, keep: int) -> torch.Tensor:
     """scores [T, X] -> the numbers [T, top] of the experts each token uses: those with the largest scores among the
-    experts of the `keep` best of `count` equal groups of neighbours, a group's rank its largest score."""
+    experts of the `keep` best of `count` runs of equal length, a run's rank its largest score."""
     T, X = scores.shape
     size = X // count
     rank = scores.view(T, count, size).max(dim=-1).values                           # [T, count]
